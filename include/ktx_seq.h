@@ -24,7 +24,7 @@ typedef void* ktx_stream_t; /* hipStream_t */
 #endif
 
 enum { KTX_SEQ_F32 = 0, KTX_SEQ_BF16 = 1 };
-enum { KTX_ACT_NONE = 0, KTX_ACT_GELU_TANH = 1 };
+enum { KTX_ACT_NONE = 0, KTX_ACT_GELU_TANH = 1, KTX_ACT_RELU_SQ = 2 /* relu(z)^2 */, KTX_ACT_SOFT_CAP = 3 /* act_arg tanh(z / act_arg) */ };
 
 /* x[t] = embed[tokens[t]] + s(pos[t]),  s(p)[2i] = sin(p * inv_freq[i]),  s(p)[2i+1] = cos(p * inv_freq[i]).
  * inv_freq: fp64 [(width + 1) / 2]; the angle and its sine are evaluated in fp64 and rounded once.  x: fp32 [T][width].
@@ -43,6 +43,9 @@ int ktx_dense_gemv_glu(int M, int F, int K, const void* d_A, int a_dtype, int64_
  * ksplit > 1 splits K over ksplit workgroups per tile that add into a ZEROED fp32 Y with atomics (small M; act must be NONE). */
 int ktx_dense_gemm(int M, int N, int K, const void* d_A, int a_dtype, int64_t lda, const void* d_W, int w_dtype, void* d_Y,
                    int y_dtype, int64_t ldy, int act, int ksplit, ktx_stream_t stream);
+/* the same with an activation that takes a number (ktx_dense_gemm: 0) */
+int ktx_dense_gemm_act(int M, int N, int K, const void* d_A, int a_dtype, int64_t lda, const void* d_W, int w_dtype, void* d_Y,
+                       int y_dtype, int64_t ldy, int act, float act_arg, int ksplit, ktx_stream_t stream);
 
 typedef struct ktx_sigattn_config {
   int32_t heads, kv_heads, dim;   /* query heads, key heads (heads % kv_heads == 0), per-head size of q, k and v (v = k) */
@@ -85,6 +88,8 @@ int ktx_sigattn_prefill(const ktx_sigattn_config* cfg, int B, int T, int max_q_l
 
 /* y = gelu_tanh(y) in place, n elements of `dtype` (the activation behind a GEMM that has no epilogue for it). */
 int ktx_gelu_tanh(size_t n, void* d_y, int dtype, ktx_stream_t stream);
+/* the same for any KTX_ACT_*: y = act(y) in place */
+int ktx_act_rows(size_t n, void* d_y, int dtype, int act, float act_arg, ktx_stream_t stream);
 
 typedef struct ktx_mlstm_config {
   int32_t heads, dim, vdim;       /* per head: q, k of size dim, v of size vdim; state S [dim][vdim], n [dim], m */

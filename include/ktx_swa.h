@@ -90,6 +90,7 @@ typedef struct ktx_swa_config {
   int32_t page_size, cache_dtype;     /* caches [rows][kv_heads][dim] and [rows][kv_heads][vdim] of KTX_SEQ_* */
   int32_t keep_first;                 /* with a window: the first keep_first positions of a sequence stay visible to every later one */
   int32_t bias_span;                  /* rows - 1 of the distance-bias table the attention calls take (distances beyond it read its last row) */
+  float softcap;                      /* > 0: the score becomes softcap tanh(score / softcap) (before a distance bias joins it); 0: off */
 } ktx_swa_config;
 
 /* Per token: rotate and norm q (times scale) -> q_out fp32 [T][heads][dim]; rotate and norm k, turn v -> cache rows cache_loc[t];
@@ -100,22 +101,25 @@ int ktx_swa_prep(const ktx_swa_config* cfg, int T, const float* d_proj, int64_t 
                  const double* d_inv_freq, const double* d_v_inv_freq, const int32_t* d_pos, const int32_t* d_cache_loc, void* d_kcache,
                  void* d_vcache, float* d_q_out, float* d_vcs, ktx_stream_t stream);
 
-/* The prep of the un-rotated form whose projections pass a short causal convolution over time: with u = proj[t] + bias (q | k | v, C =
+/* The prep of the form whose projections pass a short causal convolution over time: with u = proj[t] + bias (q | k | v, C =
  * heads dim + kv_heads (dim + vdim) channels at column 0 of fp32 rows of stride ldp; bias fp32 [C] or NULL),
  *   y[t][c] = sum_{j < taps} conv_w[c][j] u[t - taps + 1 + j][c]      (conv_w fp32 [C][taps], the last column multiplies the current token;
  *             inputs before a request's first NEW token come from its slot of conv_state fp32 [slots][taps - 1][C] when pos0 > 0 and are
  *             zero otherwise; taps <= 1: y = u, times conv_w when given)
  *   q = y_q / sqrt(mean(y_q^2) + eps) * q_norm_w * scale over ALL heads dim entries at once (q_norm_w fp32 [heads dim] or NULL: no norm),
  *   k likewise with k_norm_w over kv_heads dim entries; q -> q_out fp32 [T][heads][dim], k and v = y_v -> cache rows cache_loc[t].
+ * With rot_dims > 0 (no norms then): the first rot_dims entries of every q and k head turn with the token's position pos0[b] + i in pairs
+ * (2i, 2i + 1) behind the convolution, angles as in ktx_swa_prep (d_inv_freq fp64 [rot_dims / 2]).
  * Then (second launch) conv_state[slot[b]] = the last taps - 1 inputs u of request b; with max_q_len == 1 (no request brings more than
- * one token), 2 .. 4 taps and channel counts that are multiples of 4 the state moves on in the first launch.  cfg: rot_dims = 0,
- * rot_values = 0; taps <= 16. */
+ * one token), 2 .. 4 taps and channel counts that are multiples of 4 the state moves on in the first launch.  cfg: rot_values = 0;
+ * taps <= 16. */
 int ktx_swa_conv_prep(const ktx_swa_config* cfg, int B, int T, int max_q_len, int taps, const float* d_proj, int64_t ldp, const float* d_bias,
                       const float* d_conv_w, const float* d_q_norm_w, const float* d_k_norm_w, const int32_t* d_q_indptr,
                       const int32_t* d_pos0, const int32_t* d_slot, const int32_t* d_tok_req, float* d_conv_state,
-                      const int32_t* d_cache_loc, void* d_kcache, void* d_vcache, float* d_q_out, ktx_stream_t stream);
+                      const double* d_inv_freq, const int32_t* d_cache_loc, void* d_kcache, void* d_vcache, float* d_q_out,
+                      ktx_stream_t stream);
 
-/* out[t][h] = turn_back(sum_j p_j v_j), p = softmax over {q[t][h] . k_j + dist_bias[min(i - j, bias_span)][h] : j visible to t at
+/* out[t][h] = turn_back(sum_j p_j v_j), p = softmax over {cap(q[t][h] . k_j) + dist_bias[min(i - j, bias_span)][h] : j visible to t at
  * position i: j <= i and (i - j < window or j < keep_first)} and, with sink (fp32 [heads]), one more score sink[h] that has no value.
  * dist_bias: fp32 [bias_span + 1][heads] or NULL (not scaled: scale is folded into q).  Vector-ALU form, any sizes and either cache type: one token x the query heads of one key head x
  * one key range per workgroup; nsplit key ranges leave partial sums in scratch fp32 [nsplit][T][heads][vdim + 2], merged afterwards.

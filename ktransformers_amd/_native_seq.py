@@ -44,6 +44,10 @@ def _load() -> C.CDLL:
     lib.ktx_embed_sinpos.argtypes = [C.c_int, C.c_int, C.c_int, C.c_void_p, C.c_void_p, C.c_void_p, C.c_int, C.c_void_p, C.c_void_p, C.c_void_p]
     lib.ktx_dense_gemm.argtypes = [C.c_int, C.c_int, C.c_int, C.c_void_p, C.c_int, C.c_int64, C.c_void_p, C.c_int, C.c_void_p, C.c_int,
                                    C.c_int64, C.c_int, C.c_int, C.c_void_p]
+    if hasattr(lib, "ktx_act_rows"):
+        lib.ktx_dense_gemm_act.argtypes = [C.c_int, C.c_int, C.c_int, C.c_void_p, C.c_int, C.c_int64, C.c_void_p, C.c_int, C.c_void_p, C.c_int,
+                                           C.c_int64, C.c_int, C.c_float, C.c_int, C.c_void_p]
+        lib.ktx_act_rows.argtypes = [C.c_size_t, C.c_void_p, C.c_int, C.c_int, C.c_float, C.c_void_p]
     if hasattr(lib, "ktx_dense_gemv_glu"):
         lib.ktx_dense_gemv_glu.argtypes = [C.c_int, C.c_int, C.c_int, C.c_void_p, C.c_int, C.c_int64, C.c_void_p, C.c_void_p, C.c_int, C.c_int64,
                                            C.c_float, C.c_float, C.c_float, C.c_void_p]
@@ -76,7 +80,7 @@ def _stream_ptr(device) -> int:
 
 
 SEQ_DTYPE = {torch.float32: 0, torch.bfloat16: 1}
-ACT = {None: 0, "none": 0, "gelu_tanh": 1}
+ACT = {None: 0, "none": 0, "gelu_tanh": 1, "relu_sq": 2, "soft_cap": 3}
 
 
 def _seq_dev(t: torch.Tensor, dtype, what: str) -> torch.Tensor:
@@ -114,9 +118,9 @@ def embed_rows(tokens: torch.Tensor, embed: torch.Tensor, out: torch.Tensor | No
 
 
 def dense_gemm(a: torch.Tensor, w: torch.Tensor, out_dtype=torch.float32, act: str | None = None, out: torch.Tensor | None = None,
-               ksplit: int = 1) -> torch.Tensor:
+               ksplit: int = 1, act_arg: float = 0.0) -> torch.Tensor:
     """a [M, K] (fp32 | bf16, unit inner stride) x w [N, K]^T (contiguous bf16 | fp32: its type is the product's) -> [M, N] of
-    out_dtype (ktx_dense_gemm: any shape)."""
+    out_dtype (ktx_dense_gemm_act: any shape).  act: "gelu_tanh", "relu_sq" (relu(z)^2) or "soft_cap" (act_arg tanh(z / act_arg))."""
     if a.dim() != 2 or w.dim() != 2 or a.shape[1] != w.shape[1] or a.stride(1) != 1 or not w.is_contiguous() or not a.is_cuda \
             or a.device != w.device or a.dtype not in SEQ_DTYPE or w.dtype not in SEQ_DTYPE:
         raise KtxError(f"dense_gemm: {a.dtype} {tuple(a.shape)} x {w.dtype} {tuple(w.shape)}^T does not fit")
@@ -128,15 +132,22 @@ def dense_gemm(a: torch.Tensor, w: torch.Tensor, out_dtype=torch.float32, act: s
         a16 = a if a.dtype == torch.bfloat16 else a.to(torch.bfloat16)
         y = _library_gemm()(a16 if a16.stride(0) % 8 == 0 else a16.contiguous(), w, out_f32=out_dtype == torch.float32)
         if ACT[act]:
-            check(lib.ktx_gelu_tanh(y.numel(), y.data_ptr(), SEQ_DTYPE[y.dtype], _stream_ptr(y.device)))
+            act_rows(y, act, act_arg)
         return y
     if out is None:
         out = (torch.zeros if ksplit > 1 else torch.empty)((M, N), dtype=out_dtype, device=a.device)
     elif out.dtype != out_dtype or tuple(out.shape) != (M, N) or out.stride(1) != 1:
         raise KtxError("dense_gemm: out does not fit")
-    check(lib.ktx_dense_gemm(M, N, K, a.data_ptr(), SEQ_DTYPE[a.dtype], a.stride(0), w.data_ptr(), SEQ_DTYPE[w.dtype], out.data_ptr(),
-                             SEQ_DTYPE[out_dtype], out.stride(0), ACT[act], int(ksplit), _stream_ptr(a.device)))
+    check(lib.ktx_dense_gemm_act(M, N, K, a.data_ptr(), SEQ_DTYPE[a.dtype], a.stride(0), w.data_ptr(), SEQ_DTYPE[w.dtype], out.data_ptr(),
+                                 SEQ_DTYPE[out_dtype], out.stride(0), ACT[act], float(act_arg), int(ksplit), _stream_ptr(a.device)))
     return out
+
+
+def act_rows(y: torch.Tensor, act: str, act_arg: float = 0.0) -> torch.Tensor:
+    """y = act(y) in place over a contiguous fp32 | bf16 tensor (ktx_act_rows)."""
+    _seq_dev(y, None, "act_rows")
+    check(lib.ktx_act_rows(y.numel(), y.data_ptr(), SEQ_DTYPE[y.dtype], ACT[act], float(act_arg), _stream_ptr(y.device)))
+    return y
 
 
 GEMV_GLU_MAX_M = 16
@@ -175,9 +186,7 @@ def dense_gemm_skinny(a: torch.Tensor, w: torch.Tensor, act: str | None = None) 
     if ks == 1:
         return dense_gemm(a, w, act=act)
     y = dense_gemm(a, w, ksplit=ks)
-    if ACT[act]:
-        check(lib.ktx_gelu_tanh(y.numel(), y.data_ptr(), SEQ_DTYPE[y.dtype], _stream_ptr(y.device)))
-    return y
+    return act_rows(y, act) if ACT[act] else y
 
 
 LIBRARY_GEMM_MIN_M = 64

@@ -23,7 +23,7 @@ class _ResidArgs(C.Structure):       # include/ktx_swa.h: ktx_resid_args
 class _SwaConfig(C.Structure):       # include/ktx_swa.h: ktx_swa_config
     _fields_ = [("heads", _I32), ("kv_heads", _I32), ("dim", _I32), ("vdim", _I32), ("rot_dims", _I32), ("rot_values", _I32),
                 ("qk_norm", _I32), ("eps", _F), ("scale", _F), ("window", _I32), ("page_size", _I32), ("cache_dtype", _I32),
-                ("keep_first", _I32), ("bias_span", _I32)]
+                ("keep_first", _I32), ("bias_span", _I32), ("softcap", _F)]
 
 
 class _SsmConfig(C.Structure):       # include/ktx_swa.h: ktx_ssm_config
@@ -36,7 +36,7 @@ lib.ktx_resid_norm.argtypes = [_I, _I, _P, C.POINTER(_ResidArgs), _P]
 lib.ktx_input_conv.argtypes = [_I, _I, _I, _I, _P, _P, _P, _P, _P, _P, _P, _I, _P]
 lib.ktx_rows_mul_lookup.argtypes = [_I, _I, _P, _L, _P, _I, _L, _I, _P, _P, _I, _P]
 lib.ktx_swa_prep.argtypes = [C.POINTER(_SwaConfig), _I, _P, _L, _I, _I, _I, _P, _P, _P, _P, _P, _P, _P, _P, _P]
-lib.ktx_swa_conv_prep.argtypes = [C.POINTER(_SwaConfig), _I, _I, _I, _I, _P, _L] + [_P] * 14
+lib.ktx_swa_conv_prep.argtypes = [C.POINTER(_SwaConfig), _I, _I, _I, _I, _P, _L] + [_P] * 15
 lib.ktx_swa_forward.argtypes = [C.POINTER(_SwaConfig), _I, _P, _P, _P, _P, _P, _P, _P, _P, _P, _P, _I, _P, _P, _I, _P]
 lib.ktx_swa_mfma_eligible.argtypes = [C.POINTER(_SwaConfig)]
 lib.ktx_swa_mfma.argtypes = [C.POINTER(_SwaConfig), _I, _I, _I, _P, _P, _P, _P, _P, _P, _P, _P, _P, _P, _I, _P, _P, _I, _P]
@@ -171,18 +171,20 @@ def rows_mul_lookup(a: torch.Tensor, table: torch.Tensor, col0: int, tokens: tor
 
 
 def swa_config(heads: int, kv_heads: int, dim: int, vdim: int, rot_dims: int, rot_values: bool, qk_norm: bool, eps: float, scale: float,
-               window: int, page_size: int, cache_dtype, keep_first: int = 0, bias_span: int = 0) -> _SwaConfig:
+               window: int, page_size: int, cache_dtype, keep_first: int = 0, bias_span: int = 0, softcap: float | None = None) -> _SwaConfig:
     """keep_first: with a window, the sequence's first positions that stay visible; bias_span: rows - 1 of the distance-bias table the
-    attention calls are given (`dist_bias`)."""
+    attention calls are given (`dist_bias`); softcap: scores become softcap tanh(score / softcap) (None: off)."""
     return _SwaConfig(heads, kv_heads, dim, vdim, int(rot_dims), int(bool(rot_values)), int(bool(qk_norm)), float(eps), float(scale),
-                      int(window), int(page_size), SEQ_DTYPE[cache_dtype], int(keep_first), int(bias_span))
+                      int(window), int(page_size), SEQ_DTYPE[cache_dtype], int(keep_first), int(bias_span), float(softcap or 0.0))
 
 
 def swa_conv_prep(cfg: _SwaConfig, proj: torch.Tensor, bias: torch.Tensor | None, conv_w: torch.Tensor | None, q_norm_w: torch.Tensor | None,
-                  k_norm_w: torch.Tensor | None, batch, conv_state: torch.Tensor | None, kcache: torch.Tensor, vcache: torch.Tensor) -> torch.Tensor:
-    """The un-rotated prep with a causal convolution over time behind the projections and RMS norms over the whole q and k projections
+                  k_norm_w: torch.Tensor | None, batch, conv_state: torch.Tensor | None, kcache: torch.Tensor, vcache: torch.Tensor,
+                  inv_freq: torch.Tensor | None = None) -> torch.Tensor:
+    """The prep with a causal convolution over time behind the projections and RMS norms over the whole q and k projections
     (ktx_swa_conv_prep): proj fp32 [T, >= C] with q | k | v at column 0 -> q fp32 [T, heads * dim] (normed, scaled); key and value rows
-    are appended, the convolution's state slots move on.  conv_w fp32 [C, taps] or None."""
+    are appended, the convolution's state slots move on.  conv_w fp32 [C, taps] or None; inv_freq fp64 [rot_dims / 2]: un-normed q and k
+    heads turn behind the convolution."""
     pp, ldp = _rows_f32(proj, "swa_conv_prep proj")
     for t_, what in ((bias, "bias"), (conv_w, "conv_w"), (q_norm_w, "q_norm_w"), (k_norm_w, "k_norm_w"), (conv_state, "conv_state")):
         _f32(t_, "swa_conv_prep " + what)
@@ -198,11 +200,13 @@ def swa_conv_prep(cfg: _SwaConfig, proj: torch.Tensor, bias: torch.Tensor | None
             (k_norm_w is not None and k_norm_w.numel() != nk) or \
             (taps > 1 and (conv_state is None or tuple(conv_state.shape[1:]) != (taps - 1, Cn))):
         raise KtxError("swa_conv_prep: shapes do not fit")
+    if cfg.rot_dims and (inv_freq is None or inv_freq.dtype != torch.float64 or inv_freq.numel() != cfg.rot_dims // 2):
+        raise KtxError("swa_conv_prep: inv_freq must be fp64 [rot_dims / 2]")
     q = torch.empty((T, nq), dtype=torch.float32, device=proj.device)
     check(lib.ktx_swa_conv_prep(C.byref(cfg), batch.B, T, int(batch.max_q_len), taps, pp, ldp, _ptr(bias), _ptr(conv_w), _ptr(q_norm_w), _ptr(k_norm_w),
                                 batch.q_indptr.data_ptr(), batch.pos0.data_ptr(), batch.slot.data_ptr(), batch.tok_req.data_ptr(),
-                                _ptr(conv_state), batch.cache_loc.data_ptr(), kcache.data_ptr(), vcache.data_ptr(), q.data_ptr(),
-                                _stream_ptr(proj.device)))
+                                _ptr(conv_state), _ptr(inv_freq) if cfg.rot_dims else None, batch.cache_loc.data_ptr(), kcache.data_ptr(),
+                                vcache.data_ptr(), q.data_ptr(), _stream_ptr(proj.device)))
     return q
 
 

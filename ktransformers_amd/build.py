@@ -18,10 +18,10 @@ CSRC = os.path.join(HERE, "csrc")
 LIBDIR = os.path.join(HERE, "lib")
 OBJDIR = os.path.join(LIBDIR, "obj")
 LIB = os.path.join(LIBDIR, "libktx_hip.so")
-# the sequence-mixer, hybrid-decoder and window-attention / scan kernels alone (include/ktx_seq.h, ktx_hyb.h, ktx_swa.h): what the fp32-residual families need, built in
-# well under a minute
+# the sequence-mixer, hybrid-decoder, window-attention / scan and decayed-state kernels alone (include/ktx_seq.h, ktx_hyb.h, ktx_swa.h,
+# ktx_gla.h): what the fp32-residual families need, built in about a minute
 SEQ_LIB = os.path.join(LIBDIR, "libktx_seq.so")
-SEQ_SOURCES = ("ktx_seq.hip", "ktx_hyb.hip", "ktx_swa.hip", "ktx_err.hip")
+SEQ_SOURCES = ("ktx_seq.hip", "ktx_hyb.hip", "ktx_swa.hip", "ktx_gla.hip", "ktx_err.hip")
 
 # -ffp-contract=off: the parity contract needs every fp32 op rounded exactly as the reference's AVX512 code does;
 # FMAs appear only where the reference issues one (explicit fmaf()).
@@ -31,7 +31,8 @@ CFLAGS = ["--offload-arch=gfx950", "-O3", "-std=c++17", "-ffp-contract=off", "-f
 # per-source extra flags: the sequence-mixer kernels keep fp32 state and norms on the vector ALUs and are built without the packed
 # fp32 instructions (scalar v_fma / v_mul only)
 _NO_PACKED_FP32 = ["-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops"]
-EXTRA_CFLAGS = {"ktx_seq.hip": _NO_PACKED_FP32, "ktx_hyb.hip": _NO_PACKED_FP32, "ktx_swa.hip": _NO_PACKED_FP32}
+EXTRA_CFLAGS = {"ktx_seq.hip": _NO_PACKED_FP32, "ktx_hyb.hip": _NO_PACKED_FP32, "ktx_swa.hip": _NO_PACKED_FP32,
+                "ktx_gla.hip": _NO_PACKED_FP32}
 
 
 def sources() -> list[str]:

@@ -18,6 +18,17 @@ namespace {
 
 #include "ktx_seq_dev.inc"
 
+// the epilogues a dense product can end in (KTX_ACT_*)
+__device__ __forceinline__ float act_f32(float v, int act, float arg) {
+  if (act == KTX_ACT_GELU_TANH) return gelu_tanh_f32(v);
+  if (act == KTX_ACT_RELU_SQ) {
+    const float r = fmaxf(v, 0.f);
+    return r * r;
+  }
+  if (act == KTX_ACT_SOFT_CAP) return arg * tanhf(v / arg);
+  return v;
+}
+
 // ---------------------------------------------------------------------------------------------------------------------
 // embedding + sinusoidal positions
 template <typename WT>
@@ -44,7 +55,7 @@ __global__ void __launch_bounds__(256) embed_sinpos_kernel(int width, int vocab,
 template <typename AT, typename CT, typename YT>
 __global__ void __launch_bounds__(256) dense_gemm_kernel(int M, int N, int K, const AT* __restrict__ A, int64_t lda,
                                                          const CT* __restrict__ W, YT* __restrict__ Y, int64_t ldy, int act,
-                                                         int ksplit, bool vec_a, bool vec_w) {
+                                                         float act_arg, int ksplit, bool vec_a, bool vec_w) {
   constexpr int LD = GemmTraits<CT>::LDS_LD;
   __shared__ __attribute__((aligned(16))) CT As[64 * LD];
   __shared__ __attribute__((aligned(16))) CT Ws[64 * LD];
@@ -106,7 +117,7 @@ __global__ void __launch_bounds__(256) dense_gemm_kernel(int M, int N, int K, co
           if (ksplit > 1) {
             if constexpr (sizeof(YT) == 4) atomicAdd(reinterpret_cast<float*>(Y) + (size_t)m * ldy + n, v);
           } else {
-            if (act == KTX_ACT_GELU_TANH) v = gelu_tanh_f32(v);
+            v = act_f32(v, act, act_arg);
             st_elem(Y, (size_t)m * ldy + n, v);
           }
         }
@@ -680,7 +691,8 @@ __global__ void __launch_bounds__(256) mlstm_gate_norm_kernel(ktx_mlstm_config c
 // product's type, a wavefront owns RPW weight rows and streams them with 16-byte loads, fp32 accumulation, one wave reduction per row.
 template <typename AT, typename CT, typename YT, int MM>
 __global__ void __launch_bounds__(256) dense_gemv_kernel(int M, int N, int K, const AT* __restrict__ A, int64_t lda,
-                                                         const CT* __restrict__ W, YT* __restrict__ Y, int64_t ldy, int act, bool vec) {
+                                                         const CT* __restrict__ W, YT* __restrict__ Y, int64_t ldy, int act,
+                                                         float act_arg, bool vec) {
   extern __shared__ __attribute__((aligned(16))) unsigned char gv_lds[];
   CT* As = reinterpret_cast<CT*>(gv_lds);                 // [MM][Kp], Kp = K rounded up to 8
   const int Kp = (K + 7) & ~7;
@@ -729,7 +741,7 @@ __global__ void __launch_bounds__(256) dense_gemv_kernel(int M, int N, int K, co
     for (int m = 0; m < MM; m++) {
       float a = wave_sum(acc[m]);
       if (lane == 0 && m < M) {
-        if (act == KTX_ACT_GELU_TANH) a = gelu_tanh_f32(a);
+        a = act_f32(a, act, act_arg);
         st_elem(Y, (size_t)m * ldy + n, a);
       }
     }
@@ -744,7 +756,7 @@ __global__ void __launch_bounds__(256) dense_gemv_kernel(int M, int N, int K, co
 template <typename AT, typename YT, bool GLU>
 __global__ void __launch_bounds__(256) dense_gemv_mfma_kernel(int M, int N, int K, const AT* __restrict__ A, int64_t lda,
                                                               const bf16_t* __restrict__ W, YT* __restrict__ Y, int64_t ldy, int act,
-                                                              float limit, float slope, float shift) {
+                                                              float act_arg, float limit, float slope, float shift) {
   __shared__ float red[4][64][4];
   const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, l16 = lane & 15, lq = lane >> 4;
   const int n = blockIdx.x * 16 + l16;
@@ -784,17 +796,28 @@ __global__ void __launch_bounds__(256) dense_gemv_mfma_kernel(int M, int N, int 
           st_elem(Y, (size_t)m * ldy + (n >> 1), g * sigmoid_f32(slope * g) * (u + shift));
         }
       } else if (wok && m < M) {
-        if (act == KTX_ACT_GELU_TANH) v = gelu_tanh_f32(v);
+        v = act_f32(v, act, act_arg);
         st_elem(Y, (size_t)m * ldy + n, v);
       }
     }
   }
 }
 
+// an activation over n elements in place, 8 (bf16) or 4 (fp32) per thread where they are 16-byte aligned
 template <typename T>
-__global__ void __launch_bounds__(256) gelu_tanh_kernel(size_t n, T* __restrict__ y) {
-  const size_t e = (size_t)blockIdx.x * 256 + threadIdx.x;
-  if (e < n) st_elem(y, e, gelu_tanh_f32(ld_elem(y, e)));
+__global__ void __launch_bounds__(256) act_rows_kernel(size_t n, T* __restrict__ y, int act, float act_arg, bool vec) {
+  constexpr int N = 16 / sizeof(T);
+  const size_t e0 = ((size_t)blockIdx.x * 256 + threadIdx.x) * N;
+  if (e0 >= n) return;
+  if (vec && e0 + N <= n) {
+    union { uint4 u; T v[N]; } r;
+    r.u = *reinterpret_cast<const uint4*>(y + e0);
+#pragma unroll
+    for (int i = 0; i < N; i++) st_elem(r.v, i, act_f32(ld_elem(r.v, i), act, act_arg));
+    *reinterpret_cast<uint4*>(y + e0) = r.u;
+    return;
+  }
+  for (int i = 0; i < N && e0 + i < n; i++) st_elem(y, e0 + i, act_f32(ld_elem(y, e0 + i), act, act_arg));
 }
 
 // ---------------------------------------------------------------------------------------------------------------------
@@ -1198,7 +1221,7 @@ int ktx_dense_gemv_glu(int M, int F, int K, const void* d_A, int a_dtype, int64_
   const int N = 2 * F;
   const unsigned blocks = (unsigned)((N + 15) / 16);
 #define KTX_GLU_GO(AT, YT)                                                                                                         \
-  dense_gemv_mfma_kernel<AT, YT, true><<<blocks, 256, 0, st>>>(M, N, K, (const AT*)d_A, lda, (const bf16_t*)d_W, (YT*)d_Y, ldy, 0, limit, \
+  dense_gemv_mfma_kernel<AT, YT, true><<<blocks, 256, 0, st>>>(M, N, K, (const AT*)d_A, lda, (const bf16_t*)d_W, (YT*)d_Y, ldy, 0, 0.f, limit, \
                                                                slope, up_shift)
   if (a_dtype == KTX_SEQ_F32 && y_dtype == KTX_SEQ_F32) KTX_GLU_GO(float, float);
   else if (a_dtype == KTX_SEQ_F32) KTX_GLU_GO(float, bf16_t);
@@ -1211,10 +1234,15 @@ int ktx_dense_gemv_glu(int M, int F, int K, const void* d_A, int a_dtype, int64_
 
 int ktx_dense_gemm(int M, int N, int K, const void* d_A, int a_dtype, int64_t lda, const void* d_W, int w_dtype, void* d_Y,
                    int y_dtype, int64_t ldy, int act, int ksplit, ktx_stream_t stream) {
+  return ktx_dense_gemm_act(M, N, K, d_A, a_dtype, lda, d_W, w_dtype, d_Y, y_dtype, ldy, act, 0.f, ksplit, stream);
+}
+
+int ktx_dense_gemm_act(int M, int N, int K, const void* d_A, int a_dtype, int64_t lda, const void* d_W, int w_dtype, void* d_Y,
+                       int y_dtype, int64_t ldy, int act, float act_arg, int ksplit, ktx_stream_t stream) {
   KTX_REQUIRE(M >= 0 && N > 0 && K > 0, "ktx_dense_gemm: M >= 0, N, K > 0");
   KTX_REQUIRE(d_A && d_W && d_Y, "ktx_dense_gemm: null pointer");
   KTX_REQUIRE(lda >= K && ldy >= N, "ktx_dense_gemm: lda >= K and ldy >= N");
-  KTX_REQUIRE(act == KTX_ACT_NONE || act == KTX_ACT_GELU_TANH, "ktx_dense_gemm: unknown activation");
+  KTX_REQUIRE(act >= KTX_ACT_NONE && act <= KTX_ACT_SOFT_CAP && (act != KTX_ACT_SOFT_CAP || act_arg > 0.f), "ktx_dense_gemm: unknown activation");
   KTX_REQUIRE(ksplit >= 1 && (ksplit == 1 || (y_dtype == KTX_SEQ_F32 && act == KTX_ACT_NONE)),
               "ktx_dense_gemm: split-K adds into a zeroed fp32 output and takes no activation");
   KTX_REQUIRE(!(w_dtype == KTX_SEQ_F32 && a_dtype != KTX_SEQ_F32), "ktx_dense_gemm: an fp32 product needs fp32 activations");
@@ -1224,13 +1252,13 @@ int ktx_dense_gemm(int M, int N, int K, const void* d_A, int a_dtype, int64_t ld
       (lda * (a_dtype == KTX_SEQ_F32 ? 4 : 2)) % 16 == 0) {
     const unsigned blocks = (unsigned)((N + 15) / 16);
     if (a_dtype == KTX_SEQ_F32 && y_dtype == KTX_SEQ_F32)
-      dense_gemv_mfma_kernel<float, float, false><<<blocks, 256, 0, st>>>(M, N, K, (const float*)d_A, lda, (const bf16_t*)d_W, (float*)d_Y, ldy, act, 0.f, 0.f, 0.f);
+      dense_gemv_mfma_kernel<float, float, false><<<blocks, 256, 0, st>>>(M, N, K, (const float*)d_A, lda, (const bf16_t*)d_W, (float*)d_Y, ldy, act, act_arg, 0.f, 0.f, 0.f);
     else if (a_dtype == KTX_SEQ_F32)
-      dense_gemv_mfma_kernel<float, bf16_t, false><<<blocks, 256, 0, st>>>(M, N, K, (const float*)d_A, lda, (const bf16_t*)d_W, (bf16_t*)d_Y, ldy, act, 0.f, 0.f, 0.f);
+      dense_gemv_mfma_kernel<float, bf16_t, false><<<blocks, 256, 0, st>>>(M, N, K, (const float*)d_A, lda, (const bf16_t*)d_W, (bf16_t*)d_Y, ldy, act, act_arg, 0.f, 0.f, 0.f);
     else if (y_dtype == KTX_SEQ_F32)
-      dense_gemv_mfma_kernel<bf16_t, float, false><<<blocks, 256, 0, st>>>(M, N, K, (const bf16_t*)d_A, lda, (const bf16_t*)d_W, (float*)d_Y, ldy, act, 0.f, 0.f, 0.f);
+      dense_gemv_mfma_kernel<bf16_t, float, false><<<blocks, 256, 0, st>>>(M, N, K, (const bf16_t*)d_A, lda, (const bf16_t*)d_W, (float*)d_Y, ldy, act, act_arg, 0.f, 0.f, 0.f);
     else
-      dense_gemv_mfma_kernel<bf16_t, bf16_t, false><<<blocks, 256, 0, st>>>(M, N, K, (const bf16_t*)d_A, lda, (const bf16_t*)d_W, (bf16_t*)d_Y, ldy, act, 0.f, 0.f, 0.f);
+      dense_gemv_mfma_kernel<bf16_t, bf16_t, false><<<blocks, 256, 0, st>>>(M, N, K, (const bf16_t*)d_A, lda, (const bf16_t*)d_W, (bf16_t*)d_Y, ldy, act, act_arg, 0.f, 0.f, 0.f);
     KTX_HIP(hipGetLastError());
     return 0;
   }
@@ -1245,7 +1273,7 @@ int ktx_dense_gemm(int M, int N, int K, const void* d_A, int a_dtype, int64_t ld
 #define KTX_GEMV_GO(AT, CT, YT, MM)                                                                                     \
   do {                                                                                                                  \
     KTX_HIP(ktx_set_max_lds((const void*)dense_gemv_kernel<AT, CT, YT, MM>, 128 * 1024));                               \
-    dense_gemv_kernel<AT, CT, YT, MM><<<blocks, 256, lds, st>>>(M, N, K, (const AT*)d_A, lda, (const CT*)d_W, (YT*)d_Y, ldy, act, vec); \
+    dense_gemv_kernel<AT, CT, YT, MM><<<blocks, 256, lds, st>>>(M, N, K, (const AT*)d_A, lda, (const CT*)d_W, (YT*)d_Y, ldy, act, act_arg, vec); \
   } while (0)
 #define KTX_GEMV_MM(AT, CT, YT)            \
   do {                                     \
@@ -1269,7 +1297,7 @@ int ktx_dense_gemm(int M, int N, int K, const void* d_A, int a_dtype, int64_t ld
   const bool vec_a = aligned16(d_A) && (lda * asz) % 16 == 0 && K % 8 == 0;
   const bool vec_w = aligned16(d_W) && ((size_t)K * wsz) % 16 == 0 && K % 8 == 0;
 #define KTX_GEMM_GO(AT, CT, YT)                                                                                          \
-  dense_gemm_kernel<AT, CT, YT><<<grid, 256, 0, st>>>(M, N, K, (const AT*)d_A, lda, (const CT*)d_W, (YT*)d_Y, ldy, act, ksplit, \
+  dense_gemm_kernel<AT, CT, YT><<<grid, 256, 0, st>>>(M, N, K, (const AT*)d_A, lda, (const CT*)d_W, (YT*)d_Y, ldy, act, act_arg, ksplit, \
                                                       vec_a, vec_w)
   if (w_dtype == KTX_SEQ_BF16) {
     if (a_dtype == KTX_SEQ_F32 && y_dtype == KTX_SEQ_F32) KTX_GEMM_GO(float, bf16_t, float);
@@ -1405,17 +1433,20 @@ int ktx_sigattn_prefill(const ktx_sigattn_config* cfg, int B, int T, int max_q_l
   return 0;
 }
 
-int ktx_gelu_tanh(size_t n, void* d_y, int dtype, ktx_stream_t stream) {
-  KTX_REQUIRE(d_y || n == 0, "ktx_gelu_tanh: null pointer");
-  if (n == 0) return 0;
+int ktx_act_rows(size_t n, void* d_y, int dtype, int act, float act_arg, ktx_stream_t stream) {
+  KTX_REQUIRE((d_y || n == 0) && (dtype == KTX_SEQ_F32 || dtype == KTX_SEQ_BF16), "ktx_act_rows: null pointer / unknown type");
+  KTX_REQUIRE(act >= KTX_ACT_NONE && act <= KTX_ACT_SOFT_CAP && (act != KTX_ACT_SOFT_CAP || act_arg > 0.f), "ktx_act_rows: unknown activation");
+  if (n == 0 || act == KTX_ACT_NONE) return 0;
+  const size_t per = 256 * (dtype == KTX_SEQ_F32 ? 4 : 8);
+  const unsigned blocks = (unsigned)((n + per - 1) / per);
   hipStream_t st = (hipStream_t)stream;
-  const unsigned blocks = (unsigned)((n + 255) / 256);
-  if (dtype == KTX_SEQ_BF16) gelu_tanh_kernel<bf16_t><<<blocks, 256, 0, st>>>(n, (bf16_t*)d_y);
-  else if (dtype == KTX_SEQ_F32) gelu_tanh_kernel<float><<<blocks, 256, 0, st>>>(n, (float*)d_y);
-  else return ktx_fail("ktx_gelu_tanh: unknown element type");
+  if (dtype == KTX_SEQ_F32) act_rows_kernel<float><<<blocks, 256, 0, st>>>(n, (float*)d_y, act, act_arg, aligned16(d_y));
+  else act_rows_kernel<bf16_t><<<blocks, 256, 0, st>>>(n, (bf16_t*)d_y, act, act_arg, aligned16(d_y));
   KTX_HIP(hipGetLastError());
   return 0;
 }
+
+int ktx_gelu_tanh(size_t n, void* d_y, int dtype, ktx_stream_t stream) { return ktx_act_rows(n, d_y, dtype, KTX_ACT_GELU_TANH, 0.f, stream); }
 
 int ktx_mlstm_forward(const ktx_mlstm_config* cfg, int B, const int32_t* d_q_indptr, const int32_t* d_pos0, const int32_t* d_slot,
                       const float* d_proj, int64_t ldp, int q_off, int k_off, int v_off, int i_off, int f_off, const float* d_ib,

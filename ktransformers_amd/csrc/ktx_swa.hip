@@ -16,6 +16,7 @@
 namespace {
 
 #include "ktx_seq_dev.inc"
+#include "ktx_conv_dev.inc"
 
 __device__ __forceinline__ float silu_f32(float z) { return z / (1.0f + expf(-z)); }
 __device__ __forceinline__ float softplus_f32(float z) { return z > 20.f ? z : log1pf(expf(z)); }
@@ -249,19 +250,33 @@ __global__ void __launch_bounds__(256) swa_prep_kernel(ktx_swa_config c, const f
 // Input u[c] at relative token ii of the request: this step's projection (+ bias) for ii >= 0, the slot's state row taps - 1 + ii for
 // ii < 0 when the request has a past, zero otherwise.
 constexpr int CP_MAX_TAPS = 16;
+// with rot_dims > 0 (heads that are not normed): the first rot_dims entries of every convolved q and k head turn with the position, in
+// pairs (2i, 2i + 1); the token's cosines | sines, angles in fp64
+__device__ __forceinline__ void conv_prep_angles(const ktx_swa_config& c, int pos, const double* __restrict__ inv_freq, float* cs) {
+  const int NP = c.rot_dims / 2;
+  for (int i = threadIdx.x; i < NP; i += 256) {
+    double si, co;
+    sincos((double)pos * inv_freq[i], &si, &co);
+    cs[i] = (float)co;
+    cs[NP + i] = (float)si;
+  }
+}
 template <typename KT>
 __global__ void __launch_bounds__(256) swa_conv_prep_kernel(ktx_swa_config c, int taps, const float* __restrict__ proj, int64_t ldp,
                                                             const float* __restrict__ bias, const float* __restrict__ cw,
                                                             const float* __restrict__ qw, const float* __restrict__ kw,
                                                             const int32_t* __restrict__ q_indptr, const int32_t* __restrict__ pos0,
                                                             const int32_t* __restrict__ slot, const int32_t* __restrict__ tok_req,
-                                                            const float* __restrict__ conv_state, const int32_t* __restrict__ cache_loc,
+                                                            const float* __restrict__ conv_state, const double* __restrict__ inv_freq,
+                                                            const int32_t* __restrict__ cache_loc,
                                                             KT* __restrict__ kcache, KT* __restrict__ vcache, float* __restrict__ q_out) {
-  extern __shared__ float row[];           // [H * D | G * D | G * V]
+  extern __shared__ float row[];           // [H * D | G * D | G * V], then cos | sin of the rot_dims / 2 angles
   __shared__ float red[4];
   const int t = blockIdx.x, tid = threadIdx.x;
-  const int nq = c.heads * c.dim, nk = c.kv_heads * c.dim, nv = c.kv_heads * c.vdim, C = nq + nk + nv;
+  const int nq = c.heads * c.dim, nk = c.kv_heads * c.dim, nv = c.kv_heads * c.vdim, C = nq + nk + nv, NP = c.rot_dims / 2;
   const int b = tok_req[t], i = t - q_indptr[b];
+  float* cs = row + C;
+  conv_prep_angles(c, pos0[b] + i, inv_freq, cs);
   const bool carried = pos0[b] > 0;
   const float* st = conv_state ? conv_state + (size_t)slot[b] * (taps - 1) * C : nullptr;
   float sq = 0.f, sk = 0.f;
@@ -293,8 +308,16 @@ __global__ void __launch_bounds__(256) swa_conv_prep_kernel(ktx_swa_config c, in
   const float rq = qw ? 1.0f / sqrtf(block_sum256(sq, red) / (float)nq + c.eps) : 1.0f;
   const float rk = kw ? 1.0f / sqrtf(block_sum256(sk, red) / (float)nk + c.eps) : 1.0f;
   const size_t loc = (size_t)cache_loc[t];
-  for (int e = tid; e < C; e += 256) {      // (each thread re-reads only what it wrote)
-    const float y = row[e];
+  if (NP) __syncthreads();                  // a pair's partner is another thread's (without rotation each re-reads only what it wrote)
+  for (int e = tid; e < C; e += 256) {
+    float y = row[e];
+    if (NP && e < nq + nk) {
+      const int j = (e < nq ? e : e - nq) % c.dim;
+      if (j < 2 * NP) {
+        const float co = cs[j >> 1], si = cs[NP + (j >> 1)];
+        y = (j & 1) ? y * co + row[e - 1] * si : y * co - row[e + 1] * si;
+      }
+    }
     if (e < nq) q_out[(size_t)t * nq + e] = y * rq * (qw ? qw[e] : 1.0f) * c.scale;
     else if (e < nq + nk) st_elem(kcache, loc * nk + (e - nq), y * rk * (kw ? kw[e - nq] : 1.0f));
     else st_elem(vcache, loc * nv + (e - nq - nk), y);
@@ -312,13 +335,15 @@ __global__ void __launch_bounds__(256) swa_conv_prep_vec_kernel(ktx_swa_config c
                                                                 const int32_t* __restrict__ q_indptr, const int32_t* __restrict__ pos0,
                                                                 const int32_t* __restrict__ slot, const int32_t* __restrict__ tok_req,
                                                                 float* __restrict__ conv_state, int one_token,
-                                                                const int32_t* __restrict__ cache_loc, KT* __restrict__ kcache,
-                                                                KT* __restrict__ vcache, float* __restrict__ q_out) {
-  extern __shared__ __attribute__((aligned(16))) float row[];      // [H * D | G * D | G * V]
+                                                                const double* __restrict__ inv_freq, const int32_t* __restrict__ cache_loc,
+                                                                KT* __restrict__ kcache, KT* __restrict__ vcache, float* __restrict__ q_out) {
+  extern __shared__ __attribute__((aligned(16))) float row[];      // [H * D | G * D | G * V], then cos | sin of the rot_dims / 2 angles
   __shared__ float red[4];
   const int t = blockIdx.x, tid = threadIdx.x;
-  const int nq = c.heads * c.dim, nk = c.kv_heads * c.dim, nv = c.kv_heads * c.vdim, C = nq + nk + nv;
+  const int nq = c.heads * c.dim, nk = c.kv_heads * c.dim, nv = c.kv_heads * c.vdim, C = nq + nk + nv, NP = c.rot_dims / 2;
   const int b = tok_req[t], i = t - q_indptr[b];
+  float* cs = row + C;
+  conv_prep_angles(c, pos0[b] + i, inv_freq, cs);
   const bool carried = pos0[b] > 0;
   float* st = conv_state + (size_t)slot[b] * (TAPS - 1) * C;
   const float4 zero4 = make_float4(0.f, 0.f, 0.f, 0.f);
@@ -370,8 +395,14 @@ __global__ void __launch_bounds__(256) swa_conv_prep_vec_kernel(ktx_swa_config c
   const float rq = qw ? 1.0f / sqrtf(block_sum256(sq, red) / (float)nq + c.eps) : 1.0f;
   const float rk = kw ? 1.0f / sqrtf(block_sum256(sk, red) / (float)nk + c.eps) : 1.0f;
   const size_t loc = (size_t)cache_loc[t];
-  for (int e = tid * 4; e < C; e += 1024) {      // (each thread re-reads only what it wrote)
+  if (NP) __syncthreads();                       // (the angles; of the row each thread re-reads only what it wrote)
+  for (int e = tid * 4; e < C; e += 1024) {
     float4 y = *reinterpret_cast<const float4*>(row + e);
+    if (NP && e < nq + nk) {                     // two pairs of one head (rotating heads have dim % 4 == 0 here)
+      const int j = (e < nq ? e : e - nq) % c.dim, n = j >> 1;
+      if (j < 2 * NP) y = make_float4(y.x * cs[n] - y.y * cs[NP + n], y.y * cs[n] + y.x * cs[NP + n], y.z, y.w);
+      if (j + 2 < 2 * NP) y = make_float4(y.x, y.y, y.z * cs[n + 1] - y.w * cs[NP + n + 1], y.w * cs[n + 1] + y.z * cs[NP + n + 1]);
+    }
     if (e < nq) {
       const float4 g = qw ? *reinterpret_cast<const float4*>(qw + e) : make_float4(1.f, 1.f, 1.f, 1.f);
       const float r = rq * c.scale;
@@ -389,28 +420,6 @@ __global__ void __launch_bounds__(256) swa_conv_prep_vec_kernel(ktx_swa_config c
         *reinterpret_cast<float4*>(dst) = y;
       }
     }
-  }
-}
-
-// the state of a causal convolution over C channels moves on behind a step: the slot's rows become the last taps - 1 inputs (this step's
-// projections + bias; older ones from the old state when the request brought fewer).  thread = channel, rows oldest first
-__global__ void __launch_bounds__(256) conv_state_update_kernel(int C, int taps, const int32_t* __restrict__ q_indptr,
-                                                                const int32_t* __restrict__ pos0, const int32_t* __restrict__ slot,
-                                                                const float* __restrict__ proj, int64_t ldp, const float* __restrict__ bias,
-                                                                float* __restrict__ conv_state) {
-  const int b = blockIdx.y, e = blockIdx.x * 256 + threadIdx.x;
-  if (e >= C) return;
-  const int first = q_indptr[b], n = q_indptr[b + 1] - first;
-  if (n <= 0) return;
-  const bool carried = pos0[b] > 0;
-  const float be = bias ? bias[e] : 0.f;
-  float* st = conv_state + (size_t)slot[b] * (taps - 1) * C;
-  for (int j = 0; j < taps - 1; j++) {      // row j takes the input n - (taps - 1) + j; an old row it may need lies further on (j + n > j)
-    const int ii = n - (taps - 1) + j;
-    float v = 0.f;
-    if (ii >= 0) v = proj[(size_t)(first + ii) * ldp + e] + be;
-    else if (carried) v = st[(size_t)(j + n) * C + e];
-    st[(size_t)j * C + e] = v;
   }
 }
 
@@ -482,6 +491,7 @@ __global__ void __launch_bounds__(256) swa_fwd_kernel(ktx_swa_config c, int T, i
         const float* kj = kt + (size_t)j * DP;
         float s = 0.f;
         for (int d = 0; d < D; d++) s += qh[d] * kj[d];
+        if (c.softcap > 0.f) s = c.softcap * tanhf(s / c.softcap);
         if (dist_bias) s += dist_bias[(size_t)min(p - jpos[j], c.bias_span) * c.heads + h0 + h];
         sc[(size_t)h * KTN + j] = s;      // (scale is folded into q)
       }
@@ -605,6 +615,10 @@ __global__ void __launch_bounds__(256) swa_merge_kernel(int T, int H, int V, int
 // resident in registers) and walks 32-key tiles of the union of its rows' windows: keys staged row-major, values transposed; scores,
 // mask, running maximum and sum in fp32 (DPP reductions inside the 16-lane column groups), weights through a per-wavefront LDS tile
 // into the second product.  Key ranges (blockIdx.z) leave unnormalised partial sums that swa_merge_kernel joins.
+// cap tanh(s / cap) on v_exp_f32 + v_rcp_f32 (tanh x = 1 - 2 / (1 + e^2x); icap = 2 log2(e) / cap): an absolute error of about 1e-7 cap
+__device__ __forceinline__ float soft_cap_fast(float s, float cap, float icap) {
+  return cap > 0.f ? cap - 2.0f * cap * __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(s * icap)) : s;
+}
 constexpr int SM_KT = 32, SM_PST = SM_KT + 8, SM_KSMAX = 8;
 template <int NT, typename OT>
 __global__ void __launch_bounds__(256) swa_mfma_kernel(ktx_swa_config c, int T, int row_tiles, const float* __restrict__ q,
@@ -679,6 +693,7 @@ __global__ void __launch_bounds__(256) swa_mfma_kernel(ktx_swa_config c, int T, 
   const int32_t* pages = page_indices + page_indptr[b];
   const int ksegs = D / 8, vsegs = V / 8;
   bf16_t* Pw = Ps + (size_t)wave * 16 * SM_PST;
+  const float icap = c.softcap > 0.f ? 2.8853900817779268f / c.softcap : 0.f;      // 2 log2(e) / cap
   for (int jt = j0; jt < j1; jt += SM_KT) {
     const int nk = min(SM_KT, j1 - jt);
     __syncthreads();
@@ -722,8 +737,8 @@ __global__ void __launch_bounds__(256) swa_mfma_kernel(ktx_swa_config c, int T, 
         const bool oka = vrow[r] && ua < j1 && (ja >= lorow[r] || ja < c.keep_first) && ja <= prow[r];
         const bool okb = vrow[r] && ub < j1 && (jb >= lorow[r] || jb < c.keep_first) && jb <= prow[r];
         float sa = -INFINITY, sb = -INFINITY;      // (scale is folded into q)
-        if (oka) sa = s0[r] + (brow[r] ? brow[r][(size_t)min(prow[r] - ja, c.bias_span) * H] : 0.f);
-        if (okb) sb = s1[r] + (brow[r] ? brow[r][(size_t)min(prow[r] - jb, c.bias_span) * H] : 0.f);
+        if (oka) sa = soft_cap_fast(s0[r], c.softcap, icap) + (brow[r] ? brow[r][(size_t)min(prow[r] - ja, c.bias_span) * H] : 0.f);
+        if (okb) sb = soft_cap_fast(s1[r], c.softcap, icap) + (brow[r] ? brow[r][(size_t)min(prow[r] - jb, c.bias_span) * H] : 0.f);
         const float mt = row16_max(fmaxf(sa, sb));
         const float mn = fmaxf(mrun[r], mt);
         const float mb = mn == -INFINITY ? 0.f : mn;
@@ -1125,7 +1140,7 @@ static int swa_check(const ktx_swa_config* c, const char* who) {
               std::string(who) + ": heads a multiple of kv_heads, positive sizes, a known cache type");
   KTX_REQUIRE(c->rot_dims >= 0 && c->rot_dims % 2 == 0 && c->rot_dims <= c->dim, std::string(who) + ": rot_dims even and at most dim");
   KTX_REQUIRE(!c->rot_values || c->vdim % 2 == 0, std::string(who) + ": rotated values need an even vdim");
-  KTX_REQUIRE(c->keep_first >= 0 && c->bias_span >= 0, std::string(who) + ": keep_first and bias_span are not negative");
+  KTX_REQUIRE(c->keep_first >= 0 && c->bias_span >= 0 && c->softcap >= 0.f, std::string(who) + ": keep_first, bias_span and softcap are not negative");
   return 0;
 }
 
@@ -1155,31 +1170,33 @@ int ktx_swa_prep(const ktx_swa_config* cfg, int T, const float* d_proj, int64_t 
 
 int ktx_swa_conv_prep(const ktx_swa_config* cfg, int B, int T, int max_q_len, int taps, const float* d_proj, int64_t ldp, const float* d_bias,
                       const float* d_conv_w, const float* d_q_norm_w, const float* d_k_norm_w, const int32_t* d_q_indptr,
-                      const int32_t* d_pos0, const int32_t* d_slot, const int32_t* d_tok_req, float* d_conv_state,
+                      const int32_t* d_pos0, const int32_t* d_slot, const int32_t* d_tok_req, float* d_conv_state, const double* d_inv_freq,
                       const int32_t* d_cache_loc, void* d_kcache, void* d_vcache, float* d_q_out, ktx_stream_t stream) {
   if (swa_check(cfg, "ktx_swa_conv_prep")) return -1;
   KTX_REQUIRE(B >= 0 && T >= 0 && max_q_len >= 0 && d_proj && d_q_indptr && d_pos0 && d_slot && d_tok_req && d_cache_loc && d_kcache && d_vcache && d_q_out,
               "ktx_swa_conv_prep: null pointer");
   KTX_REQUIRE(taps >= 0 && taps <= CP_MAX_TAPS && (taps <= 1 || (d_conv_w && d_conv_state)),
               "ktx_swa_conv_prep: at most 16 taps; a convolution needs its weights and state slots");
-  KTX_REQUIRE(cfg->rot_dims == 0 && !cfg->rot_values, "ktx_swa_conv_prep: no rotation in this form");
+  KTX_REQUIRE(!cfg->rot_values && (cfg->rot_dims == 0 || (d_inv_freq && !d_q_norm_w && !d_k_norm_w)),
+              "ktx_swa_conv_prep: values do not turn in this form; turning heads have their frequencies and no norms");
   const int C = cfg->heads * cfg->dim + cfg->kv_heads * (cfg->dim + cfg->vdim);
   KTX_REQUIRE(ldp >= C, "ktx_swa_conv_prep: rows of q | k | v");
-  KTX_REQUIRE((size_t)C * 4 <= 150 * 1024, "ktx_swa_conv_prep: a token's q | k | v row must fit the LDS");
+  KTX_REQUIRE((size_t)(C + cfg->rot_dims) * 4 <= 150 * 1024, "ktx_swa_conv_prep: a token's q | k | v row and the angles must fit the LDS");
   if (T == 0 || B == 0) return 0;
   hipStream_t st = (hipStream_t)stream;
-  const size_t lds = (size_t)C * 4;
+  const size_t lds = (size_t)(C + cfg->rot_dims) * 4;
   const int nq = cfg->heads * cfg->dim, nk = cfg->kv_heads * cfg->dim, nv = cfg->kv_heads * cfg->vdim;
   const bool vec = taps >= 2 && taps <= 4 && nq % 4 == 0 && nk % 4 == 0 && nv % 4 == 0 && ldp % 4 == 0 && aligned16(d_proj) &&
                    aligned16(d_conv_w) && aligned16(d_conv_state) && (!d_bias || aligned16(d_bias)) && (!d_q_norm_w || aligned16(d_q_norm_w)) &&
-                   (!d_k_norm_w || aligned16(d_k_norm_w)) && aligned16(d_q_out) && aligned16(d_kcache) && aligned16(d_vcache);
+                   (!d_k_norm_w || aligned16(d_k_norm_w)) && aligned16(d_q_out) && aligned16(d_kcache) && aligned16(d_vcache) &&
+                   (cfg->rot_dims == 0 || cfg->dim % 4 == 0);
   if (vec) {
     const int one = max_q_len == 1 ? 1 : 0;
 #define KTX_CP_GO(KT, TAPS)                                                                                                          \
   do {                                                                                                                               \
     KTX_HIP(ktx_set_max_lds((const void*)swa_conv_prep_vec_kernel<KT, TAPS>, 150 * 1024));                                           \
     swa_conv_prep_vec_kernel<KT, TAPS><<<T, 256, lds, st>>>(*cfg, d_proj, ldp, d_bias, d_conv_w, d_q_norm_w, d_k_norm_w, d_q_indptr,  \
-                                                            d_pos0, d_slot, d_tok_req, d_conv_state, one, d_cache_loc, (KT*)d_kcache, \
+                                                            d_pos0, d_slot, d_tok_req, d_conv_state, one, d_inv_freq, d_cache_loc, (KT*)d_kcache, \
                                                             (KT*)d_vcache, d_q_out);                                                 \
   } while (0)
 #define KTX_CP_TAPS(KT)               \
@@ -1202,11 +1219,11 @@ int ktx_swa_conv_prep(const ktx_swa_config* cfg, int B, int T, int max_q_len, in
   if (cfg->cache_dtype == KTX_SEQ_F32) {
     KTX_HIP(ktx_set_max_lds((const void*)swa_conv_prep_kernel<float>, 150 * 1024));
     swa_conv_prep_kernel<float><<<T, 256, lds, st>>>(*cfg, taps, d_proj, ldp, d_bias, d_conv_w, d_q_norm_w, d_k_norm_w, d_q_indptr, d_pos0,
-                                                     d_slot, d_tok_req, d_conv_state, d_cache_loc, (float*)d_kcache, (float*)d_vcache, d_q_out);
+                                                     d_slot, d_tok_req, d_conv_state, d_inv_freq, d_cache_loc, (float*)d_kcache, (float*)d_vcache, d_q_out);
   } else {
     KTX_HIP(ktx_set_max_lds((const void*)swa_conv_prep_kernel<bf16_t>, 150 * 1024));
     swa_conv_prep_kernel<bf16_t><<<T, 256, lds, st>>>(*cfg, taps, d_proj, ldp, d_bias, d_conv_w, d_q_norm_w, d_k_norm_w, d_q_indptr, d_pos0,
-                                                      d_slot, d_tok_req, d_conv_state, d_cache_loc, (bf16_t*)d_kcache, (bf16_t*)d_vcache,
+                                                      d_slot, d_tok_req, d_conv_state, d_inv_freq, d_cache_loc, (bf16_t*)d_kcache, (bf16_t*)d_vcache,
                                                       d_q_out);
   }
   KTX_HIP(hipGetLastError());

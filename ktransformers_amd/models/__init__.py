@@ -89,6 +89,17 @@ def _vigodra_cache(config, max_tokens, max_requests, dtype, device):
     return KHybridCache(vigodra_layer_specs(config), max_tokens, max_requests=max_requests, dtype=dtype, device=device)
 
 
+def _dunusun_config(d, dtype):
+    from ktransformers_amd.models.modeling_dunusun import make_dunusun_config
+    return make_dunusun_config(d, dtype)
+
+
+def _dunusun_cache(config, max_tokens, max_requests, dtype, device):
+    from ktransformers_amd.models.custom_cache import KHybridCache
+    from ktransformers_amd.models.modeling_dunusun import dunusun_layer_specs
+    return KHybridCache(dunusun_layer_specs(config), max_tokens, max_requests=max_requests, dtype=dtype, device=device)
+
+
 def _cls(module: str, name: str):
     def get():
         import importlib
@@ -111,6 +122,8 @@ MODEL_REGISTRY = {
                           _sadosun_cache, dtypes=(torch.bfloat16, torch.float32)),
     "Vigodra": ModelEntry(_vigodra_config, _cls("ktransformers_amd.models.modeling_vigodra", "VigodraForCausalLM"), "Vigodra.yaml",
                           _vigodra_cache, dtypes=(torch.bfloat16, torch.float32)),
+    "Dunusun": ModelEntry(_dunusun_config, _cls("ktransformers_amd.models.modeling_dunusun", "DunusunForCausalLM"), "Dunusun.yaml",
+                          _dunusun_cache, dtypes=(torch.bfloat16, torch.float32)),
 }
 
 

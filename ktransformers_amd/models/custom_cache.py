@@ -178,6 +178,7 @@ class KHybridCache:
                                  fp32) for grouped-query attention, stored as the attention reads them (rotated, normed);
       "rec": (heads, dim, vdim)   — fp32 state slots S [slots, heads, dim, vdim], n [slots, heads, dim], m [slots, heads] (mLSTM);
       "delta": (heads, dim, vdim) — fp32 state slots S alone (delta rule);
+      "decay": (heads, dim, vdim) — fp32 state slots S alone (gated linear attention, the state-space-dual scan);
       "ssm": (channels, state)    — fp32 state slots S [slots, channels, state] (selective scan);
       "conv": (channels, taps)    — fp32 slots [slots, taps - 1, channels]: the inputs a short causal convolution still needs;
       "pre": [(channels, taps), ...] — the same kind of slots for convolutions on what the layer's sublayers read, one per sublayer
@@ -203,9 +204,9 @@ class KHybridCache:
         self.v_caches, self.pre_conv = [], []
         for spec in self.layer_specs:
             a, r, lat, dl, cv = spec.get("attn"), spec.get("rec"), spec.get("latent"), spec.get("delta"), spec.get("conv")
-            kv, ssm = spec.get("kv"), spec.get("ssm")
-            if sum(1 for s_ in (r, dl, ssm) if s_) > 1:
-                raise ValueError("KHybridCache: a layer run has one recurrent state (\"rec\", \"delta\" or \"ssm\")")
+            kv, ssm, dec = spec.get("kv"), spec.get("ssm"), spec.get("decay")
+            if sum(1 for s_ in (r, dl, ssm, dec) if s_) > 1:
+                raise ValueError("KHybridCache: a layer run has one recurrent state (\"rec\", \"delta\", \"decay\" or \"ssm\")")
             if a and kv:
                 raise ValueError("KHybridCache: a layer run has one key cache (\"attn\" or \"kv\")")
             self.v_caches.append(torch.zeros((rows, kv[0], kv[2]), dtype=dtype, device=self.device) if kv else None)
@@ -219,7 +220,7 @@ class KHybridCache:
             self.lat_caches.append(torch.zeros((rows, int(lat)), dtype=dtype, device=self.device) if lat else None)
             self.conv.append(torch.zeros((self.max_requests, cv[1] - 1, cv[0]), dtype=torch.float32, device=self.device)
                              if cv and cv[1] > 1 else None)
-            r = r or dl or ssm
+            r = r or dl or dec or ssm
             self.S.append(torch.zeros((self.max_requests,) + tuple(r), dtype=torch.float32, device=self.device) if r else None)
             r = spec.get("rec")
             self.n.append(torch.zeros((self.max_requests, r[0], r[1]), dtype=torch.float32, device=self.device) if r else None)

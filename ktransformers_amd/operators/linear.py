@@ -338,13 +338,15 @@ class KTransformersLinear(BaseInjectedModule):
 class KLinearDense(BaseInjectedModule):
     """A bias-free linear of ANY shape in bf16 or fp32 (config.compute_dtype) whose checkpoint tensor is the module's key itself:
     include/ktx_seq.h `ktx_dense_gemm` (bf16 or fp32 MFMA, fp32 accumulation, fp32 result).  The language-model head of the
-    fp32-residual decoders; KLinearTorch / KLinearMarlin keep serving the quantised families."""
+    fp32-residual decoders; KLinearTorch / KLinearMarlin keep serving the quantised families.  When the replaced module names a
+    `soft_cap` c, the results end as c tanh(. / c), in the product's epilogue."""
 
     def __init__(self, key: str, gguf_loader, config, orig_module: nn.Module, prefill_device: str = "cuda", generate_device: str = "cuda",
                  weight_suffix: str = "", **kwargs):
         BaseInjectedModule.__init__(self, key, gguf_loader, config, orig_module, prefill_device, generate_device, **kwargs)
         object.__setattr__(self, "compute_dtype", getattr(config, "compute_dtype", torch.bfloat16))
         object.__setattr__(self, "weight_suffix", weight_suffix)
+        object.__setattr__(self, "soft_cap", getattr(orig_module, "soft_cap", None))
         object.__setattr__(self, "w", {})
 
     def load(self):
@@ -352,6 +354,8 @@ class KLinearDense(BaseInjectedModule):
 
     def forward(self, x: torch.Tensor) -> torch.Tensor:
         from ktransformers_amd._native_seq import dense_gemm
+        if self.soft_cap:
+            return dense_gemm(x.reshape(-1, x.shape[-1]), self.w["w"], act="soft_cap", act_arg=self.soft_cap)
         return dense_gemm(x.reshape(-1, x.shape[-1]), self.w["w"])
 
 
@@ -388,4 +392,13 @@ class KLinearRider(BaseInjectedModule):
 def merged_input_weight(own: list, rider) -> torch.Tensor:
     """[own_0 ; own_1 ; ... ; rider.w] as one contiguous [rows, in] weight: all products of one input in one GEMM."""
     parts = list(own) + ([rider.w["w"]] if rider is not None else [])
+    return torch.cat(parts).contiguous()
+
+
+def padded_rows(parts: list, multiple: int = 8) -> torch.Tensor:
+    """The given weights' rows as one contiguous [rows, in] weight, filled up with zero rows to a multiple of `multiple`: the product's fp32 rows
+    then start 16-byte aligned, and the tuned GEMM (whole groups of 8 columns) takes them."""
+    rows = sum(p.shape[0] for p in parts)
+    fill = -rows % multiple
+    parts = list(parts) + ([parts[0].new_zeros((fill, parts[0].shape[1]))] if fill else [])
     return torch.cat(parts).contiguous()

@@ -102,8 +102,8 @@ kDeepseekV3MLP = KDeepseekV3MLP
 
 
 class KDenseMLP(BaseInjectedModule):
-    """Two-matrix feed-forward W_down act(W_up h) on an fp32 residual stream (act = tanh-form GELU, applied in the epilogue of the up
-    GEMM: include/ktx_seq.h `ktx_dense_gemm`).  With the decoder layer's fusion hooks the post-norm and the residual add ride in
+    """Two-matrix feed-forward W_down act(W_up h) on an fp32 residual stream (act = tanh-form GELU, or "relu_sq": relu(z)^2, applied in
+    the epilogue of the up GEMM: include/ktx_seq.h `ktx_dense_gemm_act`).  With the decoder layer's fusion hooks the post-norm and the residual add ride in
     one `ktx_rms_combine` launch behind the down GEMM.  Checkpoint tensors: `<key>.up` [ff, width], `<key>.down` [width, ff]."""
     SUPPORTS_FUSION = True
 

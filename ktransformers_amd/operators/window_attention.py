@@ -24,14 +24,19 @@ Further options, each off unless the replaced module names it:
     dist_far              a learned bias by distance is added to the scaled score, `<key>.rel` [rows, heads]: distances below rows / 2
                           have a row each, the rest share rows on a logarithmic scale that reaches the last row at distance dist_far;
     keep_first            the sequence's first positions stay visible behind the window;
-    sink = "learned"      the sink's score is `<key>.sink` [heads].
-With any of the first three the prep is `ktx_swa_conv_prep` (no rotation in that form)."""
+    sink = "learned"      the sink's score is `<key>.sink` [heads];
+    softcap               the scaled score becomes softcap tanh(score / softcap);
+    gated                 the concatenated heads are multiplied by sigmoid(W_g h) (`<key>.g`) in front of W_o (include/ktx_gla.h `ktx_gate_segments`).
+With any of the first three the prep is `ktx_swa_conv_prep` (q and k turn behind the convolution there; values do not turn, and turning
+heads are not normed).  Inside a parallel mixer (operators/mixers.py) the input projections and the output product are shared with the
+other mixer's (`in_weight_names`, `gated_segment`)."""
 from __future__ import annotations
 
 import torch
 from torch import nn
 
 from ktransformers_amd.operators.base_operator import BaseInjectedModule
+from ktransformers_amd.operators.linear import padded_rows
 
 
 class KWindowGQAttention(BaseInjectedModule):
@@ -47,11 +52,11 @@ class KWindowGQAttention(BaseInjectedModule):
                      "eps", "width"):
             object.__setattr__(self, name, getattr(o, name))
         for name, default in (("qkv_bias", False), ("out_bias_on", False), ("conv_taps", 0), ("proj_norm", False), ("dist_far", None),
-                              ("keep_first", 0), ("sink", None)):
+                              ("keep_first", 0), ("sink", None), ("softcap", None), ("gated", False)):
             object.__setattr__(self, name, getattr(o, name, default))
         object.__setattr__(self, "conv_form", bool(self.qkv_bias or self.conv_taps or self.proj_norm))
-        if self.conv_form and (self.rot_dims or self.rot_values or self.qk_norm):
-            raise ValueError(f"{key}: biases, a convolution or whole-projection norms go with un-rotated, un-normed heads")
+        if self.conv_form and (self.rot_values or self.qk_norm or (self.rot_dims and self.proj_norm)):
+            raise ValueError(f"{key}: biases, a convolution or whole-projection norms go with un-normed heads and values that do not turn")
         object.__setattr__(self, "compute_dtype", getattr(config, "compute_dtype", torch.bfloat16))
         object.__setattr__(self, "w", {})
         object.__setattr__(self, "_cfg", {})
@@ -61,6 +66,14 @@ class KWindowGQAttention(BaseInjectedModule):
         if self.conv_taps > 1:
             spec["conv"] = (self.heads * self.dim + self.kv_heads * (self.dim + self.vdim), self.conv_taps)
         return spec
+
+    def in_weight_names(self):
+        H, G, D, V = self.heads, self.kv_heads, self.dim, self.vdim
+        return [("qkv", H * D + G * (D + V))] + ([("g", H * V)] if self.gated else [])
+
+    @property
+    def out_columns(self) -> int:
+        return self.heads * self.vdim
 
     @property
     def out_bias(self):
@@ -86,6 +99,10 @@ class KWindowGQAttention(BaseInjectedModule):
                 tuple(o.shape) != (self.width, H * V):
             raise ValueError(f"{self.key}: tensor shapes do not fit heads={H} kv_heads={G} dim={D} vdim={V} width={self.width}")
         self.w.update(qkv=torch.cat([q, k, v]).contiguous(), o=o.contiguous())
+        if self.gated:
+            self.w["g"] = get("g").contiguous()
+            if tuple(self.w["g"].shape) != (H * V, self.width):
+                raise ValueError(f"{self.key}.g: expected {(H * V, self.width)}, got {tuple(self.w['g'].shape)}")
         f64 = lambda n: torch.pow(torch.tensor(float(self.rot_base), dtype=torch.float64),
                                   -2.0 * torch.arange(n // 2, dtype=torch.float64) / max(n, 1)).to(dev)
         self.w["inv_freq"] = f64(self.rot_dims) if self.rot_dims else None
@@ -121,20 +138,36 @@ class KWindowGQAttention(BaseInjectedModule):
         if k not in self._cfg:
             self._cfg[k] = swa_config(self.heads, self.kv_heads, self.dim, self.vdim, self.rot_dims, self.rot_values, self.qk_norm,
                                       self.eps, self.scale, self.window or 0, cache.page_size, cache.dtype, keep_first=self.keep_first,
-                                      bias_span=0 if self.w["dist_bias"] is None else self.w["dist_bias"].shape[0] - 1)
+                                      bias_span=0 if self.w["dist_bias"] is None else self.w["dist_bias"].shape[0] - 1, softcap=self.softcap)
         return self._cfg[k]
 
     def forward(self, h: torch.Tensor, batch, cache, cache_idx: int) -> torch.Tensor:
         """h [T, width] in the compute type -> W_o(attention) fp32 [T, width]; the step's key and value rows are appended to the cache."""
+        from ktransformers_amd._native_gla import gate_segments
         from ktransformers_amd._native_seq import dense_gemm
+        if not self.gated:
+            return dense_gemm(self.attend(dense_gemm(h, self.w["qkv"]), batch, cache, cache_idx), self.w["o"])
+        if "in" not in self.w:
+            self.w["in"] = padded_rows([self.w["qkv"], self.w["g"]])
+        seg, _keep = self.gated_segment(dense_gemm(h, self.w["in"]), 0, batch, cache, cache_idx)
+        return dense_gemm(gate_segments([seg], h.shape[0], h.device, out_dtype=self.compute_dtype), self.w["o"])
+
+    def gated_segment(self, proj: torch.Tensor, base: int, batch, cache, cache_idx: int, scale: float = 1.0):
+        """proj fp32 rows with q | k | v | g from column `base`: the attention, and the segment of gate_segments that gates its heads."""
+        from ktransformers_amd._native_gla import gate_seg
+        (_, n_qkv), (_, n_g) = self.in_weight_names()
+        o = self.attend(proj[:, base:base + n_qkv], batch, cache, cache_idx)
+        return gate_seg(o, proj[:, base + n_qkv:base + n_qkv + n_g], "sigmoid", scale=scale), o
+
+    def attend(self, proj: torch.Tensor, batch, cache, cache_idx: int) -> torch.Tensor:
+        """proj fp32 rows with q | k | v at column 0 -> the concatenated heads [T, heads * vdim] in the compute type (no gate, no W_o)."""
         from ktransformers_amd._native_swa import swa_conv_prep, swa_forward, swa_mfma, swa_mfma_eligible, swa_prep
         H, G, D = self.heads, self.kv_heads, self.dim
-        cfg, T = self._config(cache), h.shape[0]
+        cfg, T = self._config(cache), proj.shape[0]
         kc, vc = cache.k_caches[cache_idx], cache.v_caches[cache_idx]
-        proj = dense_gemm(h, self.w["qkv"])
         if self.conv_form:
             q, vcs = swa_conv_prep(cfg, proj, self.w.get("qkv_b"), self.w.get("conv"), self.w.get("q_norm"), self.w.get("k_norm"), batch,
-                                   cache.conv[cache_idx] if self.conv_taps > 1 else None, kc, vc), None
+                                   cache.conv[cache_idx] if self.conv_taps > 1 else None, kc, vc, inv_freq=self.w["inv_freq"]), None
         else:
             q, vcs = swa_prep(cfg, proj, 0, H * D, (H + G) * D, self.w["inv_freq"], self.w["v_inv_freq"], batch.positions, batch.cache_loc, kc, vc)
         bias = self.w["dist_bias"]
@@ -147,4 +180,4 @@ class KWindowGQAttention(BaseInjectedModule):
             span = batch.max_kv_len if not self.window else min(batch.max_kv_len, self.window + self.keep_first)
             nsplit = max(1, min(self.TARGET_WORKGROUPS // max(T * G, 1), (span + self.KEYS_PER_SPLIT - 1) // self.KEYS_PER_SPLIT))
             o = swa_forward(cfg, q, kc, vc, batch, self.w["sink"], vcs, nsplit=nsplit, out_dtype=self.compute_dtype, dist_bias=bias)
-        return dense_gemm(o, self.w["o"])
+        return o

@@ -19,7 +19,10 @@ PAIRS = [("ktx_moe_config", "_MoeConfig", "ktx_moe.h"), ("ktx_linear_config", "_
          ("ktx_delta_config", "_DeltaConfig", "ktx_hyb.h"), ("ktx_latattn_config", "_LatAttnConfig", "ktx_hyb.h"),
          ("ktx_postnorm_args", "_PostNormArgs", "ktx_hyb.h"),
          ("ktx_resid_args", "_ResidArgs", "ktx_swa.h"), ("ktx_swa_config", "_SwaConfig", "ktx_swa.h"),
-         ("ktx_ssm_config", "_SsmConfig", "ktx_swa.h")]
+         ("ktx_ssm_config", "_SsmConfig", "ktx_swa.h"),
+         # (ktransformers_amd/_native_gla.py)
+         ("ktx_hyper_args", "_HyperArgs", "ktx_gla.h"), ("ktx_decay_scan_args", "_DecayScanArgs", "ktx_gla.h"),
+         ("ktx_gate_seg", "_GateSeg", "ktx_gla.h")]
 
 
 @pytest.fixture(scope="module")
@@ -28,11 +31,11 @@ def native():
         from ktransformers_amd import _native
     except ImportError as e:          # the library is built by __graft_entry__.build(); without it there is nothing to mirror
         pytest.skip(f"libktx_hip.so not built: {e}")
-    from ktransformers_amd import _native_hyb, _native_seq, _native_swa
+    from ktransformers_amd import _native_gla, _native_hyb, _native_seq, _native_swa
 
     class Both:
         def __getattr__(self, name):
-            for mod in (_native, _native_seq, _native_hyb, _native_swa):
+            for mod in (_native, _native_seq, _native_hyb, _native_swa, _native_gla):
                 if hasattr(mod, name):
                     return getattr(mod, name)
             raise AttributeError(name)
