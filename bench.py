@@ -1940,11 +1940,7 @@ def run_pilavik(args, dev):
         res["decode_bs1"]["frac_of_hbm_peak"] = round(active * 2 / (res["decode_bs1"]["ms_per_step"] * 1e-3) / (HBM_PEAK_GBS * 1e9), 4)
         try:
             ms_ = MITOTAR_SIZES[sz["mitotar"]]
-            layer = {"type": "parallel", "mlp": {"kind": "dense", "ff": ms_["ff"]},
-                     "mixer": {"left": {"heads": ms_["heads"], "kv_heads": ms_["kv_heads"], "dim": ms_["dim"], "vdim": ms_["dim"],
-                                        "scale": ms_["dim"] ** -0.5, "q_temp": {"coef": 0.4, "every": 128}},
-                               "right": {"heads": ms_["r_heads"], "dim": ms_["r_dim"], "vdim": ms_["r_vdim"], "gate_cap": 15.0}}}
-            mcfg = {"architecture": "Mitotar", "width": ms_["width"], "vocab": 32000, "norm": {"eps": 1e-5}, "layers": [layer] * n_layers}
+            mcfg = mitotar_config(ms_, n_layers)
             res["mitotar"] = measure(mcfg, SeqRandomLoader(mcfg, dev), SeqKernelTimer, 0)
         except Exception as e:      # the comparison must not lose the new family's numbers
             res["mitotar"] = {"error": f"{type(e).__name__}: {e}"}
@@ -2260,6 +2256,166 @@ def run_vigodra(args, dev):
     print(json.dumps(line), flush=True)
 
 
+# ---------------------------------------------------------------------------------------------------------------------
+# --dunusun: the hyper-connected family whose layers run a soft-capped grouped-query attention beside a gated linear attention, or a
+# state-space-dual scan (models/modeling_dunusun.py), at a few layer sizes, beside Mitotar — the closest existing family: two mixers side
+# by side (full causal attention and a matrix-state recurrence of the same sizes), two-matrix feed-forwards, the same fp32 residual, cache
+# manager, step function and graph replay — at equal width and depth; and Sadosun, whose selective scan is the like of the scan layers
+# ---------------------------------------------------------------------------------------------------------------------
+DUNUSUN_SIZES = {
+    # per block of 4 layers: parallel, parallel, scan, parallel; dense feed-forwards; head sizes and states of the parallel layers = MITOTAR_SIZES
+    "w1024": dict(streams=4, rank=16, ssd_vdim=64, ssd_state=128, ssd_groups=1, mitotar="w1024", sadosun="w1024"),
+    "w2048": dict(streams=4, rank=16, ssd_vdim=64, ssd_state=128, ssd_groups=2, mitotar="w2048", sadosun="w2048"),
+    "w4096": dict(streams=4, rank=16, ssd_vdim=64, ssd_state=128, ssd_groups=4, mitotar="w4096", sadosun="w4096"),
+}
+
+
+def mitotar_config(ms_, n_layers, vocab=32000):
+    layer = {"type": "parallel", "mlp": {"kind": "dense", "ff": ms_["ff"]},
+             "mixer": {"left": {"heads": ms_["heads"], "kv_heads": ms_["kv_heads"], "dim": ms_["dim"], "vdim": ms_["dim"],
+                                "scale": ms_["dim"] ** -0.5, "q_temp": {"coef": 0.4, "every": 128}},
+                       "right": {"heads": ms_["r_heads"], "dim": ms_["r_dim"], "vdim": ms_["r_vdim"], "gate_cap": 15.0}}}
+    return {"architecture": "Mitotar", "width": ms_["width"], "vocab": vocab, "norm": {"eps": 1e-5}, "layers": [layer] * n_layers}
+
+
+def dunusun_config(sz, n_layers, vocab=32000):
+    ms_ = MITOTAR_SIZES[sz["mitotar"]]
+    mlp = {"kind": "dense", "ff": ms_["ff"]}
+    par = {"type": "parallel", "mlp": mlp,
+           "mixer": {"left": {"heads": ms_["heads"], "kv_heads": ms_["kv_heads"], "dim": ms_["dim"], "vdim": ms_["dim"], "conv": 4,
+                              "scale": ms_["dim"] ** -0.5, "softcap": 30.0, "rot": {"base": 10000.0, "dims": ms_["dim"] // 2}},
+                     "right": {"heads": ms_["r_heads"], "dim": ms_["r_dim"], "vdim": ms_["r_vdim"], "tau": 16.0},
+                     "left_scale": 0.7, "right_scale": 0.7}}
+    inner = 2 * ms_["width"]
+    ssd = {"type": "mamba2", "mlp": mlp, "mixer": {"heads": inner // sz["ssd_vdim"], "vdim": sz["ssd_vdim"], "state": sz["ssd_state"],
+                                                   "groups": sz["ssd_groups"], "conv": 4, "norm_groups": sz["ssd_groups"]}}
+    return {"architecture": "Dunusun", "width": ms_["width"], "vocab": vocab, "norm": {"eps": 1e-5}, "streams": sz["streams"], "loop": None,
+            "logit_softcap": 30.0, "layers": [(par, par, ssd, par)[i % 4] for i in range(n_layers)], "_rank": sz["rank"]}
+
+
+class GlaRandomLoader(HybRandomLoader):
+    """Random bf16 weights by tensor name for a Dunusun config (names and shapes of models/modeling_dunusun.py's checkpoint)."""
+
+    def __init__(self, cfg, dev):
+        self.dev, self.tensor_device_map, self.shapes = dev, {}, {}
+        W, S, n = cfg["width"], self.shapes, cfg["streams"]
+        S.update({"embed": (cfg["vocab"], W), "head": (cfg["vocab"], W), "final.norm": (W,), "final.norm.b": (W,)})
+        for i, L in enumerate(cfg["layers"]):
+            p, m, c = f"l{i}.", L["mixer"], L.get("mlp")
+            for q in (1, 2) if c else (1,):
+                S.update({p + f"norm{q}": (W,), p + f"norm{q}.b": (W,), p + f"hc{q}.in": (n,), p + f"hc{q}.out": (n,), p + f"hc{q}.mix": (n, n)})
+            if L["type"] == "parallel":
+                a, r, R = m["left"], m["right"], cfg["_rank"]
+                H, G, D, V, K = a["heads"], a["kv_heads"], a["dim"], a["vdim"], a["conv"]
+                for t, rows in (("q", H * D), ("k", G * D), ("v", G * V)):
+                    S.update({p + f"mix.left.{t}": (rows, W), p + f"mix.left.{t}.conv": (rows, K)})
+                S.update({p + "mix.left.g": (H * V, W), p + "mix.left.o": (W, H * V)})
+                h, d, v = r["heads"], r["dim"], r["vdim"]
+                for t, rows in (("q", h * d), ("k", h * d), ("v", h * v), ("g", h * v), ("a1", R)):
+                    S[p + f"mix.right.{t}"] = (rows, W)
+                S.update({p + "mix.right.a2": (h * d, R), p + "mix.right.a2.b": (h * d,), p + "mix.right.norm": (v,), p + "mix.right.o": (W, h * v)})
+            else:
+                h, v, N, G, K = m["heads"], m["vdim"], m["state"], m["groups"], m["conv"]
+                I, C = h * v, h * v + 2 * G * N
+                S.update({p + "mix.in": (I + C + h, W), p + "mix.conv": (C, K), p + "mix.conv.b": (C,), p + "mix.dt_bias": (h,), p + "mix.A_log": (h,),
+                          p + "mix.D": (h,), p + "mix.norm": (I,), p + "mix.o": (W, I)})
+            if c:
+                S.update({p + "mlp.up": (c["ff"], W), p + "mlp.down": (W, c["ff"])})
+
+    def load_tensor(self, name, device="cpu"):
+        shape = self.shapes[name]
+        t = super().load_tensor(name, device)
+        leaf = name.rsplit(".", 1)[-1]
+        if leaf in ("in", "out") and ".hc" in name:
+            return t.mul_(0.1).add_(1.0 / shape[0] if leaf == "in" else 1.0)
+        if leaf == "mix" and ".hc" in name:
+            return t.mul_(0.1).add_(torch.eye(shape[0], device=self.dev, dtype=torch.bfloat16))
+        return t
+
+
+class GlaKernelTimer(SwaKernelTimer):
+    """HIP events around every binding a Dunusun step calls."""
+    HYB, SWA, SEQ = (), ("swa_conv_prep", "swa_forward", "swa_mfma"), ("embed_rows", "dense_gemm")
+    GLA = ("hyper_mix", "lowrank_decay", "ssd_prep", "decay_scan", "gate_segments")
+
+    def _cost(self, name, a, kw, out):
+        nb = lambda t: t.numel() * t.element_size() if isinstance(t, torch.Tensor) else 0
+        if name == "hyper_mix":
+            w = kw.get("write")
+            return name, 0.0, nb(a[0]) + nb(kw.get("out")) + (nb(w[0]) if w is not None else 0) + nb(out)
+        if name == "decay_scan":
+            S, T = a[5], a[0].shape[0]
+            H, D, V = S.shape[1:]
+            label = f"decay_scan {'per head' if a[3].shape[1] == H else 'per channel'}"
+            return label, 5.0 * T * H * D * V, 2.0 * a[4].B * H * D * V * 4 + sum(nb(t) for t in a[:4]) + nb(out)
+        if name == "gate_segments":
+            return name, 0.0, 3 * nb(out)
+        if name == "swa_conv_prep":
+            return name, 0.0, nb(a[1]) + nb(out) + out.shape[0] * (a[0].kv_heads * (a[0].dim + a[0].vdim)) * 2
+        return super()._cost(name, a, kw, out)
+
+    def __enter__(self):
+        from ktransformers_amd import _native_gla
+        super().__enter__()
+        for name in self.GLA:
+            fn = getattr(_native_gla, name)
+            self.saved[(_native_gla, name)] = fn
+
+            def wrapped(*a, _fn=fn, _name=name, **kw):
+                e0, e1 = torch.cuda.Event(enable_timing=True), torch.cuda.Event(enable_timing=True)
+                e0.record()
+                out = _fn(*a, **kw)
+                e1.record()
+                self.rows.append((e0, e1) + self._cost(_name, a, kw, out))
+                return out
+            setattr(_native_gla, name, wrapped)
+        return self
+
+
+def run_dunusun(args, dev):
+    """Prefill (one prompt of --prefill-tokens) and decode (batch 1 and 8 at a 2048-token context) throughput of Dunusun at
+    DUNUSUN_SIZES, each beside Mitotar and Sadosun of equal width and depth, with a per-kernel table and the fraction of its roofline (bf16
+    MFMA peak or HBM peak, whichever bounds).  Random weights, synthetic tokens.  Prints one JSON line; the whole record goes to
+    bench_dunusun.json beside this file."""
+    n_layers, T, ctx = args.layers or 4, args.prefill_tokens, 2048
+    sizes = [s for s in (args.dunusun.split(",") if args.dunusun != "all" else DUNUSUN_SIZES) if s in DUNUSUN_SIZES]
+    record = {"metric": "dunusun_prefill_decode", "unit": "tok/s", "layers": n_layers, "prefill_tokens": T, "decode_ctx": ctx,
+              "dtype": "bf16 weights / activations / key and value caches, fp32 residual streams, norms, scores, state", "data": "synthetic",
+              "sizes": {}}
+    for name in sizes:
+        sz = DUNUSUN_SIZES[name]
+        cfg = dunusun_config(sz, n_layers)
+        loader = GlaRandomLoader(cfg, dev)
+        res = family_measure(args, dev, cfg, loader, GlaKernelTimer, 0, T, ctx)
+        active = loader.active_params(cfg)
+        res["weights_GB"] = res["active_weights_GB"] = round(active * 2 / 1e9, 3)
+        res["decode_bs1"]["frac_of_hbm_peak"] = round(active * 2 / (res["decode_bs1"]["ms_per_step"] * 1e-3) / (HBM_PEAK_GBS * 1e9), 4)
+        for other in ("mitotar", "sadosun"):
+            try:
+                if other == "mitotar":
+                    ocfg = mitotar_config(MITOTAR_SIZES[sz["mitotar"]], n_layers)
+                    ol = SeqRandomLoader(ocfg, dev)
+                    res[other] = family_measure(args, dev, ocfg, ol, SeqKernelTimer, 0, T, ctx)
+                    res[other]["active_weights_GB"] = round(sum(math.prod(v) for k, v in ol.shapes.items() if k != "embed") * 2 / 1e9, 3)
+                else:
+                    ssz = SADOSUN_SIZES[sz["sadosun"]]
+                    ocfg = sadosun_config(ssz, n_layers)
+                    ol = SwaRandomLoader(ocfg, dev)
+                    res[other] = family_measure(args, dev, ocfg, ol, SwaKernelTimer, ssz["window"], T, ctx)
+            except Exception as e:      # the comparison must not lose the new family's numbers
+                res[other] = {"error": f"{type(e).__name__}: {e}"}
+        record["sizes"][name] = res
+        log(f"[dunusun] {name}: prefill {res['prefill']['tok_s']} tok/s, decode bs1 {res['decode_bs1']['tok_s']} tok/s, "
+            f"bs8 {res['decode_bs8']['tok_s']} tok/s")
+    with open(os.path.join(ROOT, "bench_dunusun.json"), "w") as f:
+        json.dump(record, f, indent=1)
+    line = {"metric": record["metric"], "unit": "tok/s", "layers": n_layers, "data": "synthetic",
+            "sizes": {k: {"prefill": v["prefill"]["tok_s"], "decode_bs1": v["decode_bs1"]["tok_s"], "decode_bs8": v["decode_bs8"]["tok_s"],
+                          **{f"{o}_{w}": v[o].get(w, {}).get("tok_s") for o in ("mitotar", "sadosun") for w in ("prefill", "decode_bs1", "decode_bs8")}}
+                      for k, v in record["sizes"].items()}}
+    print(json.dumps(line), flush=True)
+
+
 def main():
     ap = argparse.ArgumentParser()
     ap.add_argument("--gpus", type=int, default=1)
@@ -2313,6 +2469,11 @@ def main():
                          "depth-weighted average, biased grouped-query window attention behind convolved projections, gated latent window "
                          "attention with shared latent rows, a bounded GLU) at layer sizes from VIGODRA_SIZES (comma-separated, or 'all'), "
                          "beside Sadosun of equal width and depth; one JSON line, detail in bench_vigodra.json")
+    ap.add_argument("--dunusun", default="", metavar="SIZES",
+                    help="instead of the default workload: prefill / decode throughput of the Dunusun family (hyper-connected residual streams, "
+                         "soft-capped grouped-query attention beside gated linear attention, a state-space-dual scan, relu^2 feed-forwards) at "
+                         "layer sizes from DUNUSUN_SIZES (comma-separated, or 'all'), beside Mitotar and Sadosun of equal width and depth; one "
+                         "JSON line, detail in bench_dunusun.json")
     ap.add_argument("--pmc-child", action="store_true", help=argparse.SUPPRESS)
     ap.add_argument("--trace-child", action="store_true", help=argparse.SUPPRESS)
     args = ap.parse_args()
@@ -2346,6 +2507,10 @@ def main():
     if args.vigodra:
         torch.cuda.set_device(dev)
         run_vigodra(args, dev)
+        return
+    if args.dunusun:
+        torch.cuda.set_device(dev)
+        run_dunusun(args, dev)
         return
     torch.cuda.set_device(dev)
     if args.pmc_child:
