@@ -1528,8 +1528,16 @@ class SeqKernelTimer:
             return name, 4.0 * pairs * cfg.heads * cfg.dim, keys * (gd * kc.element_size() + 4 * cfg.kv_heads) + nb(a[1]) + nb(out)
         if name == "mlstm_forward":
             cfg, S = a[0], a[8]
-            B = a[7].numel()
-            return name, 0.0, 2.0 * B * cfg.heads * cfg.dim * cfg.vdim * 4 + nb(out)
+            B, T = a[7].numel(), a[1].shape[0]
+            qkv = T * cfg.heads * (2 * cfg.dim + cfg.vdim) * 4
+            return name, 5.0 * T * cfg.heads * cfg.dim * cfg.vdim, 2.0 * B * cfg.heads * cfg.dim * cfg.vdim * 4 + qkv + nb(out)
+        if name == "sigattn_prep":          # projections read, folded queries and the step's key rows written
+            cfg, T = a[0], a[1].shape[0]
+            return name, 0.0, 2 * nb(out) + T * cfg.kv_heads * cfg.dim * (4 + a[9].element_size())
+        if name == "mlstm_gate_norm":
+            return name, 0.0, nb(a[1]) * 2 + nb(out)
+        if name in ("embed_sinpos", "embed_rows"):
+            return name, 0.0, out.numel() * a[2 if name == "embed_sinpos" else 1].element_size() + nb(out)
         return name, 0.0, sum(nb(t) for t in a) + nb(out)
 
     def __enter__(self):
@@ -2048,6 +2056,9 @@ class SwaKernelTimer(HybKernelTimer):
             cfg, q, kc, vc = a[0], a[1], a[2], a[3]
             pairs, keys = self.kv_len_of()
             return name, 2.0 * pairs * cfg.heads * (cfg.dim + cfg.vdim), keys * cfg.kv_heads * (cfg.dim + cfg.vdim) * kc.element_size() + nb(q) + nb(out)
+        if name == "swa_prep":              # projections read, queries and the step's key and value rows written
+            cfg, T = a[0], a[1].shape[0]
+            return name, 0.0, 2 * T * cfg.heads * cfg.dim * 4 + T * cfg.kv_heads * (cfg.dim + cfg.vdim) * (4 + a[9].element_size())
         if name == "ssm_scan":
             cfg, xc = a[0], a[1]
             B = a[11].B
@@ -2349,7 +2360,7 @@ class GlaKernelTimer(SwaKernelTimer):
             label = f"decay_scan {'per head' if a[3].shape[1] == H else 'per channel'}"
             return label, 5.0 * T * H * D * V, 2.0 * a[4].B * H * D * V * 4 + sum(nb(t) for t in a[:4]) + nb(out)
         if name == "gate_segments":
-            return name, 0.0, 3 * nb(out)
+            return name, 0.0, nb(out) + sum(a[1] * s.n * (4 + (2 if s.o_dtype else 4)) for s in a[0])
         if name == "swa_conv_prep":
             return name, 0.0, nb(a[1]) + nb(out) + out.shape[0] * (a[0].kv_heads * (a[0].dim + a[0].vdim)) * 2
         return super()._cost(name, a, kw, out)

@@ -169,6 +169,7 @@ def gate_seg(o: torch.Tensor, gate: torch.Tensor, act: str, norm: tuple | None =
     if not o.is_cuda or o.dtype not in SEQ_DTYPE or o.dim() != 2 or o.stride(1) != 1 or tuple(o.shape) != tuple(gate.shape):
         raise KtxError("gate_seg: o must be rows of the gate's shape")
     s = _GateSeg()
+    s.tensors = [o, gate]            # (the struct holds addresses only: the segment keeps what it points to alive)
     s.o, s.ldo, s.o_dtype, s.gate, s.ldg, s.n = o.data_ptr(), o.stride(0), SEQ_DTYPE[o.dtype], gp, ldg, o.shape[1]
     s.act, s.gate_first, s.scale = {"sigmoid": 0, "silu": 1}[act], int(bool(gate_first)), float(scale)
     if norm is not None:
@@ -176,6 +177,7 @@ def gate_seg(o: torch.Tensor, gate: torch.Tensor, act: str, norm: tuple | None =
         _f32(w, "gate_seg norm weight")
         if w.numel() not in (group, o.shape[1]) or o.shape[1] % group:
             raise KtxError("gate_seg: the norm's groups divide the columns, its weight has a group's or all columns' entries")
+        s.tensors.append(w)
         s.w, s.group, s.w_mod, s.eps = w.data_ptr(), int(group), w.numel(), float(eps)
     return s
 

@@ -62,7 +62,7 @@ class KGatedLinearAttention(BaseInjectedModule):
             c += rows
         alpha = lowrank_decay(cols["a1"], self.w["a2_t"], self.w["a2_b"], self.tau)
         o = decay_scan(cols["q"], cols["k"], cols["v"], alpha, batch, cache.S[cache_idx], q_scale=self.dim ** -0.5)
-        return gate_seg(o, cols["g"], "silu", norm=(self.w["norm"], self.vdim, self.eps), scale=scale), o
+        return gate_seg(o, cols["g"], "silu", norm=(self.w["norm"], self.vdim, self.eps), scale=scale)
 
     def forward(self, h: torch.Tensor, batch, cache, cache_idx: int) -> torch.Tensor:
         """h [T, width] in the compute type -> W_o(...) fp32 [T, width]; the slot states of the batch's requests advance in place."""
@@ -70,5 +70,5 @@ class KGatedLinearAttention(BaseInjectedModule):
         from ktransformers_amd._native_seq import dense_gemm
         if "in" not in self.w:       # used on its own: all input projections as one product
             self.w["in"] = padded_rows([self.w[n] for n in self.IN_ORDER])
-        seg, _keep = self.gated_segment(dense_gemm(h, self.w["in"]), 0, batch, cache, cache_idx)
+        seg = self.gated_segment(dense_gemm(h, self.w["in"]), 0, batch, cache, cache_idx)
         return dense_gemm(gate_segments([seg], h.shape[0], h.device, out_dtype=self.compute_dtype), self.w["o"])

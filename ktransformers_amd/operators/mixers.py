@@ -82,6 +82,6 @@ class KScaledParallelMixer(BaseInjectedModule):
         from ktransformers_amd._native_gla import gate_segments
         from ktransformers_amd._native_seq import dense_gemm
         proj = dense_gemm(h, self.w["in"])
-        left, lo = self.orig_module.left.gated_segment(proj, 0, batch, cache, cache_idx, scale=self.scales[0])
-        right, ro = self.orig_module.right.gated_segment(proj, self.w["right_base"], batch, cache, cache_idx, scale=self.scales[1])
+        left = self.orig_module.left.gated_segment(proj, 0, batch, cache, cache_idx, scale=self.scales[0])
+        right = self.orig_module.right.gated_segment(proj, self.w["right_base"], batch, cache, cache_idx, scale=self.scales[1])
         return dense_gemm(gate_segments([left, right], h.shape[0], h.device, out_dtype=self.compute_dtype), self.w["o"])

@@ -149,7 +149,7 @@ class KWindowGQAttention(BaseInjectedModule):
             return dense_gemm(self.attend(dense_gemm(h, self.w["qkv"]), batch, cache, cache_idx), self.w["o"])
         if "in" not in self.w:
             self.w["in"] = padded_rows([self.w["qkv"], self.w["g"]])
-        seg, _keep = self.gated_segment(dense_gemm(h, self.w["in"]), 0, batch, cache, cache_idx)
+        seg = self.gated_segment(dense_gemm(h, self.w["in"]), 0, batch, cache, cache_idx)
         return dense_gemm(gate_segments([seg], h.shape[0], h.device, out_dtype=self.compute_dtype), self.w["o"])
 
     def gated_segment(self, proj: torch.Tensor, base: int, batch, cache, cache_idx: int, scale: float = 1.0):
@@ -157,7 +157,7 @@ class KWindowGQAttention(BaseInjectedModule):
         from ktransformers_amd._native_gla import gate_seg
         (_, n_qkv), (_, n_g) = self.in_weight_names()
         o = self.attend(proj[:, base:base + n_qkv], batch, cache, cache_idx)
-        return gate_seg(o, proj[:, base + n_qkv:base + n_qkv + n_g], "sigmoid", scale=scale), o
+        return gate_seg(o, proj[:, base + n_qkv:base + n_qkv + n_g], "sigmoid", scale=scale)
 
     def attend(self, proj: torch.Tensor, batch, cache, cache_idx: int) -> torch.Tensor:
         """proj fp32 rows with q | k | v at column 0 -> the concatenated heads [T, heads * vdim] in the compute type (no gate, no W_o)."""
