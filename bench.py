@@ -1819,6 +1819,8 @@ class HybKernelTimer(SeqKernelTimer):
             M, K = a[0].shape
             N = a[1].shape[0]
             return f"dense_gemm M={'prompt' if M > 16 else 'decode'}", 2.0 * M * N * K, M * K * a[0].element_size() + nb(a[1]) + nb(out)
+        if name == "embed_rows":
+            return name, 0.0, out.numel() * a[1].element_size() + nb(out)
         if name == "head_gemm":
             G, N, K = a[2].shape
             M = a[0].shape[0]
