@@ -121,6 +121,7 @@ __device__ __forceinline__ float ktx_dpp_f(float v) { return __int_as_float(ktx_
 #define KTX_DPP_QUAD_2301 0x4E
 #define KTX_DPP_ROW_HALF_MIRROR 0x141
 #define KTX_DPP_ROW_MIRROR 0x140
+#define KTX_DPP_ROW_ROR8 0x128
 
 // all-reduce inside each row of 16 lanes (the MFMA column group): every lane gets its row's result
 __device__ __forceinline__ float row16_max(float v) {

@@ -388,6 +388,240 @@ __global__ void __launch_bounds__(1024) decay_scan_kernel(ScanDims c, const int3
     if (vok && (FULL || i < live)) dst[(size_t)(d0 + i) * V + col] = S[i];
 }
 
+// The same scan for prompts on the fp32 matrix cores, SM_T tokens at a time.  Workgroup = (request, chunk) x head x NT / 64 tiles of 16 value
+// columns; a wavefront keeps its columns of the state, all key rows, as the accumulators of v_mfma_f32_16x16x4_f32.  With p_t the product
+// of the decays of the block's tokens up to t and s_t that of the tokens behind t — products of factors that are at most 1: nothing is divided
+// by a decay and nothing overflows —
+//   o_t = (q_t p_t)^T S + sum_{i <= t} A[t][i] v_i,   A[t][i] = m_i sum_d q_td k_id prod_{i < j <= t} a_jd  (+ skip where i = t)
+//   S  <- diag(p_last) S + sum_t (k_t s_t m_t) v_t^T
+// With one decay per head A is a matrix product (key rows dealt out to the wavefronts) times the products of decays; with a decay per key
+// channel it is formed on the vector ALUs, thread = (token i, a slice of the channels) that walks t with k_i's running product.  An accumulator
+// holds rows 4 g + r of a tile in lane group g, register r: with the contraction visiting rows in the order (r, g) it is the next product's
+// operand as it stands.
+constexpr int SM_T = 16, SM_AST = 20, SCAN_MFMA_MIN = 8;
+typedef float f32x4 __attribute__((ext_vector_type(4)));
+
+// v[j] and v[j + N] meet across the lane pairs CTRL joins: a lane keeps the one its bit names
+template <int N, int CTRL>
+__device__ __forceinline__ void fold_pairs(float (&v)[SM_T], bool upper) {
+#pragma unroll
+  for (int j = 0; j < N; j++) {
+    const float give = upper ? v[j] : v[j + N], keep = upper ? v[j + N] : v[j];
+    v[j] = keep + ktx_dpp_f<CTRL>(give);
+  }
+}
+
+template <int DT, int NT, bool PH>
+struct ScanTile {
+  static constexpr int DW = DT * 16, DP = DW + 4;              // row stride: lane groups four rows apart meet different LDS banks
+  static constexpr int RAW_A = PH ? SM_T : SM_T * DP;
+  static constexpr int PARTS = !PH ? 1 : DT < NT / 64 ? DT : NT / 64;      // partial products of A
+  // raw q | k | a | m, then q p | k s m | p_last | A (its parts), and with one decay per head the products of decays
+  static constexpr int QR = 0, KR = SM_T * DP, AR = 2 * SM_T * DP, MR = AR + RAW_A, QP = MR + SM_T, KP = QP + SM_T * DP, PL = KP + SM_T * DP,
+                       AS = PL + DP, RT = AS + PARTS * SM_T * SM_AST, FLOATS = RT + (PH ? SM_T * SM_AST : 0);
+};
+
+template <int DT, int NT, bool PH, bool OUT>
+__global__ void __launch_bounds__(NT, DT == 8 && NT == 256 && !PH && OUT ? 3 : 4) decay_scan_mfma_kernel(ScanDims c, const int32_t* __restrict__ q_indptr, const int32_t* __restrict__ pos0,
+                                                             const int32_t* __restrict__ slot, const float* __restrict__ q,
+                                                             const float* __restrict__ k, const float* __restrict__ v, const float* __restrict__ a,
+                                                             const float* __restrict__ vmul, const float* __restrict__ skip, float* Sg,
+                                                             float* delta, float* __restrict__ o) {
+  typedef ScanTile<DT, NT, PH> L;
+  constexpr int DW = L::DW, DP = L::DP, E = SM_T * DW / NT, SL = NT / SM_T, CPS = DW / SL, VW = CPS >= 4 ? 4 : CPS;
+  extern __shared__ __attribute__((aligned(16))) float lds[];
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, l16 = lane & 15, g = lane >> 4;
+  const int b = blockIdx.x / c.nch, ch = blockIdx.x % c.nch, h = blockIdx.y;
+  const int q1 = q_indptr[b + 1], t0 = q_indptr[b] + ch * c.L, t1 = min(q1, t0 + c.L);
+  if (t0 >= t1 || (!OUT && t1 == q1)) return;      // (the last chunk's own state is nobody's start)
+  const int D = c.dim, V = c.vdim, col = (blockIdx.z * (NT / 64) + wave) * 16 + l16;
+  const bool vok = col < V;
+  float* dl = delta ? delta + ((size_t)blockIdx.x * c.heads + h) * D * V : nullptr;
+  float* Sp = Sg + ((size_t)slot[b] * c.heads + h) * D * V;
+  const float* init = OUT ? (dl ? dl : (pos0[b] > 0 ? Sp : nullptr)) : nullptr;
+  const uint32_t off_s = g * 4 * (uint32_t)V + col;
+  f32x4 S[DT];
+#pragma unroll
+  for (int d = 0; d < DT; d++)
+#pragma unroll
+    for (int r = 0; r < 4; r++) S[d][r] = init && vok && g * 4 < D - (d * 16 + r) ? (init + (size_t)(d * 16 + r) * V)[off_s] : 0.f;
+  const float* kb = k + (h / c.hpk) * D;
+  const float* qb = OUT ? q + (h / c.hpk) * D : nullptr;
+  const float* ab = PH ? a + h : a + h * D;
+  const float* vb = v + (size_t)h * V;
+  float* ob = o + (size_t)h * V;
+  const float sk = OUT && skip ? skip[h] : 0.f;
+  // a thread's elements lie RS rows apart: one 32-bit offset per operand, the rest of every address is uniform
+  constexpr int RS = NT / DW;
+  const int row0 = tid / DW, cc0 = tid % DW;
+  const uint32_t off_k = row0 * (uint32_t)c.ldk + cc0, off_q = row0 * (uint32_t)c.ldq + cc0, off_a = PH ? tid * (uint32_t)c.lda : row0 * (uint32_t)c.lda + cc0,
+                 off_v = g * 4 * (uint32_t)c.ldv + col, off_o = g * 4 * (uint32_t)(c.heads * V) + col, off_m = tid * (uint32_t)c.ldm;
+  float rq[OUT ? E : 1], rk[E], ra[PH ? 1 : E], rm = 0.f, rv[4];
+  auto fetch = [&](int tb) {
+#pragma unroll
+    for (int n = 0; n < E; n++) {
+      const int t = tb + n * RS;
+      const bool ok = t + row0 < t1 && cc0 < D;
+      rk[n] = ok ? (kb + (size_t)t * c.ldk)[off_k] : 0.f;
+      if constexpr (OUT) rq[n] = ok ? (qb + (size_t)t * c.ldq)[off_q] : 0.f;
+      if constexpr (!PH) ra[n] = ok ? (ab + (size_t)t * c.lda)[off_a] : 1.f;
+    }
+    if (tid < SM_T) {
+      rm = tb + tid < t1 ? (vmul ? (vmul + (size_t)tb * c.ldm + h)[off_m] : 1.f) : 0.f;
+      if constexpr (PH) ra[0] = tb + tid < t1 ? (ab + (size_t)tb * c.lda)[off_a] : 1.f;
+    }
+#pragma unroll
+    for (int s = 0; s < 4; s++) rv[s] = vok && tb + g * 4 + s < t1 ? (vb + (size_t)(tb + s) * c.ldv)[off_v] : 0.f;
+  };
+  auto put = [&]() {
+#pragma unroll
+    for (int n = 0; n < E; n++) {
+      const int at = (row0 + n * RS) * DP + cc0;
+      lds[L::KR + at] = rk[n];
+      if constexpr (OUT) lds[L::QR + at] = rq[n] * c.q_scale;
+      if constexpr (!PH) lds[L::AR + at] = ra[n];
+    }
+    if (tid < SM_T) {
+      lds[L::MR + tid] = rm;
+      if constexpr (PH) lds[L::AR + tid] = ra[0];
+    }
+  };
+  fetch(t0);
+  put();
+  for (int tb = t0; tb < t1; tb += SM_T) {
+    float cv[4];
+#pragma unroll
+    for (int s = 0; s < 4; s++) cv[s] = rv[s];
+    if (tb + SM_T < t1) fetch(tb + SM_T);
+    __syncthreads();                       // the block's rows are there; the last block's products have been read
+    if constexpr (OUT) {
+      // (what follows compares the thread's place with constants: an opaque copy of it keeps those masks from being held across the loop)
+      int tl = tid;
+      asm volatile("" : "+v"(tl));
+      if constexpr (PH) {
+        if (wave < L::PARTS) {
+          f32x4 acc = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+          for (int d = wave; d < DT; d += L::PARTS) {
+            const float4 x = *reinterpret_cast<const float4*>(lds + L::QR + l16 * DP + d * 16 + g * 4);
+            const float4 y = *reinterpret_cast<const float4*>(lds + L::KR + l16 * DP + d * 16 + g * 4);
+            acc = __builtin_amdgcn_mfma_f32_16x16x4f32(x.x, y.x, acc, 0, 0, 0);
+            acc = __builtin_amdgcn_mfma_f32_16x16x4f32(x.y, y.y, acc, 0, 0, 0);
+            acc = __builtin_amdgcn_mfma_f32_16x16x4f32(x.z, y.z, acc, 0, 0, 0);
+            acc = __builtin_amdgcn_mfma_f32_16x16x4f32(x.w, y.w, acc, 0, 0, 0);
+          }
+#pragma unroll
+          for (int r = 0; r < 4; r++) lds[L::AS + (wave * SM_T + g * 4 + r) * SM_AST + l16] = acc[r];
+        }
+        if (tid < SM_T * SM_T) {           // m_i prod_{i < j <= t} a_j, 0 for i > t
+          const int t = tl / SM_T, i = tl % SM_T;
+          float p = i <= t ? lds[L::MR + i] : 0.f;
+#pragma unroll
+          for (int j = 1; j < SM_T; j++) p *= j > i && j <= t ? lds[L::AR + j] : 1.f;
+          lds[L::RT + t * SM_AST + i] = p;
+        }
+      } else {
+        const int i = tl / SL, sl = tl % SL, i0 = wave * 64 / SL;
+        float kk[CPS], w[CPS], sum[SM_T];
+#pragma unroll
+        for (int m = 0; m < CPS; m++) {
+          kk[m] = lds[L::KR + i * DP + (m / VW) * SL * VW + sl * VW + m % VW];
+          w[m] = 0.f;
+        }
+#pragma unroll
+        for (int t = 0; t < SM_T; t++) {
+          sum[t] = 0.f;
+          if (t >= i0) {                   // (uniform over the wavefront)
+#pragma unroll
+            for (int m = 0; m < CPS; m++) {
+              const int cc = (m / VW) * SL * VW + sl * VW + m % VW;
+              w[m] = t == i ? kk[m] : w[m] * lds[L::AR + t * DP + cc];
+              sum[t] = fmaf(lds[L::QR + t * DP + cc], w[m], sum[t]);
+            }
+          }
+        }
+        // the 16 sums over the row's 16 lanes: every step halves the sums a lane carries (partners 8, 7, 2, 1 lanes' bits away)
+        fold_pairs<8, KTX_DPP_ROW_ROR8>(sum, tl & 8);
+        fold_pairs<4, KTX_DPP_ROW_HALF_MIRROR>(sum, tl & 4);
+        fold_pairs<2, KTX_DPP_QUAD_2301>(sum, tl & 2);
+        fold_pairs<1, KTX_DPP_QUAD_1032>(sum, tl & 1);
+        float st = sum[0];
+        if constexpr (SL == 32) st += __shfl_xor(st, 16);
+        if (sl < 16) lds[L::AS + sl * SM_AST + i] = fmaf(st, lds[L::MR + i], sl == i ? sk : 0.f);
+      }
+    }
+    if (row0 == 0) {                       // thread = key channel, one group of threads per operand
+      float p = 1.f;
+#pragma unroll
+      for (int t = SM_T - 1; t >= 0; t--) {
+        lds[L::KP + t * DP + cc0] = lds[L::KR + t * DP + cc0] * (lds[L::MR + t] * p);
+        p *= lds[L::AR + (PH ? t : t * DP + cc0)];
+      }
+      lds[L::PL + cc0] = p;
+    } else if (OUT && row0 == 1) {
+      float p = 1.f;
+#pragma unroll
+      for (int t = 0; t < SM_T; t++) {
+        p *= lds[L::AR + (PH ? t : t * DP + cc0)];
+        lds[L::QP + t * DP + cc0] = lds[L::QR + t * DP + cc0] * p;
+      }
+    }
+    __syncthreads();
+    if (tb + SM_T < t1) put();             // (the raw rows have been read)
+    if constexpr (OUT) {
+      f32x4 acc = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+      for (int d = 0; d < DT; d++) {
+        const float4 x = *reinterpret_cast<const float4*>(lds + L::QP + l16 * DP + d * 16 + g * 4);
+        acc = __builtin_amdgcn_mfma_f32_16x16x4f32(x.x, S[d][0], acc, 0, 0, 0);
+        acc = __builtin_amdgcn_mfma_f32_16x16x4f32(x.y, S[d][1], acc, 0, 0, 0);
+        acc = __builtin_amdgcn_mfma_f32_16x16x4f32(x.z, S[d][2], acc, 0, 0, 0);
+        acc = __builtin_amdgcn_mfma_f32_16x16x4f32(x.w, S[d][3], acc, 0, 0, 0);
+        if (d & 1) __builtin_amdgcn_sched_barrier(0);      // (all tiles' operands requested at once would cost the registers of a wavefront)
+      }
+      float4 y = *reinterpret_cast<const float4*>(lds + L::AS + l16 * SM_AST + g * 4);
+      if constexpr (PH) {
+#pragma unroll
+        for (int n = 1; n < L::PARTS; n++) {
+          const float4 z = *reinterpret_cast<const float4*>(lds + L::AS + (n * SM_T + l16) * SM_AST + g * 4);
+          y = make_float4(y.x + z.x, y.y + z.y, y.z + z.z, y.w + z.w);
+        }
+        const float4 w = *reinterpret_cast<const float4*>(lds + L::RT + l16 * SM_AST + g * 4);
+        const int i = l16 - g * 4;
+        y = make_float4(fmaf(y.x, w.x, i == 0 ? sk : 0.f), fmaf(y.y, w.y, i == 1 ? sk : 0.f), fmaf(y.z, w.z, i == 2 ? sk : 0.f), fmaf(y.w, w.w, i == 3 ? sk : 0.f));
+      }
+      acc = __builtin_amdgcn_mfma_f32_16x16x4f32(y.x, cv[0], acc, 0, 0, 0);
+      acc = __builtin_amdgcn_mfma_f32_16x16x4f32(y.y, cv[1], acc, 0, 0, 0);
+      acc = __builtin_amdgcn_mfma_f32_16x16x4f32(y.z, cv[2], acc, 0, 0, 0);
+      acc = __builtin_amdgcn_mfma_f32_16x16x4f32(y.w, cv[3], acc, 0, 0, 0);
+#pragma unroll
+      for (int r = 0; r < 4; r++) {
+        if (vok && tb + g * 4 + r < t1) (ob + (size_t)(tb + r) * c.heads * V)[off_o] = acc[r];
+      }
+    }
+#pragma unroll
+    for (int d = 0; d < DT; d++) {
+      const float4 p = *reinterpret_cast<const float4*>(lds + L::PL + d * 16 + g * 4);
+      S[d][0] *= p.x;
+      S[d][1] *= p.y;
+      S[d][2] *= p.z;
+      S[d][3] *= p.w;
+#pragma unroll
+      for (int s = 0; s < 4; s++) S[d] = __builtin_amdgcn_mfma_f32_16x16x4f32(lds[L::KP + (g * 4 + s) * DP + d * 16 + l16], cv[s], S[d], 0, 0, 0);
+      if (d & 1) __builtin_amdgcn_sched_barrier(0);
+    }
+  }
+  if (OUT && t1 != q1) return;
+  float* dst = OUT ? Sp : dl;
+  int gl = g * 4;
+  asm volatile("" : "+v"(gl));
+#pragma unroll
+  for (int d = 0; d < DT; d++)
+#pragma unroll
+    for (int r = 0; r < 4; r++)
+      if (vok && gl < D - (d * 16 + r)) (dst + (size_t)(d * 16 + r) * V)[off_s] = S[d][r];
+}
+
 // between the two passes over the chunks: (i) the product of a chunk's decays, thread = key row (or the head), (ii) thread = 4 (or 1)
 // state entries walks the request's chunks and replaces every chunk's own state by the one it starts from
 __global__ void __launch_bounds__(256) chunk_decay_kernel(ScanDims c, int cols, const int32_t* __restrict__ q_indptr, const float* __restrict__ a,
@@ -653,6 +887,31 @@ int ktx_decay_scan(int B, int T, int max_q_len, const int32_t* d_q_indptr, const
   const dim3 grid((unsigned)B * nch, a->heads, (a->vdim + 63) / 64);
   float* delta = nch > 1 ? a->scratch : nullptr;
   float* lam = nch > 1 ? a->scratch + (size_t)B * nch * a->heads * a->dim * a->vdim : nullptr;
+  // prompts: the matrix cores, as many value columns per workgroup as a head has (up to 128)
+  const bool mfma = a->dim <= 128 && max_q_len > SCAN_MFMA_MIN;
+#define KTX_SCANM_GO(DT, NT, PH, OUT)                                                                                                              \
+  do {                                                                                                                                          \
+    const size_t lds = (size_t)ScanTile<DT, NT, PH>::FLOATS * 4;                                                                                 \
+    KTX_HIP(ktx_set_max_lds((const void*)decay_scan_mfma_kernel<DT, NT, PH, OUT>, 128 * 1024));                                                   \
+    decay_scan_mfma_kernel<DT, NT, PH, OUT><<<dim3((unsigned)B * nch, a->heads, (a->vdim + NT / 4 - 1) / (NT / 4)), NT, lds, st>>>(              \
+        c, d_q_indptr, d_pos0, d_slot, a->q, a->k, a->v, a->a, a->vmul, a->skip, a->S, delta, a->o);                                              \
+  } while (0)
+#define KTX_SCANM_P(DT, NT, OUT)                       \
+  do {                                                 \
+    if (a->a_per_head) KTX_SCANM_GO(DT, NT, true, OUT); \
+    else KTX_SCANM_GO(DT, NT, false, OUT);             \
+  } while (0)
+#define KTX_SCANM_N(DT, OUT)                        \
+  do {                                              \
+    if (a->vdim > 64) KTX_SCANM_P(DT, 512, OUT);    \
+    else KTX_SCANM_P(DT, 256, OUT);                 \
+  } while (0)
+#define KTX_SCANM(OUT)                              \
+  do {                                              \
+    if (a->dim <= 32) KTX_SCANM_N(2, OUT);          \
+    else if (a->dim <= 64) KTX_SCANM_N(4, OUT);     \
+    else KTX_SCANM_N(8, OUT);                       \
+  } while (0)
 #define KTX_SCAN_GO(RR, PH, OUT, FULL)                                                                                                          \
   do {                                                                                                                                          \
     const size_t lds = (OUT) && NW > 1 ? (size_t)2 * NW * SC_TG * 64 * 4 : 0;                                                                    \
@@ -677,7 +936,8 @@ int ktx_decay_scan(int B, int T, int max_q_len, const int32_t* d_q_indptr, const
     else KTX_SCAN_P(32, OUT);             \
   } while (0)
   if (nch > 1) {
-    KTX_SCAN(false);
+    if (mfma) KTX_SCANM(false);
+    else KTX_SCAN(false);
     const int cols = a->a_per_head ? a->heads : a->heads * a->dim;
     chunk_decay_kernel<<<dim3((unsigned)B * nch, (cols + 255) / 256), 256, 0, st>>>(c, cols, d_q_indptr, a->a, lam);
     const int DV = a->dim * a->vdim;
@@ -688,7 +948,12 @@ int ktx_decay_scan(int B, int T, int max_q_len, const int32_t* d_q_indptr, const
     else if (a->a_per_head) chunk_chain_kernel<float, true><<<cg, 256, 0, st>>>(c, d_q_indptr, d_pos0, d_slot, a->S, lam, delta);
     else chunk_chain_kernel<float, false><<<cg, 256, 0, st>>>(c, d_q_indptr, d_pos0, d_slot, a->S, lam, delta);
   }
-  KTX_SCAN(true);
+  if (mfma) KTX_SCANM(true);
+  else KTX_SCAN(true);
+#undef KTX_SCANM
+#undef KTX_SCANM_N
+#undef KTX_SCANM_P
+#undef KTX_SCANM_GO
 #undef KTX_SCAN
 #undef KTX_SCAN_P
 #undef KTX_SCAN_F
