@@ -66,7 +66,8 @@ int ktx_ssd_prep(int B, int T, int max_q_len, int C, int taps, int H, const floa
  *   S <- diag(a_t) S + k_t (m_t v_t)^T;   o[t][h] = q_scale S^T q_t + skip[h] v_t
  * a: per key channel, a[t * lda + h * dim + d], or (a_per_head) one number a[t * lda + h]; m = vmul[t * ldm + h] (NULL: 1); skip fp32
  * [heads] or NULL.  q, k, v: fp32 rows with strides ldq, ldk, ldv, head g's dim entries at g * dim, head h's vdim entries at h * vdim.
- * 0 <= a is assumed.  o fp32 [T][heads * vdim].
+ * 0 <= a <= 1 is assumed.  o fp32 [T][heads * vdim].  Steps of a few tokens, and dim > 128, run token by token on the vector ALUs; prompts
+ * with dim <= 128 run 16 tokens at a time on the fp32 matrix cores.  dim <= 512.
  * Requests longer than chunk_len tokens are cut into chunks that run side by side: every chunk's own state from zero, a pass over the
  * chunks' states, then every chunk from the state it starts with.  Scratch for that (needed when max_q_len > chunk_len):
  * ktx_decay_scan_scratch() floats; n = ceil(max_q_len / chunk_len) chunks per request are launched. */

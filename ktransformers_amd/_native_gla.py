@@ -129,7 +129,13 @@ def ssd_prep(proj: torch.Tensor, c_off: int, dt_off: int, w: torch.Tensor, bias:
     return u, gates
 
 
-SCAN_CHUNK = 64      # tokens per chunk of a prompt (chunks run side by side)
+SCAN_CHUNK = 64      # tokens per chunk of a prompt (chunks run side by side); twice as many where that still leaves SCAN_GROUPS workgroups
+SCAN_GROUPS = 512
+
+
+def scan_chunk(heads: int, vdim: int, batch) -> int:
+    groups = heads * ((vdim + 127) // 128) * (batch.T // (2 * SCAN_CHUNK))
+    return 2 * SCAN_CHUNK if groups >= SCAN_GROUPS else SCAN_CHUNK
 
 
 def decay_scan(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, decay: torch.Tensor, batch, S: torch.Tensor, heads_per_key: int = 1,
@@ -153,7 +159,7 @@ def decay_scan(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, decay: torch.T
     a.a_per_head = 1 if decay.shape[1] == H and D > 1 else 0
     a.skip, a.q_scale, a.S = _ptr(skip), float(q_scale), S.data_ptr()
     o = torch.empty((T, H * V), dtype=torch.float32, device=q.device)
-    a.o, a.chunk_len = o.data_ptr(), int(SCAN_CHUNK if chunk_len is None else chunk_len)
+    a.o, a.chunk_len = o.data_ptr(), int(scan_chunk(H, V, batch) if chunk_len is None else chunk_len)
     need = lib.ktx_decay_scan_scratch(C.byref(a), batch.B, int(batch.max_q_len))
     scratch = torch.empty(need, dtype=torch.float32, device=q.device) if need else None
     a.scratch = _ptr(scratch)

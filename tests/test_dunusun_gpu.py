@@ -263,7 +263,7 @@ def test_decayed_scan_whole_portions_and_chunks(H, D, V, per_head, hpk):
             want[:, h] += d64(skip[h]) * d64(v[:, h])
     final = None
     for cut, chunk in (([T], 0), ([T], 8), ([T], 64), ([T], 75), ([T], 5), ([1] * T, 64), ([40, 2, 1, 2, 30], 16), ([2] * 37 + [1], 64), ([64, 11], 64),
-                       ([9, 66], 32)):
+                       ([9, 66], 32), ([5] * 15, 64), ([17, 16, 15, 27], 64)):
         got, S = run_scan(q, k, v, a, per_head, hpk, q_scale, vmul, skip, cut, chunk)
         assert rel(got, want) < 5e-6, (cut[:4], chunk)
         assert rows_rel(got.reshape(T, -1), want.reshape(T, -1)) < 5e-5, (cut[:4], chunk)
@@ -286,7 +286,7 @@ def test_decayed_scan_remembers_one_far_token(per_head):
         kk[j, :, 3] = 1.0
         vv[j] = torch.randn(H, V, generator=g)
         a = torch.ones(T, H, 1 if per_head else D)
-        for chunk in (16, 64, 0):
+        for chunk in (16, 64, 128, 0):
             got, _ = run_scan(q, kk, vv, a, per_head, 1, 1.0, None, None, [T], chunk)
             assert rel(got[-1], vv[j]) < 1e-6 and float(got[:-1].abs().max()) == 0.0, j
         if j < T - 1:
