@@ -2,7 +2,7 @@
 # kernel resource usage of one csrc/*.hip: name, VGPRs, AGPRs, spills, scratch, LDS, code bytes.  usage: scripts/kres.sh ktx_linear [filter]
 f=$1; pat=${2:-.}
 mkdir -p /tmp/kres && cd /tmp/kres
-hipcc --offload-arch=gfx950 -O3 -std=c++17 -ffp-contract=off -Wno-unused-value --cuda-device-only -c /root/repo/ktransformers_amd/csrc/$f.hip -o $f.co -Rpass-analysis=kernel-resource-usage 2> $f.rem
+hipcc --offload-arch=gfx950 -O3 -std=c++17 -ffp-contract=off -Wno-unused-value -Xclang -target-feature -Xclang -packed-fp32-ops --cuda-device-only -c /root/repo/ktransformers_amd/csrc/$f.hip -o $f.co -Rpass-analysis=kernel-resource-usage 2> $f.rem
 python3 - "$f.rem" "$pat" <<'PY'
 import re, sys, subprocess
 txt = open(sys.argv[1]).read()
