@@ -3,7 +3,7 @@
     python -m ktransformers_amd.build [--force]
 
 Every csrc/*.hip is compiled to its own object (in parallel, only when it or a header it may include changed) and the
-objects are linked into ktransformers_amd/lib/libktx_hip.so (git-ignored, travels with the gpurun snapshot).
+objects are linked into ktransformers_amd/lib/libktx_hip.so (git-ignored).
 """
 from __future__ import annotations
 
