@@ -70,13 +70,15 @@ int ktx_ssd_prep(int B, int T, int max_q_len, int C, int taps, int H, const floa
  * with dim <= 128 run 16 tokens at a time on the fp32 matrix cores.  dim <= 512.
  * Requests longer than chunk_len tokens are cut into chunks that run side by side: every chunk's own state from zero, a pass over the
  * chunks' states, then every chunk from the state it starts with.  Scratch for that (needed when max_q_len > chunk_len):
- * ktx_decay_scan_scratch() floats; n = ceil(max_q_len / chunk_len) chunks per request are launched. */
+ * ktx_decay_scan_scratch() floats; n = ceil(max_q_len / chunk_len) chunks per request are launched.  A decay
+ * that never changes is one row with stride lda = 0. */
 typedef struct ktx_decay_scan_args {
   int32_t heads, dim, vdim, heads_per_key;
   const float *q, *k, *v, *a, *vmul, *skip;
   int64_t ldq, ldk, ldv, lda, ldm;
   int32_t a_per_head;
   float q_scale;
+  int32_t qkv_act;    /* != 0: q, k and v are silu of what q, k, v hold */
   float* S;
   float* o;
   float* scratch;
@@ -87,7 +89,7 @@ int ktx_decay_scan(int B, int T, int max_q_len, const int32_t* d_q_indptr, const
                    const ktx_decay_scan_args* a, ktx_stream_t stream);
 
 /* ---- gate / norm segments side by side ------------------------------------------------------------------------------------------------ */
-/* out[t][out_off + c] = scale * f(o[t][c], gate[t][c]), c < n, for up to KTX_GATE_SEGS segments in one launch; per segment
+/* out[t][out_off + c] = scale * f(o[t][c], gate[t][c / gate_div]), c < n (gate_div = 1: a gate per column; a head's size: one per head), for up to KTX_GATE_SEGS segments in one launch; per segment
  *   group == 0:                 f = o act(gate)
  *   gate_first == 0:            f = o r w act(gate), r = 1 / sqrt(mean(o^2 over the group of c) + eps)
  *   gate_first != 0:            f = p r w,           p = o act(gate), r = 1 / sqrt(mean(p^2 over the group of c) + eps)
@@ -101,7 +103,7 @@ typedef struct ktx_gate_seg {
   const float* gate;
   int64_t ldg;
   const float* w;
-  int32_t n, group, w_mod, act, gate_first;
+  int32_t n, group, w_mod, act, gate_first, gate_div;
   float eps, scale;
   int32_t out_off;
 } ktx_gate_seg;

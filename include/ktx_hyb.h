@@ -26,17 +26,18 @@ int ktx_rows_add(int T, int W, float* d_x, const float* d_x0, const float* d_vec
 int ktx_layer_norm(int T, int W, const float* d_x, const float* d_w, const float* d_b, float eps, const int32_t* d_rows, void* d_out,
                    int out_dtype, ktx_stream_t stream);
 
-/* The gated, post-normed residual update of one sublayer, one launch:
+/* The gated, post-normed residual update of one sublayer, one launch (norm = layer norm, or with rms != 0 the RMS norm
+ * v / sqrt(mean(v^2) + eps) * w + b):
  *   z[t] = (y ? y[t] : 0) + (ybias ? ybias : 0) + sum_{k < top} topk_w[t][k] * ey[pair_pos[t * top + k]]     (ey NULL: no such term)
  *   z   *= sigmoid(gl[t] + gbias)                                                                            (gl NULL: no gate)
- *   x[t] += layer_norm(z; wn, bn, eps)
- *   next_out[t] = layer_norm(x[t]; next_w, next_b, next_eps)      (next_w NULL: not written) — the pre-norm of the sublayer that follows
+ *   x[t] += norm(z; wn, bn, eps)
+ *   next_out[t] = norm(x[t]; next_w, next_b, next_eps)            (next_w NULL: not written) — the pre-norm of the sublayer that follows
  * y fp32 rows of stride ldy, ey fp32 [pairs][W], gl fp32 rows of stride ldg, all vectors fp32 [W]; x fp32 [T][W] in place;
  * next_out [T][W] of next_dtype. */
 int ktx_gated_norm_add(int T, int W, const float* d_y, int64_t ldy, const float* d_ybias, const float* d_ey, const int32_t* d_pair_pos,
                        const float* d_topk_w, int top, const float* d_gl, int64_t ldg, const float* d_gbias, const float* d_wn,
                        const float* d_bn, float eps, float* d_x, const float* d_next_w, const float* d_next_b, float next_eps,
-                       void* d_next_out, int next_dtype, ktx_stream_t stream);
+                       void* d_next_out, int next_dtype, int rms, ktx_stream_t stream);
 
 /* The post-normed residual update of one sublayer with a scaled residual, and the depth-weighted average behind a layer, one launch:
  *   v[t] = layer_norm(alpha * x_in[t] + (y ? y[t] : 0) + (ybias ? ybias : 0); w, b, eps)
@@ -69,11 +70,11 @@ int ktx_poly_norm(int T, int F, const float* d_z, int64_t ldz, const float* d_bi
 /* out[r][f] = silu(in[r][f]) * in[r][F + f]: fp32 rows of 2F (stride ldi) -> [R][F] of out_dtype. */
 int ktx_silu_mul_rows(int R, int F, const float* d_in, int64_t ldi, void* d_out, int out_dtype, ktx_stream_t stream);
 
-/* out[r][f] = g * sigmoid(slope * g) * (u + up_shift) with g = min(gate, limit), u = clamp(up, -limit, limit): the activation of a GLU
- * whose gate is capped from above and whose linear half is clamped (limit = INFINITY: neither); fp32 rows of 2F (stride ldi) holding
- * gate = in[r][f], up = in[r][F + f], or — paired != 0 — gate = in[r][2f], up = in[r][2f + 1]; -> [R][F] of out_dtype. */
-int ktx_glu_clamp_rows(int R, int F, const float* d_in, int64_t ldi, float limit, float slope, float up_shift, int paired, void* d_out,
-                       int out_dtype, ktx_stream_t stream);
+/* out[r][f] = glu(gate, up) (ktx_glu_act of ktx_seq.h: the halves bounded, then swish or GELU of the gate times the shifted linear half);
+ * fp32 rows of 2F (stride ldi) holding gate = in[r][f], up = in[r][F + f], or — paired != 0 — gate = in[r][2f], up = in[r][2f + 1];
+ * -> [R][F] of out_dtype. */
+int ktx_glu_clamp_rows(int R, int F, const float* d_in, int64_t ldi, const ktx_glu_act* glu, int paired, void* d_out, int out_dtype,
+                       ktx_stream_t stream);
 
 /* out[r][c] = o[r][c] * sigmoid(gate[r][c]): o [R][N] of o_dtype, gate fp32 rows of stride ldg -> [R][N] of out_dtype (an output gate
  * on an attention's concatenated heads). */
@@ -119,6 +120,7 @@ typedef struct ktx_latattn_config {
   float eps;                                  /* of the latent's RMS norm */
   int32_t page_size, cache_dtype;             /* cache rows [rows][kv_rank + rot_dim] of KTX_SEQ_* */
   int32_t rot_half;                           /* != 0: the turning pairs are (i, i + rot_dims / 2) instead of (2i, 2i + 1) */
+  float rot_scale;                            /* multiplies every cosine and sine (1: a pure rotation) */
 } ktx_latattn_config;
 
 /* Per token: the first kv_rank entries of the down projection, RMS-normed with weight wn, and the last rot_dim, rotated at the token's
@@ -130,6 +132,13 @@ typedef struct ktx_latattn_config {
 int ktx_latattn_prep(const ktx_latattn_config* cfg, int T, const float* d_proj, int64_t ldp, int q_off, int c_off, const float* d_wn,
                      const double* d_inv_freq, const int32_t* d_pos, const int32_t* d_cache_loc, void* d_cache, float* d_q_out,
                      ktx_stream_t stream);
+
+/* The latent rows of a step whose queries pass a latent of their own: per token, d_cache row cache_loc[t] as ktx_latattn_prep writes it
+ * (from the down projection at c_off), and q_lat[t] = the q_rank entries at cq_off of proj, RMS-normed (eps of cfg) with weight wq
+ * (fp32 [q_rank]) -> [T][q_rank] of q_dtype.  The queries then are a product of q_lat; ktx_latattn_prep without a cache turns them. */
+int ktx_latattn_latents(const ktx_latattn_config* cfg, int T, const float* d_proj, int64_t ldp, int cq_off, int q_rank, int c_off,
+                        const float* d_wq, const float* d_wn, const double* d_inv_freq, const int32_t* d_pos, const int32_t* d_cache_loc,
+                        void* d_cache, void* d_q_lat, int q_dtype, ktx_stream_t stream);
 
 /* out[t][h] = sum_j w_j c_j over the keys j in the window of token t, w = softmax over {scale q[t][h] . row_j} u {sink[h]} with the
  * sink's weight dropped (it has no value; d_sink NULL: an ordinary softmax over the keys).  q fp32 [T][heads][kv_rank + rot_dim]; out [T][heads][kv_rank] of out_dtype.
@@ -163,8 +172,9 @@ int ktx_moe_plan(int T, int E, int top, int tile_m, const int32_t* d_topk_idx, i
                  ktx_stream_t stream);
 
 enum { KTX_GG_TILE_M = 64, KTX_GG_TILE_M_WIDE = 128 };
-/* epilogues of the grouped products: none; silu(gate) * up over a [2N][K] matrix (streaming form only); relu(y)^2 */
-enum { KTX_GG_ACT_NONE = 0, KTX_GG_ACT_GLU_SILU = 1, KTX_GG_ACT_RELU_SQ = 2 };
+/* epilogues of the grouped products: none; silu(gate) * up over a [2N][K] matrix (streaming form only); relu(y)^2; a gated linear unit
+ * over matrices whose rows ALTERNATE gate_f, up_f: Y holds half as many columns as the matrices have rows */
+enum { KTX_GG_ACT_NONE = 0, KTX_GG_ACT_GLU_SILU = 1, KTX_GG_ACT_RELU_SQ = 2, KTX_GG_ACT_GLU_PAIRS = 3 };
 
 /* Grouped GEMM  Y_g = A_g W_g^T  on the matrix cores (the product runs in W's type like ktx_dense_gemm; Y fp32 or bf16).
  * W: G matrices [N][K] back to back.
@@ -174,18 +184,20 @@ enum { KTX_GG_ACT_NONE = 0, KTX_GG_ACT_GLU_SILU = 1, KTX_GG_ACT_RELU_SQ = 2 };
  *   Y row is r; tiles come from ktx_moe_plan (max_tiles bounds the launch, num_tiles[0] on the device says how many are real) and hold
  *   tile_m = 64 rows, or 128 (bf16 products only: the wide tile prompts take).  The plan may hold MORE groups than G (a router whose
  *   last outputs stand for experts without weights): their tiles are skipped and their Y rows left untouched.
- * act: KTX_GG_ACT_NONE or KTX_GG_ACT_RELU_SQ, applied to Y. */
+ * act: KTX_GG_ACT_NONE, KTX_GG_ACT_RELU_SQ, or (N even; glu says which unit) KTX_GG_ACT_GLU_PAIRS: Y[r][f] = glu(y_2f, y_2f+1), f < N / 2. */
 int ktx_grouped_gemm(int G, int M, int N, int K, const void* d_A, int a_dtype, int64_t lda, int64_t a_goff, const int32_t* d_a_rows,
                      const void* d_W, int w_dtype, void* d_Y, int y_dtype, int64_t ldy, int64_t y_goff, const int32_t* d_group_off,
                      const int32_t* d_tile_group, const int32_t* d_tile_row0, const int32_t* d_num_tiles, int max_tiles, int tile_m,
-                     int act, ktx_stream_t stream);
+                     int act, const ktx_glu_act* glu, ktx_stream_t stream);
 
 /* The ragged products for a handful of rows (decode steps), streaming each row's weights once: Y[r] = W_g A[a_rows ? a_rows[r] : r]
  * with g = row_group[r]; rows whose group is >= G (no weights) are left untouched.  act = KTX_GG_ACT_GLU_SILU: W_g is [2N][K] (gate
  * rows, then up rows) and Y[r][n] = silu(gate_n . a) * (up_n . a) — the activation of a GLU expert in the same launch;
- * KTX_GG_ACT_RELU_SQ: Y = relu(Y)^2.  fp32 accumulation on the vector ALUs; any N, K. */
+ * KTX_GG_ACT_RELU_SQ: Y = relu(Y)^2; KTX_GG_ACT_GLU_PAIRS: W_g is [2N][K], rows alternating gate_n, up_n, Y[r][n] = glu(gate_n . a, up_n . a).
+ * fp32 accumulation on the vector ALUs; any N, K. */
 int ktx_grouped_gemv(int R, int N, int K, const void* d_A, int a_dtype, int64_t lda, const int32_t* d_a_rows, const void* d_W, int w_dtype,
-                     void* d_Y, int y_dtype, int64_t ldy, const int32_t* d_row_group, int act, int G, ktx_stream_t stream);
+                     void* d_Y, int y_dtype, int64_t ldy, const int32_t* d_row_group, int act, const ktx_glu_act* glu, int G,
+                     ktx_stream_t stream);
 
 #ifdef __cplusplus
 }

@@ -91,12 +91,14 @@ typedef struct ktx_swa_config {
   int32_t keep_first;                 /* with a window: the first keep_first positions of a sequence stay visible to every later one */
   int32_t bias_span;                  /* rows - 1 of the distance-bias table the attention calls take (distances beyond it read its last row) */
   float softcap;                      /* > 0: the score becomes softcap tanh(score / softcap) (before a distance bias joins it); 0: off */
+  float rot_scale;                    /* multiplies the cosines and sines that turn q and k (1: a pure rotation) */
 } ktx_swa_config;
 
 /* Per token: rotate and norm q (times scale) -> q_out fp32 [T][heads][dim]; rotate and norm k, turn v -> cache rows cache_loc[t];
  * the cosines | sines of the value rotation at the token's position -> vcs fp32 [T][vdim] (read again when results are turned back).
  * Angles = pos * inv_freq[i] in fp64 (inv_freq fp64 [rot_dims / 2], v_inv_freq fp64 [vdim / 2]), rounded once.
- * proj fp32 rows of stride ldp with q, k, v at their offsets. */
+ * proj fp32 rows of stride ldp with q, k, v at their offsets.  d_kcache and d_vcache NULL (rot_values = 0): only q_out is written — the layer
+ * reads keys and values another layer of equal kv_heads, sizes and rotation cached. */
 int ktx_swa_prep(const ktx_swa_config* cfg, int T, const float* d_proj, int64_t ldp, int q_off, int k_off, int v_off,
                  const double* d_inv_freq, const double* d_v_inv_freq, const int32_t* d_pos, const int32_t* d_cache_loc, void* d_kcache,
                  void* d_vcache, float* d_q_out, float* d_vcs, ktx_stream_t stream);
@@ -131,7 +133,7 @@ int ktx_swa_forward(const ktx_swa_config* cfg, int T, const float* d_q, const vo
 
 /* The same operator on the matrix cores for prompts, portions and decode steps: the (token, head) pairs of a request that share a key
  * head are the rows of one query matrix; workgroups of 64 rows walk 32-key tiles, bf16 MFMA for q . k and weights x values, scores /
- * mask / softmax in fp32.  Eligible: bf16 caches, dim a multiple of 32 up to 256, vdim a multiple of 16 up to 128, or 256. */
+ * mask / softmax in fp32.  Eligible: bf16 caches, dim a multiple of 8 up to 256, vdim a multiple of 16 up to 128, or 256. */
 int ktx_swa_mfma_eligible(const ktx_swa_config* cfg);
 int ktx_swa_mfma(const ktx_swa_config* cfg, int B, int T, int max_q_len, const float* d_q, const void* d_kcache, const void* d_vcache,
                  const int32_t* d_q_indptr, const int32_t* d_pos0, const int32_t* d_page_indptr, const int32_t* d_page_indices,
@@ -163,16 +165,17 @@ int ktx_ssm_scan(const ktx_ssm_config* cfg, int B, int T, int max_q_len, const i
                  int z_off, float* d_S, float* d_conv_state, void* d_out, int out_dtype, ktx_stream_t stream);
 
 /* ---- softmax router --------------------------------------------------------------------------------------------------------------- */
-/* s = softmax(logits[t]) over all E router outputs (fp32 rows of stride ldl); the `top` largest s + correction (fp32 [E] or NULL; lowest
- * index first on ties) -> topk_idx int32 [T][top]; topk_w fp32 [T][top] = the chosen s (without the correction) over (their sum + sum_eps). */
-int ktx_softmax_route(int T, int E, int top, float sum_eps, const float* d_logits, int64_t ldl, const float* d_correction,
+/* s = softmax(z) over all E router outputs, z = logits[t] + bias (logits: fp32 rows of stride ldl; bias fp32 [E] or NULL); the `top` largest
+ * s + correction (fp32 [E]; NULL: the largest z; lowest index first on ties) -> topk_idx int32 [T][top]; topk_w fp32 [T][top] = the chosen s
+ * (without the correction) over (their sum + sum_eps); sum_eps = 0 is the softmax over the chosen z alone. */
+int ktx_softmax_route(int T, int E, int top, float sum_eps, const float* d_logits, int64_t ldl, const float* d_bias, const float* d_correction,
                       int32_t* d_topk_idx, float* d_topk_w, ktx_stream_t stream);
 
 /* The same router followed, in the same launch, by the expert sort of ktx_moe_plan (ktx_hyb.h; same outputs, E groups): for small steps
  * (decode), T <= KTX_ROUTE_PLAN_MAX_T, where one workgroup routes and sorts. */
 enum { KTX_ROUTE_PLAN_MAX_T = 256 };
-int ktx_softmax_route_plan(int T, int E, int top, float sum_eps, const float* d_logits, int64_t ldl, const float* d_correction,
-                           int32_t* d_topk_idx, float* d_topk_w, int tile_m, int32_t* d_group_off, int32_t* d_sorted_tok,
+int ktx_softmax_route_plan(int T, int E, int top, float sum_eps, const float* d_logits, int64_t ldl, const float* d_bias,
+                           const float* d_correction, int32_t* d_topk_idx, float* d_topk_w, int tile_m, int32_t* d_group_off, int32_t* d_sorted_tok,
                            int32_t* d_pair_pos, int32_t* d_sorted_group, int32_t* d_tile_group, int32_t* d_tile_row0, int32_t* d_num_tiles,
                            ktx_stream_t stream);
 

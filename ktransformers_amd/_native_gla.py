@@ -21,12 +21,12 @@ class _HyperArgs(C.Structure):       # include/ktx_gla.h: ktx_hyper_args
 class _DecayScanArgs(C.Structure):   # include/ktx_gla.h: ktx_decay_scan_args
     _fields_ = [("heads", _I32), ("dim", _I32), ("vdim", _I32), ("heads_per_key", _I32), ("q", _P), ("k", _P), ("v", _P), ("a", _P),
                 ("vmul", _P), ("skip", _P), ("ldq", _L), ("ldk", _L), ("ldv", _L), ("lda", _L), ("ldm", _L), ("a_per_head", _I32),
-                ("q_scale", _F), ("S", _P), ("o", _P), ("scratch", _P), ("chunk_len", _I32)]
+                ("q_scale", _F), ("qkv_act", _I32), ("S", _P), ("o", _P), ("scratch", _P), ("chunk_len", _I32)]
 
 
 class _GateSeg(C.Structure):         # include/ktx_gla.h: ktx_gate_seg
     _fields_ = [("o", _P), ("ldo", _L), ("o_dtype", _I32), ("gate", _P), ("ldg", _L), ("w", _P), ("n", _I32), ("group", _I32), ("w_mod", _I32),
-                ("act", _I32), ("gate_first", _I32), ("eps", _F), ("scale", _F), ("out_off", _I32)]
+                ("act", _I32), ("gate_first", _I32), ("gate_div", _I32), ("eps", _F), ("scale", _F), ("out_off", _I32)]
 
 
 if not hasattr(lib, "ktx_decay_scan"):
@@ -139,9 +139,10 @@ def scan_chunk(heads: int, vdim: int, batch) -> int:
 
 
 def decay_scan(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, decay: torch.Tensor, batch, S: torch.Tensor, heads_per_key: int = 1,
-               vmul: torch.Tensor | None = None, skip: torch.Tensor | None = None, q_scale: float = 1.0, chunk_len: int | None = None) -> torch.Tensor:
+               vmul: torch.Tensor | None = None, skip: torch.Tensor | None = None, q_scale: float = 1.0, chunk_len: int | None = None, qkv_silu: bool = False) -> torch.Tensor:
     """The decayed outer-product scan (ktx_decay_scan): q, k fp32 rows [T, (heads / heads_per_key) * dim], v [T, heads * vdim] (column
-    slices are fine), decay [T, heads * dim] (per key channel) or [T, heads]; vmul [T, heads]: multiplies the values that enter the state;
+    slices are fine), decay [T, heads * dim] (per key channel) or [T, heads] (rows may be one row expanded: a decay that never changes);
+    qkv_silu: q, k and v are silu of what the rows hold; vmul [T, heads]: multiplies the values that enter the state;
     skip fp32 [heads]: adds skip[h] v_t to the read-out.  S fp32 [slots, heads, dim, vdim] moves on -> o fp32 [T, heads * vdim]."""
     _f32(S, "decay_scan S"), _f32(skip, "decay_scan skip")
     H, D, V = S.shape[1:]
@@ -157,7 +158,7 @@ def decay_scan(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, decay: torch.T
     if decay.shape[1] not in (H, H * D) or batch.T != T or (skip is not None and skip.numel() != H):
         raise KtxError("decay_scan: a decay per head or per key channel, one token per row")
     a.a_per_head = 1 if decay.shape[1] == H and D > 1 else 0
-    a.skip, a.q_scale, a.S = _ptr(skip), float(q_scale), S.data_ptr()
+    a.skip, a.q_scale, a.S, a.qkv_act = _ptr(skip), float(q_scale), S.data_ptr(), 1 if qkv_silu else 0
     o = torch.empty((T, H * V), dtype=torch.float32, device=q.device)
     a.o, a.chunk_len = o.data_ptr(), int(scan_chunk(H, V, batch) if chunk_len is None else chunk_len)
     need = lib.ktx_decay_scan_scratch(C.byref(a), batch.B, int(batch.max_q_len))
@@ -168,15 +169,18 @@ def decay_scan(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, decay: torch.T
     return o
 
 
-def gate_seg(o: torch.Tensor, gate: torch.Tensor, act: str, norm: tuple | None = None, gate_first: bool = False, scale: float = 1.0):
-    """One segment of gate_segments: o [T, n] (fp32 | bf16 rows), gate fp32 rows [T, n]; norm = (weight fp32, group, eps): RMS norm over
+def gate_seg(o: torch.Tensor, gate: torch.Tensor, act: str, norm: tuple | None = None, gate_first: bool = False, scale: float = 1.0,
+             gate_div: int = 1):
+    """One segment of gate_segments: o [T, n] (fp32 | bf16 rows), gate fp32 rows [T, n], or [T, n / gate_div]: one gate per gate_div columns; norm = (weight fp32, group, eps): RMS norm over
     groups of `group` columns, weight of `group` (shared by the groups) or n entries; gate_first: the gate multiplies before the norm."""
     gp, ldg = _rows_f32(gate, "gate_seg gate")
-    if not o.is_cuda or o.dtype not in SEQ_DTYPE or o.dim() != 2 or o.stride(1) != 1 or tuple(o.shape) != tuple(gate.shape):
+    if not o.is_cuda or o.dtype not in SEQ_DTYPE or o.dim() != 2 or o.stride(1) != 1 or gate.shape[0] != o.shape[0] or \
+            gate.shape[1] * gate_div != o.shape[1]:
         raise KtxError("gate_seg: o must be rows of the gate's shape")
     s = _GateSeg()
     s.tensors = [o, gate]            # (the struct holds addresses only: the segment keeps what it points to alive)
     s.o, s.ldo, s.o_dtype, s.gate, s.ldg, s.n = o.data_ptr(), o.stride(0), SEQ_DTYPE[o.dtype], gp, ldg, o.shape[1]
+    s.gate_div = int(gate_div)
     s.act, s.gate_first, s.scale = {"sigmoid": 0, "silu": 1}[act], int(bool(gate_first)), float(scale)
     if norm is not None:
         w, group, eps = norm

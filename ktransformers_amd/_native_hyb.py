@@ -8,7 +8,7 @@ import ctypes as C
 
 import torch
 
-from ktransformers_amd._native_seq import SEQ_DTYPE, KtxError, _seq_dev, _stream_ptr, check, lib
+from ktransformers_amd._native_seq import SEQ_DTYPE, KtxError, _GluAct, _seq_dev, _stream_ptr, check, lib
 
 
 class _DeltaConfig(C.Structure):     # include/ktx_hyb.h: ktx_delta_config
@@ -25,7 +25,7 @@ class _PostNormArgs(C.Structure):    # include/ktx_hyb.h: ktx_postnorm_args
 class _LatAttnConfig(C.Structure):   # include/ktx_hyb.h: ktx_latattn_config
     _fields_ = [("heads", C.c_int32), ("dim", C.c_int32), ("rot_dim", C.c_int32), ("vdim", C.c_int32), ("kv_rank", C.c_int32),
                 ("rot_dims", C.c_int32), ("scale", C.c_float), ("window", C.c_int32), ("eps", C.c_float), ("page_size", C.c_int32),
-                ("cache_dtype", C.c_int32), ("rot_half", C.c_int32)]
+                ("cache_dtype", C.c_int32), ("rot_half", C.c_int32), ("rot_scale", C.c_float)]
 
 
 _P, _I, _L, _F = C.c_void_p, C.c_int, C.c_int64, C.c_float
@@ -33,23 +33,24 @@ if not hasattr(lib, "ktx_grouped_gemm"):
     raise ImportError("the loaded kernel library predates include/ktx_hyb.h: rebuild with `python -m ktransformers_amd.build [--seq]`")
 lib.ktx_rows_add.argtypes = [_I, _I, _P, _P, _P, _P]
 lib.ktx_layer_norm.argtypes = [_I, _I, _P, _P, _P, _F, _P, _P, _I, _P]
-lib.ktx_gated_norm_add.argtypes = [_I, _I, _P, _L, _P, _P, _P, _P, _I, _P, _L, _P, _P, _P, _F, _P, _P, _P, _F, _P, _I, _P]
+lib.ktx_gated_norm_add.argtypes = [_I, _I, _P, _L, _P, _P, _P, _P, _I, _P, _L, _P, _P, _P, _F, _P, _P, _P, _F, _P, _I, _I, _P]
 lib.ktx_poly_norm.argtypes = [_I, _I, _P, _L, _P, _P, _F, _P, _I, _P]
 lib.ktx_silu_mul_rows.argtypes = [_I, _I, _P, _L, _P, _I, _P]
 lib.ktx_postnorm_mix.argtypes = [_I, _I, _P, _P, C.POINTER(_PostNormArgs), _P]
-lib.ktx_glu_clamp_rows.argtypes = [_I, _I, _P, _L, _F, _F, _F, _I, _P, _I, _P]
+lib.ktx_glu_clamp_rows.argtypes = [_I, _I, _P, _L, C.POINTER(_GluAct), _I, _P, _I, _P]
 lib.ktx_sigmoid_gate_rows.argtypes = [_I, _I, _P, _I, _P, _L, _P, _I, _P]
 lib.ktx_head_gate_norm.argtypes = [_I, _I, _I, _F, _P, _P, _L, _P, _I, _I, _P, _I, _P]
 lib.ktx_delta_prep.argtypes = [C.POINTER(_DeltaConfig), _I, _I, _P, _P, _P, _P, _P, _L, _I, _I, _I, _I, _I, _P, _P, _P, _P, _P, _P, _P]
 lib.ktx_delta_forward.argtypes = [C.POINTER(_DeltaConfig), _I, _P, _P, _P, _P, _P, _P, _P, _P]
 lib.ktx_latattn_prep.argtypes = [C.POINTER(_LatAttnConfig), _I, _P, _L, _I, _I, _P, _P, _P, _P, _P, _P, _P]
+lib.ktx_latattn_latents.argtypes = [C.POINTER(_LatAttnConfig), _I, _P, _L, _I, _I, _I, _P, _P, _P, _P, _P, _P, _P, _I, _P]
 lib.ktx_latattn_forward.argtypes = [C.POINTER(_LatAttnConfig), _I, _P, _P, _P, _P, _P, _P, _P, _I, _P, _P, _I, _P]
 lib.ktx_latattn_mfma_eligible.argtypes = [C.POINTER(_LatAttnConfig)]
 lib.ktx_latattn_mfma.argtypes = [C.POINTER(_LatAttnConfig), _I, _I, _I, _P, _P, _P, _P, _P, _P, _P, _I, _P, _P, _I, _P]
 lib.ktx_moe_route.argtypes = [_I, _I, _I, _F, _F, _P, _L, _P, _P, _P]
 lib.ktx_moe_plan.argtypes = [_I, _I, _I, _I, _P, _P, _P, _P, _P, _P, _P, _P, _P]
-lib.ktx_grouped_gemv.argtypes = [_I, _I, _I, _P, _I, _L, _P, _P, _I, _P, _I, _L, _P, _I, _I, _P]
-lib.ktx_grouped_gemm.argtypes = [_I, _I, _I, _I, _P, _I, _L, _L, _P, _P, _I, _P, _I, _L, _L, _P, _P, _P, _P, _I, _I, _I, _P]
+lib.ktx_grouped_gemv.argtypes = [_I, _I, _I, _P, _I, _L, _P, _P, _I, _P, _I, _L, _P, _I, C.POINTER(_GluAct), _I, _P]
+lib.ktx_grouped_gemm.argtypes = [_I, _I, _I, _I, _P, _I, _L, _L, _P, _P, _I, _P, _I, _L, _L, _P, _P, _P, _P, _I, _I, _I, C.POINTER(_GluAct), _P]
 
 TILE_M = 64
 TILE_M_WIDE, WIDE_MIN_ROWS_PER_EXPERT = 128, 96      # bf16 steps whose experts average this many rows take 128-row tiles
@@ -102,9 +103,9 @@ def layer_norm(x: torch.Tensor, w: torch.Tensor, b: torch.Tensor | None, eps: fl
 def gated_norm_add(x: torch.Tensor, wn: torch.Tensor, bn: torch.Tensor | None, eps: float, y: torch.Tensor | None = None,
                    ybias: torch.Tensor | None = None, gate_logits: torch.Tensor | None = None, gate_bias: torch.Tensor | None = None,
                    expert_rows: torch.Tensor | None = None, pair_pos: torch.Tensor | None = None, topk_w: torch.Tensor | None = None,
-                   next_norm: tuple | None = None):
-    """x += layer_norm((y + ybias + sum_k topk_w[t, k] expert_rows[pair_pos[t, k]]) * sigmoid(gate_logits + gate_bias)), in place.
-    next_norm = (weight, bias or None, eps, dtype): also returns layer_norm(updated x) in that type — (x, h) instead of x."""
+                   next_norm: tuple | None = None, rms: bool = False):
+    """x += norm((y + ybias + sum_k topk_w[t, k] expert_rows[pair_pos[t, k]]) * sigmoid(gate_logits + gate_bias)), in place; norm = layer norm,
+    or the RMS norm (rms).  next_norm = (weight, bias or None, eps, dtype): also returns norm(updated x) in that type — (x, h) instead of x."""
     _f32(x, "gated_norm_add x"), _f32(wn, "wn"), _f32(bn, "bn"), _f32(ybias, "ybias"), _f32(gate_bias, "gate_bias")
     _f32(expert_rows, "expert_rows"), _i32(pair_pos, "pair_pos"), _f32(topk_w, "topk_w")
     T, W = x.shape
@@ -127,7 +128,7 @@ def gated_norm_add(x: torch.Tensor, wn: torch.Tensor, bn: torch.Tensor | None, e
         h = torch.empty((T, W), dtype=ndt, device=x.device)
     check(lib.ktx_gated_norm_add(T, W, yp, ldy, _ptr(ybias), _ptr(expert_rows), _ptr(pair_pos), _ptr(topk_w), top, gp, ldg, _ptr(gate_bias),
                                  wn.data_ptr(), _ptr(bn), float(eps), x.data_ptr(), _ptr(nw), _ptr(nb), float(neps), _ptr(h),
-                                 SEQ_DTYPE[ndt], _stream_ptr(x.device)))
+                                 SEQ_DTYPE[ndt], 1 if rms else 0, _stream_ptr(x.device)))
     return x if next_norm is None else (x, h)
 
 
@@ -175,15 +176,13 @@ def postnorm_mix(x_in: torch.Tensor, x_out: torch.Tensor, w: torch.Tensor, b: to
     return x_out if lp is None else lp
 
 
-def glu_clamp_rows(gu: torch.Tensor, limit: float | None, slope: float = 1.0, up_shift: float = 0.0, out_dtype=torch.float32,
-                   paired: bool = False) -> torch.Tensor:
-    """[R, 2F] (gate | up; paired: gate_0, up_0, gate_1, up_1, ...) -> g * sigmoid(slope * g) * (u + up_shift), g = min(gate, limit),
-    u = clamp(up, -limit, limit); [R, F] (ktx_glu_clamp_rows; limit None: neither is bounded)."""
+def glu_clamp_rows(gu: torch.Tensor, unit: _GluAct, out_dtype=torch.float32, paired: bool = False) -> torch.Tensor:
+    """[R, 2F] (gate | up; paired: gate_0, up_0, gate_1, up_1, ...) -> unit(gate, up) (ktransformers_amd._native_seq.glu_act), [R, F]
+    (ktx_glu_clamp_rows)."""
     p, ld = _rows_f32(gu, "glu_clamp_rows")
     R, F = gu.shape[0], gu.shape[1] // 2
     out = torch.empty((R, F), dtype=out_dtype, device=gu.device)
-    check(lib.ktx_glu_clamp_rows(R, F, p, ld, float("inf") if limit is None else float(limit), float(slope), float(up_shift),
-                                 1 if paired else 0, out.data_ptr(), SEQ_DTYPE[out_dtype], _stream_ptr(gu.device)))
+    check(lib.ktx_glu_clamp_rows(R, F, p, ld, C.byref(unit), 1 if paired else 0, out.data_ptr(), SEQ_DTYPE[out_dtype], _stream_ptr(gu.device)))
     return out
 
 
@@ -246,9 +245,9 @@ def delta_forward(cfg: _DeltaConfig, qkv: torch.Tensor, gb: torch.Tensor, batch,
 
 
 def latattn_config(heads: int, dim: int, rot_dim: int, vdim: int, kv_rank: int, rot_dims: int, scale: float, window: int, eps: float,
-                   page_size: int, cache_dtype, rot_half: bool = False) -> _LatAttnConfig:
+                   page_size: int, cache_dtype, rot_half: bool = False, rot_scale: float = 1.0) -> _LatAttnConfig:
     return _LatAttnConfig(heads, dim, rot_dim, vdim, kv_rank, int(rot_dims), float(scale), int(window), float(eps), int(page_size),
-                          SEQ_DTYPE[cache_dtype], 1 if rot_half else 0)
+                          SEQ_DTYPE[cache_dtype], 1 if rot_half else 0, float(rot_scale))
 
 
 def latattn_prep(cfg: _LatAttnConfig, proj: torch.Tensor, q_off: int, c_off: int, wn: torch.Tensor | None, inv_freq: torch.Tensor,
@@ -267,6 +266,25 @@ def latattn_prep(cfg: _LatAttnConfig, proj: torch.Tensor, q_off: int, c_off: int
         raise KtxError("latattn_prep: cache / latent norm do not fit")
     check(lib.ktx_latattn_prep(C.byref(cfg), T, pp, ldp, q_off, c_off, _ptr(wn), inv_freq.data_ptr(), positions.data_ptr(),
                                cache_loc.data_ptr(), _ptr(cache), q_out.data_ptr(), _stream_ptr(proj.device)))
+
+
+def latattn_latents(cfg: _LatAttnConfig, proj: torch.Tensor, cq_off: int, q_rank: int, c_off: int, wq: torch.Tensor, wn: torch.Tensor,
+                    inv_freq: torch.Tensor, positions: torch.Tensor, cache_loc: torch.Tensor, cache: torch.Tensor, out_dtype) -> torch.Tensor:
+    """The step's latent rows appended to the cache, and the queries' own latent: the q_rank columns of proj at cq_off, RMS-normed with weight
+    wq -> [T, q_rank] of out_dtype (ktx_latattn_latents)."""
+    pp, ldp = _rows_f32(proj, "latattn_latents proj")
+    _f32(wq, "latattn_latents wq"), _f32(wn, "latattn_latents wn"), _i32(positions, "positions"), _i32(cache_loc, "cache_loc")
+    _seq_dev(inv_freq, torch.float64, "latattn_latents inv_freq")
+    T, E = proj.shape[0], cfg.kv_rank + cfg.rot_dim
+    if positions.numel() != T or cache_loc.numel() != T or wq.numel() != q_rank or wn.numel() != cfg.kv_rank or cache.shape[-1] != E or \
+            not cache.is_contiguous() or SEQ_DTYPE.get(cache.dtype) != cfg.cache_dtype or inv_freq.numel() != cfg.rot_dims // 2 or \
+            proj.shape[1] < max(cq_off + q_rank, c_off + E):
+        raise KtxError("latattn_latents: shapes do not fit")
+    out = torch.empty((T, q_rank), dtype=out_dtype, device=proj.device)
+    check(lib.ktx_latattn_latents(C.byref(cfg), T, pp, ldp, int(cq_off), int(q_rank), int(c_off), wq.data_ptr(), wn.data_ptr(), inv_freq.data_ptr(),
+                                  positions.data_ptr(), cache_loc.data_ptr(), cache.data_ptr(), out.data_ptr(), SEQ_DTYPE[out_dtype],
+                                  _stream_ptr(proj.device)))
+    return out
 
 
 def latattn_forward(cfg: _LatAttnConfig, q: torch.Tensor, cache: torch.Tensor, batch, sink: torch.Tensor, nsplit: int = 1,
@@ -346,39 +364,41 @@ def head_gemm(a: torch.Tensor, a_goff: int, w: torch.Tensor, out: torch.Tensor, 
     _gg_types(a, w, out.dtype)
     M = a.shape[0]
     check(lib.ktx_grouped_gemm(G, M, N, K, a.data_ptr(), SEQ_DTYPE[a.dtype], a.stride(0), a_goff, None, w.data_ptr(), SEQ_DTYPE[w.dtype],
-                               out.data_ptr(), SEQ_DTYPE[out.dtype], out.stride(0), y_goff, None, None, None, None, 0, TILE_M, 0, _stream_ptr(a.device)))
+                               out.data_ptr(), SEQ_DTYPE[out.dtype], out.stride(0), y_goff, None, None, None, None, 0, TILE_M, 0, None, _stream_ptr(a.device)))
     return out
 
 
 GEMV_MAX_ROWS = 64      # up to this many (token, choice) pairs a step's expert products stream the weights per row instead of tiling
 
 
-GG_ACT = {None: 0, "none": 0, "glu_silu": 1, "relu_sq": 2}
+GG_ACT = {None: 0, "none": 0, "glu_silu": 1, "relu_sq": 2, "glu_pairs": 3}
 
 
 def expert_gemm(a: torch.Tensor, w: torch.Tensor, plan: MoePlan, gather: bool, out_dtype=torch.float32, glu: bool = False,
-                act: str | None = None) -> torch.Tensor:
+                act: str | None = None, unit: _GluAct | None = None) -> torch.Tensor:
     """Sorted row r (expert g = the group it falls in) : out[r] = a[plan.sorted_tok[r] if gather else r] @ w[g]^T.  w [E, N, K]; rows
     of groups >= E (a plan over more groups than there are weights) are left as they are.
     glu (only for steps of at most GEMV_MAX_ROWS pairs): w[g] = [gate ; up] and out[r] = silu(gate a) * (up a), [pairs, N / 2].
-    act = "relu_sq": out = relu(out)^2 in the product's epilogue."""
+    act = "relu_sq": out = relu(out)^2 in the product's epilogue.  unit (ktransformers_amd._native_seq.glu_act; w[g]'s rows alternate gate_f, up_f):
+    out[r] = unit(gate_f a, up_f a) in the epilogue, [pairs, N / 2]."""
     G, N, K = w.shape
     _gg_types(a, w, out_dtype)
-    if glu and act:
-        raise KtxError("expert_gemm: one epilogue")
+    if (glu and act) or (unit is not None and (glu or act)) or (unit is not None and N % 2):
+        raise KtxError("expert_gemm: one epilogue; a gated unit takes pairs of rows")
+    code, uref = (GG_ACT["glu_pairs"], C.byref(unit)) if unit is not None else (GG_ACT["glu_silu" if glu else act], None)
+    n_out = N // 2 if glu or unit is not None else N
     if plan.pairs <= GEMV_MAX_ROWS:
-        n_out = N // 2 if glu else N
         out = torch.empty((plan.pairs, n_out), dtype=out_dtype, device=a.device)
         check(lib.ktx_grouped_gemv(plan.pairs, n_out, K, a.data_ptr(), SEQ_DTYPE[a.dtype], a.stride(0),
                                    plan.sorted_tok.data_ptr() if gather else None, w.data_ptr(), SEQ_DTYPE[w.dtype], out.data_ptr(),
-                                   SEQ_DTYPE[out_dtype], out.stride(0), plan.sorted_group.data_ptr(), 1 if glu else GG_ACT[act], G,
+                                   SEQ_DTYPE[out_dtype], out.stride(0), plan.sorted_group.data_ptr(), code, uref, G,
                                    _stream_ptr(a.device)))
         return out
     if glu:
         raise KtxError("expert_gemm: the fused activation is the streaming form's (at most GEMV_MAX_ROWS pairs)")
-    out = torch.empty((plan.pairs, N), dtype=out_dtype, device=a.device)
+    out = torch.empty((plan.pairs, n_out), dtype=out_dtype, device=a.device)
     check(lib.ktx_grouped_gemm(G, plan.pairs, N, K, a.data_ptr(), SEQ_DTYPE[a.dtype], a.stride(0), 0,
                                plan.sorted_tok.data_ptr() if gather else None, w.data_ptr(), SEQ_DTYPE[w.dtype], out.data_ptr(),
                                SEQ_DTYPE[out_dtype], out.stride(0), 0, plan.group_off.data_ptr(), plan.tile_group.data_ptr(),
-                               plan.tile_row0.data_ptr(), plan.num_tiles.data_ptr(), plan.max_tiles, plan.tile_m, GG_ACT[act], _stream_ptr(a.device)))
+                               plan.tile_row0.data_ptr(), plan.num_tiles.data_ptr(), plan.max_tiles, plan.tile_m, code, uref, _stream_ptr(a.device)))
     return out

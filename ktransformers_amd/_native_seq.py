@@ -30,6 +30,20 @@ class _MlstmConfig(C.Structure):     # include/ktx_seq.h: ktx_mlstm_config
                 ("denom_eps", C.c_float)]
 
 
+class _GluAct(C.Structure):          # include/ktx_seq.h: ktx_glu_act
+    _fields_ = [("kind", C.c_int32), ("limit", C.c_float), ("slope", C.c_float), ("up_shift", C.c_float)]
+
+
+GLU_KIND = {"swish": 0, "gelu_tanh": 1}
+
+
+def glu_act(kind: str = "swish", limit: float | None = None, slope: float = 1.0, up_shift: float = 0.0) -> _GluAct:
+    """A gated linear unit act(g) (u + up_shift) on g = min(gate, limit), u = clamp(up, -limit, limit) (None: unbounded); act = g sigmoid(slope g)
+    ("swish") or the tanh form of GELU."""
+    if limit is not None and not limit > 0:
+        raise KtxError(f"glu_act: the bound must be positive, got {limit}")
+    return _GluAct(GLU_KIND[kind], float("inf") if limit is None else float(limit), float(slope), float(up_shift))
+
 
 def _load() -> C.CDLL:
     have = [p for p in LIB_PATHS if os.path.exists(p)]
@@ -50,7 +64,7 @@ def _load() -> C.CDLL:
         lib.ktx_act_rows.argtypes = [C.c_size_t, C.c_void_p, C.c_int, C.c_int, C.c_float, C.c_void_p]
     if hasattr(lib, "ktx_dense_gemv_glu"):
         lib.ktx_dense_gemv_glu.argtypes = [C.c_int, C.c_int, C.c_int, C.c_void_p, C.c_int, C.c_int64, C.c_void_p, C.c_void_p, C.c_int, C.c_int64,
-                                           C.c_float, C.c_float, C.c_float, C.c_void_p]
+                                           C.POINTER(_GluAct), C.c_void_p]
     lib.ktx_sigattn_prep.argtypes = [C.POINTER(_SigAttnConfig), C.c_int, C.c_void_p, C.c_int64, C.c_int, C.c_int, C.c_void_p, C.c_void_p,
                                      C.c_float] + [C.c_void_p] * 6
     lib.ktx_sigattn_forward.argtypes = [C.POINTER(_SigAttnConfig), C.c_int] + [C.c_void_p] * 9 + [C.c_int, C.c_void_p, C.c_void_p, C.c_int,
@@ -158,17 +172,16 @@ def dense_gemv_glu_eligible(a: torch.Tensor, w: torch.Tensor) -> bool:
             and a.stride(1) == 1 and (a.stride(0) * a.element_size()) % 16 == 0 and a.data_ptr() % 16 == 0 and w.data_ptr() % 16 == 0)
 
 
-def dense_gemv_glu(a: torch.Tensor, w_pairs: torch.Tensor, limit: float | None, slope: float, up_shift: float, out_dtype=torch.float32) -> torch.Tensor:
+def dense_gemv_glu(a: torch.Tensor, w_pairs: torch.Tensor, unit: _GluAct, out_dtype=torch.float32) -> torch.Tensor:
     """Decode-sized GLU front half in one launch (ktx_dense_gemv_glu): a [M <= 16, K] x w_pairs [2F, K] (bf16, rows alternating gate_f,
-    up_f) -> g sigmoid(slope g) (u + up_shift) with the bounded g, u; [M, F] of out_dtype."""
+    up_f) -> unit(gate, up) (glu_act), [M, F] of out_dtype."""
     if not dense_gemv_glu_eligible(a, w_pairs) or not w_pairs.is_contiguous() or w_pairs.shape[1] != a.shape[1] or w_pairs.shape[0] % 2:
         raise KtxError(f"dense_gemv_glu: {a.dtype} {tuple(a.shape)} x {w_pairs.dtype} {tuple(w_pairs.shape)}^T does not fit")
     M, K = a.shape
     Fh = w_pairs.shape[0] // 2
     out = torch.empty((M, Fh), dtype=out_dtype, device=a.device)
     check(lib.ktx_dense_gemv_glu(M, Fh, K, a.data_ptr(), SEQ_DTYPE[a.dtype], a.stride(0), w_pairs.data_ptr(), out.data_ptr(), SEQ_DTYPE[out_dtype],
-                                 out.stride(0), float("inf") if limit is None else float(limit), float(slope), float(up_shift),
-                                 _stream_ptr(a.device)))
+                                 out.stride(0), C.byref(unit), _stream_ptr(a.device)))
     return out
 
 

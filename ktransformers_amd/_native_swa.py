@@ -23,7 +23,7 @@ class _ResidArgs(C.Structure):       # include/ktx_swa.h: ktx_resid_args
 class _SwaConfig(C.Structure):       # include/ktx_swa.h: ktx_swa_config
     _fields_ = [("heads", _I32), ("kv_heads", _I32), ("dim", _I32), ("vdim", _I32), ("rot_dims", _I32), ("rot_values", _I32),
                 ("qk_norm", _I32), ("eps", _F), ("scale", _F), ("window", _I32), ("page_size", _I32), ("cache_dtype", _I32),
-                ("keep_first", _I32), ("bias_span", _I32), ("softcap", _F)]
+                ("keep_first", _I32), ("bias_span", _I32), ("softcap", _F), ("rot_scale", _F)]
 
 
 class _SsmConfig(C.Structure):       # include/ktx_swa.h: ktx_ssm_config
@@ -43,8 +43,8 @@ lib.ktx_swa_mfma.argtypes = [C.POINTER(_SwaConfig), _I, _I, _I, _P, _P, _P, _P, 
 lib.ktx_ssm_conv.argtypes = [C.POINTER(_SsmConfig), _I, _I, _P, _P, _P, _P, _P, _L, _I, _P, _P, _P, _P, _P]
 lib.ktx_ssm_scan.argtypes = [C.POINTER(_SsmConfig), _I, _I, _I, _P, _P, _P, _P, _P, _P, _L, _P, _L, _P, _P, _P, _P, _L, _I, _I, _P, _P, _P,
                              _I, _P]
-lib.ktx_softmax_route.argtypes = [_I, _I, _I, _F, _P, _L, _P, _P, _P, _P]
-lib.ktx_softmax_route_plan.argtypes = [_I, _I, _I, _F, _P, _L, _P, _P, _P, _I, _P, _P, _P, _P, _P, _P, _P, _P]
+lib.ktx_softmax_route.argtypes = [_I, _I, _I, _F, _P, _L, _P, _P, _P, _P, _P]
+lib.ktx_softmax_route_plan.argtypes = [_I, _I, _I, _F, _P, _L, _P, _P, _P, _P, _I, _P, _P, _P, _P, _P, _P, _P, _P]
 
 
 FUSED_CONV_MAX_TAPS = 9      # ktx_resid_norm's one-token form keeps the state rows of one channel in registers
@@ -171,11 +171,13 @@ def rows_mul_lookup(a: torch.Tensor, table: torch.Tensor, col0: int, tokens: tor
 
 
 def swa_config(heads: int, kv_heads: int, dim: int, vdim: int, rot_dims: int, rot_values: bool, qk_norm: bool, eps: float, scale: float,
-               window: int, page_size: int, cache_dtype, keep_first: int = 0, bias_span: int = 0, softcap: float | None = None) -> _SwaConfig:
+               window: int, page_size: int, cache_dtype, keep_first: int = 0, bias_span: int = 0, softcap: float | None = None,
+               rot_scale: float = 1.0) -> _SwaConfig:
     """keep_first: with a window, the sequence's first positions that stay visible; bias_span: rows - 1 of the distance-bias table the
-    attention calls are given (`dist_bias`); softcap: scores become softcap tanh(score / softcap) (None: off)."""
+    attention calls are given (`dist_bias`); softcap: scores become softcap tanh(score / softcap) (None: off); rot_scale: multiplies the
+    cosines and sines that turn q and k."""
     return _SwaConfig(heads, kv_heads, dim, vdim, int(rot_dims), int(bool(rot_values)), int(bool(qk_norm)), float(eps), float(scale),
-                      int(window), int(page_size), SEQ_DTYPE[cache_dtype], int(keep_first), int(bias_span), float(softcap or 0.0))
+                      int(window), int(page_size), SEQ_DTYPE[cache_dtype], int(keep_first), int(bias_span), float(softcap or 0.0), float(rot_scale))
 
 
 def swa_conv_prep(cfg: _SwaConfig, proj: torch.Tensor, bias: torch.Tensor | None, conv_w: torch.Tensor | None, q_norm_w: torch.Tensor | None,
@@ -211,14 +213,19 @@ def swa_conv_prep(cfg: _SwaConfig, proj: torch.Tensor, bias: torch.Tensor | None
 
 
 def swa_prep(cfg: _SwaConfig, proj: torch.Tensor, q_off: int, k_off: int, v_off: int, inv_freq: torch.Tensor | None,
-             v_inv_freq: torch.Tensor | None, positions: torch.Tensor, cache_loc: torch.Tensor, kcache: torch.Tensor, vcache: torch.Tensor):
-    """-> (q fp32 [T, heads * dim] rotated, normed, scaled; vcs fp32 [T, vdim] or None); the step's key and value rows are appended."""
+             v_inv_freq: torch.Tensor | None, positions: torch.Tensor, cache_loc: torch.Tensor, kcache: torch.Tensor | None,
+             vcache: torch.Tensor | None):
+    """-> (q fp32 [T, heads * dim] rotated, normed, scaled; vcs fp32 [T, vdim] or None); the step's key and value rows are appended
+    (kcache and vcache None: only the queries — the layer reads another layer's rows)."""
     pp, ldp = _rows_f32(proj, "swa_prep proj")
     _i32(positions, "positions"), _i32(cache_loc, "cache_loc")
     T = proj.shape[0]
-    if positions.numel() != T or cache_loc.numel() != T or tuple(kcache.shape[1:]) != (cfg.kv_heads, cfg.dim) or \
-            tuple(vcache.shape[1:]) != (cfg.kv_heads, cfg.vdim) or not kcache.is_contiguous() or not vcache.is_contiguous() or \
-            kcache.dtype != vcache.dtype or SEQ_DTYPE.get(kcache.dtype) != cfg.cache_dtype:
+    own = kcache is not None
+    if positions.numel() != T or cache_loc.numel() != T or proj.shape[1] < q_off + cfg.heads * cfg.dim or (not own and vcache is not None) or \
+            (own and (tuple(kcache.shape[1:]) != (cfg.kv_heads, cfg.dim) or
+                      tuple(vcache.shape[1:]) != (cfg.kv_heads, cfg.vdim) or not kcache.is_contiguous() or not vcache.is_contiguous() or
+                      kcache.dtype != vcache.dtype or SEQ_DTYPE.get(kcache.dtype) != cfg.cache_dtype or
+                      proj.shape[1] < max(k_off + cfg.kv_heads * cfg.dim, v_off + cfg.kv_heads * cfg.vdim))):
         raise KtxError("swa_prep: shapes do not fit")
     if cfg.rot_dims and (inv_freq is None or inv_freq.dtype != torch.float64 or inv_freq.numel() != cfg.rot_dims // 2):
         raise KtxError("swa_prep: inv_freq must be fp64 [rot_dims / 2]")
@@ -227,8 +234,8 @@ def swa_prep(cfg: _SwaConfig, proj: torch.Tensor, q_off: int, k_off: int, v_off:
     q = torch.empty((T, cfg.heads * cfg.dim), dtype=torch.float32, device=proj.device)
     vcs = torch.empty((T, cfg.vdim), dtype=torch.float32, device=proj.device) if cfg.rot_values else None
     check(lib.ktx_swa_prep(C.byref(cfg), T, pp, ldp, q_off, k_off, v_off, _ptr(inv_freq) if cfg.rot_dims else None,
-                           _ptr(v_inv_freq) if cfg.rot_values else None, positions.data_ptr(), cache_loc.data_ptr(), kcache.data_ptr(),
-                           vcache.data_ptr(), q.data_ptr(), _ptr(vcs), _stream_ptr(proj.device)))
+                           _ptr(v_inv_freq) if cfg.rot_values else None, positions.data_ptr(), cache_loc.data_ptr(), _ptr(kcache),
+                           _ptr(vcache), q.data_ptr(), _ptr(vcs), _stream_ptr(proj.device)))
     return q, vcs
 
 
@@ -312,30 +319,31 @@ def ssm_scan(cfg: _SsmConfig, xc: torch.Tensor, Bm: torch.Tensor, Cm: torch.Tens
     return out
 
 
-def softmax_route(logits: torch.Tensor, top: int, sum_eps: float, correction: torch.Tensor | None = None):
-    """logits fp32 rows [T, E] -> (topk_idx int32 [T, top], topk_w fp32 [T, top]) (ktx_softmax_route)."""
+def softmax_route(logits: torch.Tensor, top: int, sum_eps: float, correction: torch.Tensor | None = None, bias: torch.Tensor | None = None):
+    """logits fp32 rows [T, E] -> (topk_idx int32 [T, top], topk_w fp32 [T, top]) (ktx_softmax_route); bias fp32 [E] joins the logits."""
     lp, ldl = _rows_f32(logits, "softmax_route logits")
-    _f32(correction, "softmax_route correction")
+    _f32(correction, "softmax_route correction"), _f32(bias, "softmax_route bias")
     T, E = logits.shape
-    if correction is not None and correction.numel() != E:
+    if any(t is not None and t.numel() != E for t in (correction, bias)):
         raise KtxError("softmax_route: one correction per router output")
     idx = torch.empty((T, top), dtype=torch.int32, device=logits.device)
     w = torch.empty((T, top), dtype=torch.float32, device=logits.device)
-    check(lib.ktx_softmax_route(T, E, top, float(sum_eps), lp, ldl, _ptr(correction), idx.data_ptr(), w.data_ptr(), _stream_ptr(logits.device)))
+    check(lib.ktx_softmax_route(T, E, top, float(sum_eps), lp, ldl, _ptr(bias), _ptr(correction), idx.data_ptr(), w.data_ptr(),
+                                _stream_ptr(logits.device)))
     return idx, w
 
 
 ROUTE_PLAN_MAX_T = 64        # up to this many tokens a step routes and sorts in one launch (ktx_softmax_route_plan takes up to 256)
 
 
-def softmax_route_plan(logits: torch.Tensor, top: int, sum_eps: float, correction: torch.Tensor | None = None):
+def softmax_route_plan(logits: torch.Tensor, top: int, sum_eps: float, correction: torch.Tensor | None = None, bias: torch.Tensor | None = None):
     """softmax_route and the expert sort over all E router outputs (ktransformers_amd._native_hyb.moe_plan, 64-row tiles) in ONE launch,
     for small steps -> (topk_idx, topk_w, plan)."""
     from ktransformers_amd._native_hyb import TILE_M, MoePlan
     lp, ldl = _rows_f32(logits, "softmax_route_plan logits")
-    _f32(correction, "softmax_route_plan correction")
+    _f32(correction, "softmax_route_plan correction"), _f32(bias, "softmax_route_plan bias")
     T, E = logits.shape
-    if correction is not None and correction.numel() != E:
+    if any(t is not None and t.numel() != E for t in (correction, bias)):
         raise KtxError("softmax_route_plan: one correction per router output")
     idx = torch.empty((T, top), dtype=torch.int32, device=logits.device)
     w = torch.empty((T, top), dtype=torch.float32, device=logits.device)
@@ -348,7 +356,7 @@ def softmax_route_plan(logits: torch.Tensor, top: int, sum_eps: float, correctio
                     ("tile_row0", p.max_tiles), ("num_tiles", 1)):
         setattr(p, name, meta[at:at + n])
         at += n
-    check(lib.ktx_softmax_route_plan(T, E, top, float(sum_eps), lp, ldl, _ptr(correction), idx.data_ptr(), w.data_ptr(), p.tile_m,
+    check(lib.ktx_softmax_route_plan(T, E, top, float(sum_eps), lp, ldl, _ptr(bias), _ptr(correction), idx.data_ptr(), w.data_ptr(), p.tile_m,
                                      p.group_off.data_ptr(), p.sorted_tok.data_ptr(), p.pair_pos.data_ptr(), p.sorted_group.data_ptr(),
                                      p.tile_group.data_ptr(), p.tile_row0.data_ptr(), p.num_tiles.data_ptr(), _stream_ptr(logits.device)))
     return idx, w, p

@@ -295,7 +295,9 @@ struct ScanDims {
   int heads, dim, vdim, hpk, L, nch;
   int64_t ldq, ldk, ldv, lda, ldm;
   float q_scale;
+  int act;                                 // != 0: q, k and v pass silu on their way in
 };
+__device__ __forceinline__ float silu_fast(float z) { return z * sigmoid_fast(z); }
 
 template <int R, bool PH, bool OUT, bool FULL>
 __device__ __forceinline__ void scan_token(const ScanDims& c, float (&S)[R], int live, const float* __restrict__ kr, const float* __restrict__ qr,
@@ -309,6 +311,30 @@ __device__ __forceinline__ void scan_token(const ScanDims& c, float (&S)[R], int
     S[i] = fmaf(kk, vv, aa * S[i]);
     if constexpr (OUT) {
       const float qq = ok ? qr[i] : 0.f;
+      if (i & 1) acc1 = fmaf(S[i], qq, acc1);
+      else acc0 = fmaf(S[i], qq, acc0);
+    }
+  }
+}
+
+// the same with silu on keys and queries: lanes 0 .. R - 1 take the keys, lanes R .. 2 R - 1 the queries of the wavefront's rows, one activation
+// per lane, and hand them out
+template <int R, bool PH, bool OUT, bool FULL>
+__device__ __forceinline__ void scan_token_act(const ScanDims& c, float (&S)[R], int live, int lane, const float* __restrict__ kr,
+                                               const float* __restrict__ qr, const float* __restrict__ ar, float vv, float& acc0, float& acc1) {
+  const int i0 = lane & (R - 1);           // (R is a power of two up to 32)
+  const bool isq = OUT && (lane & R);
+  const float z = FULL || i0 < live ? (isq ? qr[i0] : kr[i0]) : 0.f;
+  const int s = __builtin_bit_cast(int, silu_fast(z));
+  const float ah = PH ? ar[0] : 0.f;
+#pragma unroll
+  for (int i = 0; i < R; i++) {
+    const bool ok = FULL || i < live;
+    const float kk = __builtin_bit_cast(float, __builtin_amdgcn_readlane(s, i));
+    const float aa = PH ? ah : (ok ? ar[i] : 0.f);
+    S[i] = fmaf(kk, vv, aa * S[i]);
+    if constexpr (OUT) {
+      const float qq = __builtin_bit_cast(float, __builtin_amdgcn_readlane(s, R + i));
       if (i & 1) acc1 = fmaf(S[i], qq, acc1);
       else acc0 = fmaf(S[i], qq, acc0);
     }
@@ -359,7 +385,12 @@ __global__ void __launch_bounds__(1024) decay_scan_kernel(ScanDims c, const int3
         const size_t t = tb + i;
         const float m = vmul ? vmul[t * c.ldm + h] : 1.0f;
         float a0 = 0.f, a1 = 0.f;
-        scan_token<R, PH, OUT, FULL>(c, S, live, kb + t * c.ldk, OUT ? qb + t * c.ldq : nullptr, ab + t * c.lda, cv[i] * m, a0, a1);
+        if (c.act) {
+          cv[i] = silu_fast(cv[i]);
+          scan_token_act<R, PH, OUT, FULL>(c, S, live, lane, kb + t * c.ldk, OUT ? qb + t * c.ldq : nullptr, ab + t * c.lda, cv[i] * m, a0, a1);
+        } else {
+          scan_token<R, PH, OUT, FULL>(c, S, live, kb + t * c.ldk, OUT ? qb + t * c.ldq : nullptr, ab + t * c.lda, cv[i] * m, a0, a1);
+        }
         if constexpr (OUT) po[i] = fmaf(a0 + a1, c.q_scale, sk * cv[i]);
       }
     }
@@ -477,8 +508,8 @@ __global__ void __launch_bounds__(NT, DT == 8 && NT == 256 && !PH && OUT ? 3 : 4
 #pragma unroll
     for (int n = 0; n < E; n++) {
       const int at = (row0 + n * RS) * DP + cc0;
-      lds[L::KR + at] = rk[n];
-      if constexpr (OUT) lds[L::QR + at] = rq[n] * c.q_scale;
+      lds[L::KR + at] = c.act ? silu_fast(rk[n]) : rk[n];
+      if constexpr (OUT) lds[L::QR + at] = (c.act ? silu_fast(rq[n]) : rq[n]) * c.q_scale;
       if constexpr (!PH) lds[L::AR + at] = ra[n];
     }
     if (tid < SM_T) {
@@ -491,7 +522,7 @@ __global__ void __launch_bounds__(NT, DT == 8 && NT == 256 && !PH && OUT ? 3 : 4
   for (int tb = t0; tb < t1; tb += SM_T) {
     float cv[4];
 #pragma unroll
-    for (int s = 0; s < 4; s++) cv[s] = rv[s];
+    for (int s = 0; s < 4; s++) cv[s] = c.act ? silu_fast(rv[s]) : rv[s];
     if (tb + SM_T < t1) fetch(tb + SM_T);
     __syncthreads();                       // the block's rows are there; the last block's products have been read
     if constexpr (OUT) {
@@ -685,6 +716,9 @@ __device__ __forceinline__ float seg_o(const ktx_gate_seg& s, int t, int c) {
   return s.o_dtype == KTX_SEQ_F32 ? reinterpret_cast<const float*>(s.o)[(size_t)t * s.ldo + c]
                                   : bf16_to_f32(reinterpret_cast<const bf16_t*>(s.o)[(size_t)t * s.ldo + c]);
 }
+__device__ __forceinline__ float seg_gate(const ktx_gate_seg& s, int t, int c) {
+  return s.gate[(size_t)t * s.ldg + (s.gate_div == 1 ? c : c / s.gate_div)];
+}
 __device__ __forceinline__ float seg_act(const ktx_gate_seg& s, float g) { return s.act ? silu_f32(g) : sigmoid_f32(g); }
 
 template <typename OT>
@@ -709,7 +743,7 @@ __global__ void __launch_bounds__(256) gate_segments_kernel(int n_segs, GateSegs
           const int c = lane + i * 64;
           const bool ok = c < nc;
           p[i] = ok ? seg_o(s, t, c0 + c) : 0.f;
-          g[i] = ok ? s.gate[(size_t)t * s.ldg + c0 + c] : 0.f;
+          g[i] = ok ? seg_gate(s, t, c0 + c) : 0.f;
           w[i] = ok && s.group ? s.w[(c0 + c) % s.w_mod] : 1.f;
         }
 #pragma unroll
@@ -733,7 +767,7 @@ __global__ void __launch_bounds__(256) gate_segments_kernel(int n_segs, GateSegs
 #pragma unroll 4
         for (int c = tid; c < s.group; c += 256) {
           float p = seg_o(s, t, c0 + c);
-          if (s.gate_first) p *= seg_act(s, s.gate[(size_t)t * s.ldg + c0 + c]);
+          if (s.gate_first) p *= seg_act(s, seg_gate(s, t, c0 + c));
           row[c] = p;
           ss += p * p;
         }
@@ -741,7 +775,7 @@ __global__ void __launch_bounds__(256) gate_segments_kernel(int n_segs, GateSegs
 #pragma unroll 4
         for (int c = tid; c < s.group; c += 256) {      // (each thread re-reads only what it wrote)
           float p = row[c] * r * s.w[(c0 + c) % s.w_mod];
-          if (!s.gate_first) p *= seg_act(s, s.gate[(size_t)t * s.ldg + c0 + c]);
+          if (!s.gate_first) p *= seg_act(s, seg_gate(s, t, c0 + c));
           st_elem(orow, c0 + c, p);
         }
       }
@@ -877,7 +911,7 @@ int ktx_decay_scan(int B, int T, int max_q_len, const int32_t* d_q_indptr, const
   const int nch = scan_chunks(a, max_q_len);
   KTX_REQUIRE(nch == 1 || a->scratch, "ktx_decay_scan: chunks need scratch");
   hipStream_t st = (hipStream_t)stream;
-  ScanDims c{a->heads, a->dim, a->vdim, a->heads_per_key, nch == 1 ? max_q_len : a->chunk_len, nch, a->ldq, a->ldk, a->ldv, a->lda, a->ldm, a->q_scale};
+  ScanDims c{a->heads, a->dim, a->vdim, a->heads_per_key, nch == 1 ? max_q_len : a->chunk_len, nch, a->ldq, a->ldk, a->ldv, a->lda, a->ldm, a->q_scale, a->qkv_act};
   // few tokens: many short wavefronts, so that the state streams in and out side by side; prompts: long ones, whose fixed work per token
   // (values, read-out) is shared by more rows
   const int R = a->dim > 256 ? 32 : max_q_len <= 4 ? 8 : (a->dim > 128 || a->dim % 32 == 0) ? 32 : a->dim % 16 == 0 ? 16 : 8;
@@ -969,7 +1003,7 @@ int ktx_gate_segments(int T, int n_segs, const ktx_gate_seg* segs, void* d_out, 
   size_t lds = 0;
   for (int i = 0; i < n_segs; i++) {
     const ktx_gate_seg& s = segs[i];
-    KTX_REQUIRE(s.o && s.gate && s.n > 0 && s.group >= 0 && dtype_ok(s.o_dtype) && s.ldo >= s.n && s.ldg >= s.n && s.out_off >= 0 &&
+    KTX_REQUIRE(s.o && s.gate && s.n > 0 && s.group >= 0 && dtype_ok(s.o_dtype) && s.ldo >= s.n && s.gate_div > 0 && s.ldg >= (s.n + s.gate_div - 1) / s.gate_div && s.out_off >= 0 &&
                     ldout >= s.out_off + s.n && (s.act == 0 || s.act == 1),
                 "ktx_gate_segments: rows that hold the segment, a known activation");
     KTX_REQUIRE(s.group == 0 || (s.n % s.group == 0 && s.w && (s.w_mod == s.group || s.w_mod == s.n)), "ktx_gate_segments: groups divide the columns");

@@ -66,7 +66,7 @@ __global__ void __launch_bounds__(256) gated_norm_add_kernel(int W, const float*
                                                              const float* __restrict__ gbias, const float* __restrict__ wn,
                                                              const float* __restrict__ bn, float eps, float* __restrict__ x,
                                                              const float* __restrict__ nw, const float* __restrict__ nb, float neps,
-                                                             OT* __restrict__ nout) {
+                                                             OT* __restrict__ nout, int rms) {
   extern __shared__ float zrow[];
   __shared__ float red[4];
   const int t = blockIdx.x, tid = threadIdx.x;
@@ -83,7 +83,7 @@ __global__ void __launch_bounds__(256) gated_norm_add_kernel(int W, const float*
     zrow[e] = z;
     s += z;
   }
-  const float mean = block_sum256(s, red) / (float)W;
+  const float mean = rms ? 0.f : block_sum256(s, red) / (float)W;
   float q = 0.f;
   for (int e = tid; e < W; e += 256) {
     const float d = zrow[e] - mean;
@@ -98,7 +98,7 @@ __global__ void __launch_bounds__(256) gated_norm_add_kernel(int W, const float*
     s2 += v;
   }
   if (!nw) return;
-  const float mean2 = block_sum256(s2, red) / (float)W;
+  const float mean2 = rms ? 0.f : block_sum256(s2, red) / (float)W;
   float q2 = 0.f;
   for (int e = tid; e < W; e += 256) {
     const float d = zrow[e] - mean2;
@@ -106,6 +106,116 @@ __global__ void __launch_bounds__(256) gated_norm_add_kernel(int W, const float*
   }
   const float r2 = 1.0f / sqrtf(block_sum256(q2, red) / (float)W + neps);
   for (int e = tid; e < W; e += 256) st_elem(nout, (size_t)t * W + e, (zrow[e] - mean2) * r2 * nw[e] + (nb ? nb[e] : 0.f));
+}
+
+// The same update for rows of at most 1024 * EV entries whose pieces are 16-byte aligned, held in registers: a thread owns the four entries at
+// 4 (tid + 256 i), i < EV; everything a phase reads (the result, the residual and the norm's weight; the mixture's rows KB at a time) is
+// requested before any of it is used.
+__device__ __forceinline__ float4 f4_ld(const float* p, bool in) { return in ? *reinterpret_cast<const float4*>(p) : make_float4(0.f, 0.f, 0.f, 0.f); }
+__device__ __forceinline__ float f4_sum(const float4& v) { return (v.x + v.y) + (v.z + v.w); }
+__device__ __forceinline__ float f4_sq(const float4& v) { return (v.x * v.x + v.y * v.y) + (v.z * v.z + v.w * v.w); }
+__device__ __forceinline__ float4 f4_affine(const float4& v, float r, const float4& w, const float4& b) {
+  return make_float4(v.x * r * w.x + b.x, v.y * r * w.y + b.y, v.z * r * w.z + b.z, v.w * r * w.w + b.w);
+}
+template <typename OT, int EV, bool RMS>
+__global__ void __launch_bounds__(256) gated_norm_vec_kernel(int W, const float* __restrict__ y, int64_t ldy,
+                                                             const float* __restrict__ ybias, const float* __restrict__ ey,
+                                                             const int32_t* __restrict__ pair_pos, const float* __restrict__ topk_w,
+                                                             int top, const float* __restrict__ gl, int64_t ldg,
+                                                             const float* __restrict__ gbias, const float* __restrict__ wn,
+                                                             const float* __restrict__ bn, float eps, float* __restrict__ x,
+                                                             const float* __restrict__ nw, const float* __restrict__ nb, float neps,
+                                                             OT* __restrict__ nout) {
+  constexpr int KB = EV <= 2 ? 4 : 2;
+  __shared__ float red[4];
+  const int t = blockIdx.x, tid = threadIdx.x;
+  const size_t ro = (size_t)t * W;
+  float4 z[EV], xv[EV], wv[EV], bv[EV];
+  auto at = [&](int i) { return (tid + i * 256) * 4; };
+#pragma unroll
+  for (int i = 0; i < EV; i++) {
+    const int e = at(i);
+    z[i] = f4_ld(y ? y + (size_t)t * ldy + e : x, y && e < W);
+    xv[i] = f4_ld(x + ro + e, e < W);
+    wv[i] = f4_ld(wn + e, e < W);
+    bv[i] = f4_ld(bn ? bn + e : x, bn && e < W);
+  }
+  if (ybias) {
+#pragma unroll
+    for (int i = 0; i < EV; i++) {
+      const float4 b = f4_ld(ybias + at(i), at(i) < W);
+      z[i] = make_float4(z[i].x + b.x, z[i].y + b.y, z[i].z + b.z, z[i].w + b.w);
+    }
+  }
+  if (ey) {
+    float4 m[EV];
+#pragma unroll
+    for (int i = 0; i < EV; i++) m[i] = make_float4(0.f, 0.f, 0.f, 0.f);
+    for (int k0 = 0; k0 < top; k0 += KB) {
+      float4 part[KB][EV];
+      float wk[KB];
+#pragma unroll
+      for (int k = 0; k < KB; k++) {
+        const bool ok = k0 + k < top;
+        wk[k] = ok ? topk_w[(size_t)t * top + k0 + k] : 0.f;
+        const float* row = ey + (ok ? (size_t)pair_pos[(size_t)t * top + k0 + k] : 0) * W;
+#pragma unroll
+        for (int i = 0; i < EV; i++) part[k][i] = f4_ld(row + at(i), ok && at(i) < W);
+      }
+#pragma unroll
+      for (int k = 0; k < KB; k++)
+#pragma unroll
+        for (int i = 0; i < EV; i++)
+          m[i] = make_float4(m[i].x + wk[k] * part[k][i].x, m[i].y + wk[k] * part[k][i].y, m[i].z + wk[k] * part[k][i].z, m[i].w + wk[k] * part[k][i].w);
+    }
+#pragma unroll
+    for (int i = 0; i < EV; i++) z[i] = make_float4(z[i].x + m[i].x, z[i].y + m[i].y, z[i].z + m[i].z, z[i].w + m[i].w);
+  }
+  if (gl) {
+#pragma unroll
+    for (int i = 0; i < EV; i++) {
+      const int e = at(i);
+      const float4 g = f4_ld(gl + (size_t)t * ldg + e, e < W), b = f4_ld(gbias ? gbias + e : gl, gbias && e < W);
+      z[i] = make_float4(z[i].x * sigmoid_f32(g.x + b.x), z[i].y * sigmoid_f32(g.y + b.y), z[i].z * sigmoid_f32(g.z + b.z), z[i].w * sigmoid_f32(g.w + b.w));
+    }
+  }
+  // v - mean(v) in place (entries beyond W stay 0), returns 1 / sqrt(mean of squares + e)
+  auto centre = [&](float4 (&v)[EV], float e) {
+    if constexpr (!RMS) {
+      float s = 0.f;
+#pragma unroll
+      for (int i = 0; i < EV; i++) s += f4_sum(v[i]);
+      const float mean = block_sum256(s, red) / (float)W;
+#pragma unroll
+      for (int i = 0; i < EV; i++)
+        if (at(i) < W) v[i] = make_float4(v[i].x - mean, v[i].y - mean, v[i].z - mean, v[i].w - mean);
+    }
+    float q = 0.f;
+#pragma unroll
+    for (int i = 0; i < EV; i++) q += f4_sq(v[i]);
+    return 1.0f / sqrtf(block_sum256(q, red) / (float)W + e);
+  };
+  const float r = centre(z, eps);
+#pragma unroll
+  for (int i = 0; i < EV; i++) {
+    const float4 a = f4_affine(z[i], r, wv[i], bv[i]);
+    xv[i] = make_float4(xv[i].x + a.x, xv[i].y + a.y, xv[i].z + a.z, xv[i].w + a.w);
+    const int e = at(i);
+    if (e < W) *reinterpret_cast<float4*>(x + ro + e) = xv[i];
+    wv[i] = f4_ld(nw ? nw + e : x, nw && e < W);
+    bv[i] = f4_ld(nb ? nb + e : x, nb && e < W);
+  }
+  if (!nw) return;
+  const float r2 = centre(xv, neps);
+#pragma unroll
+  for (int i = 0; i < EV; i++) {
+    const float4 a = f4_affine(xv[i], r2, wv[i], bv[i]);
+    const size_t e = ro + at(i);
+    if (at(i) < W) {
+      if constexpr (sizeof(OT) == 2) *reinterpret_cast<uint2*>(nout + e) = make_uint2(ktx_pk_bf16(a.x, a.y), ktx_pk_bf16(a.z, a.w));
+      else *reinterpret_cast<float4*>(nout + e) = a;
+    }
+  }
 }
 
 // v = layer_norm(alpha * x + y + ybias); with a stack: level `level` of it receives v, and with dwa the row handed on is the weighted
@@ -260,18 +370,30 @@ __global__ void __launch_bounds__(256) poly_norm_kernel(int F, const float* __re
   }
 }
 
-// out[r][f] = g * sigmoid(slope * g) * (u + up_shift), g = min(gate, limit), u = clamp(up, -limit, limit); (gate, up) = in[r][f],
-// in[r][F + f], or — paired — in[r][2f], in[r][2f + 1]
+// out[r][f] = glu(gate, up), (gate, up) = in[r][f], in[r][F + f], or — paired — in[r][2f], in[r][2f + 1]
 template <typename OT>
-__global__ void __launch_bounds__(256) glu_clamp_rows_kernel(size_t n, int F, const float* __restrict__ in, int64_t ldi, float limit,
-                                                             float slope, float up_shift, int paired, OT* __restrict__ out) {
+__global__ void __launch_bounds__(256) glu_clamp_rows_kernel(size_t n, int F, const float* __restrict__ in, int64_t ldi, ktx_glu_act glu,
+                                                             int paired, OT* __restrict__ out) {
   const size_t i = (size_t)blockIdx.x * 256 + threadIdx.x;
   if (i >= n) return;
   const size_t r = i / F;
   const int f = (int)(i % F);
   const float gv = paired ? in[r * ldi + 2 * f] : in[r * ldi + f], uv = paired ? in[r * ldi + 2 * f + 1] : in[r * ldi + F + f];
-  const float g = fminf(gv, limit), u = fminf(fmaxf(uv, -limit), limit);
-  st_elem(out, i, g * sigmoid_f32(slope * g) * (u + up_shift));
+  st_elem(out, i, glu_act_f32(gv, uv, glu));
+}
+
+// the paired form, four results per thread (F % 4 == 0, aligned rows)
+template <typename OT>
+__global__ void __launch_bounds__(256) glu_pairs_vec_kernel(int F, const float* __restrict__ in, int64_t ldi, ktx_glu_act glu,
+                                                            OT* __restrict__ out) {
+  const int f = (blockIdx.y * 256 + threadIdx.x) * 4;
+  if (f >= F) return;
+  const float4* p = reinterpret_cast<const float4*>(in + (size_t)blockIdx.x * ldi + 2 * f);
+  const float4 a = p[0], b = p[1];
+  const float4 o = make_float4(glu_act_f32(a.x, a.y, glu), glu_act_f32(a.z, a.w, glu), glu_act_f32(b.x, b.y, glu), glu_act_f32(b.z, b.w, glu));
+  OT* d = out + (size_t)blockIdx.x * F + f;
+  if constexpr (sizeof(OT) == 2) *reinterpret_cast<uint2*>(d) = make_uint2(ktx_pk_bf16(o.x, o.y), ktx_pk_bf16(o.z, o.w));
+  else *reinterpret_cast<float4*>(d) = o;
 }
 
 // out[r][c] = o[r][c] * sigmoid(gate[r][c])
@@ -515,7 +637,64 @@ __global__ void __launch_bounds__(NW * 64) delta_fwd_kernel(ktx_delta_config c, 
 }
 
 // ---------------------------------------------------------------------------------------------------------------------
-// latent attention: prep (one workgroup per token)
+// latent attention: prep (one workgroup per token).  A rotated part in turning: entry j of v; j < rot_dims turns with its partner — its
+// neighbour (pairs 2i, 2i + 1), or, in the half layout, the entry rot_dims / 2 further on (pairs i, i + rot_dims / 2)
+struct LatTurn {
+  const float* cs;                         // cos | sin of the NP angles, times rot_scale
+  int NP;
+  bool half;
+  __device__ __forceinline__ float operator()(const float* v, int j) const {
+    if (j >= 2 * NP) return v[j];
+    const int i = half ? (j < NP ? j : j - NP) : j >> 1;
+    const float a = v[half ? i : 2 * i], b = v[half ? i + NP : 2 * i + 1];
+    const bool second = half ? j >= NP : j & 1;
+    return second ? b * cs[i] + a * cs[NP + i] : a * cs[i] - b * cs[NP + i];
+  }
+};
+__device__ __forceinline__ LatTurn lat_angles(const ktx_latattn_config& c, int pos, const double* __restrict__ inv_freq, float* cs) {
+  const int NP = c.rot_dims / 2;
+  for (int i = threadIdx.x; i < NP; i += 256) {
+    double si, co;
+    sincos((double)pos * inv_freq[i], &si, &co);
+    cs[i] = (float)co * c.rot_scale;
+    cs[NP + i] = (float)si * c.rot_scale;
+  }
+  return LatTurn{cs, NP, c.rot_half != 0};
+}
+// one token's latent row: the first kv_rank entries of lat normed, the rest turned (the norm's barriers also publish the angles)
+template <typename KT>
+__device__ __forceinline__ void lat_row(const ktx_latattn_config& c, const float* __restrict__ lat, const float* __restrict__ wn,
+                                        const LatTurn& turned, KT* __restrict__ row, float* red) {
+  const int L = c.kv_rank, tid = threadIdx.x;
+  float s = 0.f;
+  for (int e = tid; e < L; e += 256) s += lat[e] * lat[e];
+  const float r = 1.0f / sqrtf(block_sum256(s, red) / (float)L + c.eps);
+  for (int e = tid; e < L; e += 256) st_elem(row, e, lat[e] * r * wn[e]);
+  for (int j = tid; j < c.rot_dim; j += 256) st_elem(row, L + j, turned(lat + L, j));
+}
+
+template <typename KT, typename OT>
+__global__ void __launch_bounds__(256) latattn_latents_kernel(ktx_latattn_config c, const float* __restrict__ proj, int64_t ldp, int cq_off,
+                                                              int q_rank, int c_off, const float* __restrict__ wq,
+                                                              const float* __restrict__ wn, const double* __restrict__ inv_freq,
+                                                              const int32_t* __restrict__ pos, const int32_t* __restrict__ cache_loc,
+                                                              KT* __restrict__ cache, OT* __restrict__ q_lat) {
+  extern __shared__ float cs[];
+  __shared__ float red[4];
+  const int t = blockIdx.x, tid = threadIdx.x;
+  const float* base = proj + (size_t)t * ldp;
+  if (blockIdx.y == 0) {                     // the cached row
+    const LatTurn turned = lat_angles(c, pos[t], inv_freq, cs);
+    lat_row(c, base + c_off, wn, turned, cache + (size_t)cache_loc[t] * (c.kv_rank + c.rot_dim), red);
+  } else {                                   // the queries' latent
+    const float* a = base + cq_off;
+    float s = 0.f;
+    for (int e = tid; e < q_rank; e += 256) s += a[e] * a[e];
+    const float r = 1.0f / sqrtf(block_sum256(s, red) / (float)q_rank + c.eps);
+    for (int e = tid; e < q_rank; e += 256) st_elem(q_lat, (size_t)t * q_rank + e, a[e] * r * wq[e]);
+  }
+}
+
 template <typename KT>
 __global__ void __launch_bounds__(256) latattn_prep_kernel(ktx_latattn_config c, const float* __restrict__ proj, int64_t ldp, int q_off,
                                                            int c_off, const float* __restrict__ wn, const double* __restrict__ inv_freq,
@@ -524,38 +703,10 @@ __global__ void __launch_bounds__(256) latattn_prep_kernel(ktx_latattn_config c,
   extern __shared__ float cs[];            // cos | sin of the rot_dims / 2 angles
   __shared__ float red[4];
   const int t = blockIdx.x, tid = threadIdx.x;
-  const int L = c.kv_rank, R = c.rot_dim, E = L + R, NP = c.rot_dims / 2;
-  const double p = (double)pos[t];
-  for (int i = tid; i < NP; i += 256) {
-    const double a = p * inv_freq[i];
-    cs[i] = (float)cos(a);
-    cs[NP + i] = (float)sin(a);
-  }
-  // rotated parts: entry j of a rotated vector; j < rot_dims turns with its partner — its neighbour (pairs 2i, 2i + 1), or, in the
-  // half layout, the entry rot_dims / 2 further on (pairs i, i + rot_dims / 2)
-  const bool half = c.rot_half != 0;
-  auto turned = [&](const float* v, int j) -> float {
-    if (j >= 2 * NP) return v[j];
-    if (half) {
-      const int i = j < NP ? j : j - NP;
-      const float a = v[i], bb = v[i + NP];
-      return j < NP ? a * cs[i] - bb * cs[NP + i] : bb * cs[i] + a * cs[NP + i];
-    }
-    const int i = j >> 1;
-    const float a = v[2 * i], bb = v[2 * i + 1];
-    return (j & 1) ? bb * cs[i] + a * cs[NP + i] : a * cs[i] - bb * cs[NP + i];
-  };
-  if (cache) {                               // (a layer that reads another layer's latent rows has none of its own to append)
-    const float* lat = proj + (size_t)t * ldp + c_off;
-    float s = 0.f;
-    for (int e = tid; e < L; e += 256) s += lat[e] * lat[e];
-    const float r = 1.0f / sqrtf(block_sum256(s, red) / (float)L + c.eps);      // (its barriers also publish cs)
-    KT* row = cache + (size_t)cache_loc[t] * E;
-    for (int e = tid; e < L; e += 256) st_elem(row, e, lat[e] * r * wn[e]);
-    for (int j = tid; j < R; j += 256) st_elem(row, L + j, turned(lat + L, j));
-  } else {
-    __syncthreads();
-  }
+  const int L = c.kv_rank, R = c.rot_dim, E = L + R;
+  const LatTurn turned = lat_angles(c, pos[t], inv_freq, cs);
+  if (cache) lat_row(c, proj + (size_t)t * ldp + c_off, wn, turned, cache + (size_t)cache_loc[t] * E, red);
+  else __syncthreads();                      // (the layer's latent rows are appended elsewhere)
   const int D = c.dim;
   for (int e = tid; e < c.heads * R; e += 256) {
     const int h = e / R, j = e % R;
@@ -995,13 +1146,25 @@ __device__ __forceinline__ float gg_act(float v, int act) {
   return v;
 }
 
+// KTX_GG_ACT_GLU_PAIRS: columns 2f and 2f + 1 of a tile sit in neighbouring lanes; the even one writes their result (N is even: a pair is
+// inside or outside together)
+template <typename YT>
+__device__ __forceinline__ void gg_store(YT* __restrict__ Y, int64_t ldy, int m, int n, bool in, float v, int act, const ktx_glu_act& glu) {
+  if (act == KTX_GG_ACT_GLU_PAIRS) {
+    const float other = ktx_dpp_f<KTX_DPP_QUAD_1032>(v);
+    if (in && !(n & 1)) st_elem(Y, (size_t)m * ldy + (n >> 1), glu_act_f32(v, other, glu));
+  } else if (in) {
+    st_elem(Y, (size_t)m * ldy + n, gg_act(v, act));
+  }
+}
+
 template <typename AT, typename CT, typename YT>
 __global__ void __launch_bounds__(256) grouped_gemm_kernel(int M, int N, int K, const AT* __restrict__ A, int64_t lda, int64_t a_goff,
                                                            const int32_t* __restrict__ a_rows, const CT* __restrict__ W,
                                                            YT* __restrict__ Y, int64_t ldy, int64_t y_goff,
                                                            const int32_t* __restrict__ group_off, const int32_t* __restrict__ tile_group,
                                                            const int32_t* __restrict__ tile_row0, const int32_t* __restrict__ num_tiles,
-                                                           bool vec_a, bool vec_w, int G, int act) {
+                                                           bool vec_a, bool vec_w, int G, int act, ktx_glu_act glu) {
   constexpr int LD = GemmTraits<CT>::LDS_LD;
   __shared__ __attribute__((aligned(16))) CT As[64 * LD];
   __shared__ __attribute__((aligned(16))) CT Ws[64 * LD];
@@ -1068,7 +1231,7 @@ __global__ void __launch_bounds__(256) grouped_gemm_kernel(int M, int N, int K, 
 #pragma unroll
       for (int r = 0; r < 4; r++) {
         const int m = m0 + wm + i * 16 + lq * 4 + r, n = n0 + wn + j * 16 + l16;
-        if (m < m_end && n < N) st_elem(Y, (size_t)m * ldy + n, gg_act(acc[i][j][r], act));
+        gg_store(Y, ldy, m, n, m < m_end && n < N, acc[i][j][r], act, glu);
       }
 }
 
@@ -1080,7 +1243,7 @@ __global__ void __launch_bounds__(256) grouped_gemm128_kernel(int N, int K, cons
                                                               YT* __restrict__ Y, int64_t ldy, const int32_t* __restrict__ group_off,
                                                               const int32_t* __restrict__ tile_group, const int32_t* __restrict__ tile_row0,
                                                               const int32_t* __restrict__ num_tiles, bool vec_a, bool vec_w, int G,
-                                                              int act) {
+                                                              int act, ktx_glu_act glu) {
   constexpr int LD = GemmTraits<bf16_t>::LDS_LD;
   __shared__ __attribute__((aligned(16))) bf16_t As[128 * LD];
   __shared__ __attribute__((aligned(16))) bf16_t Ws[128 * LD];
@@ -1123,29 +1286,29 @@ __global__ void __launch_bounds__(256) grouped_gemm128_kernel(int N, int K, cons
 #pragma unroll
       for (int r = 0; r < 4; r++) {
         const int m = m0 + wm + i * 16 + lq * 4 + r, n = n0 + wn + j * 16 + l16;
-        if (m < m_end && n < N) st_elem(Y, (size_t)m * ldy + n, gg_act(acc[i][j][r], act));
+        gg_store(Y, ldy, m, n, m < m_end && n < N, acc[i][j][r], act, glu);
       }
 }
 
 // the same products for a handful of rows (decode steps): no tile, the weights stream once per row.  Workgroup = (8 output columns,
 // one sorted row); a wavefront owns two columns and its lanes stride over K in 16-byte pieces.  glu: column f pairs rows f and
-// F + f of the group's [2F][K] matrix and writes silu(first) * second.
+// F + f — or, in the paired layout, 2f and 2f + 1 — of the group's [2F][K] matrix and writes silu(first) * second (or the given unit).
 template <typename AT, typename CT, typename YT>
 __global__ void __launch_bounds__(256) grouped_gemv_kernel(int N, int K, const AT* __restrict__ A, int64_t lda,
                                                            const int32_t* __restrict__ a_rows, const CT* __restrict__ W, int w_rows,
                                                            YT* __restrict__ Y, int64_t ldy, const int32_t* __restrict__ row_group,
-                                                           int act, bool vec, int G) {
+                                                           int act, ktx_glu_act unit, bool vec, int G) {
   const int r = blockIdx.y, wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
   if (row_group[r] >= G) return;         // a group without weights
-  const bool glu = act == KTX_GG_ACT_GLU_SILU;
+  const bool pairs = act == KTX_GG_ACT_GLU_PAIRS, glu = act == KTX_GG_ACT_GLU_SILU || pairs;
   const AT* a = A + (size_t)(a_rows ? a_rows[r] : r) * lda;
   const CT* Wg = W + (size_t)row_group[r] * w_rows * K;
 #pragma unroll
   for (int c2 = 0; c2 < 2; c2++) {
     const int n = blockIdx.x * 8 + wave * 2 + c2;
     if (n >= N) continue;
-    const CT* w0 = Wg + (size_t)n * K;
-    const CT* w1 = Wg + (size_t)(N + n) * K;
+    const CT* w0 = Wg + (size_t)(pairs ? 2 * n : n) * K;
+    const CT* w1 = Wg + (size_t)(pairs ? 2 * n + 1 : N + n) * K;
     float s0 = 0.f, s1 = 0.f;
     if (vec) {
       for (int k = lane * 8; k < K; k += 512) {
@@ -1191,7 +1354,7 @@ __global__ void __launch_bounds__(256) grouped_gemv_kernel(int N, int K, const A
     }
     s0 = wave_sum(s0);
     if (glu) s1 = wave_sum(s1);
-    if (lane == 0) st_elem(Y, (size_t)r * ldy + n, glu ? silu_f32(s0) * s1 : gg_act(s0, act));
+    if (lane == 0) st_elem(Y, (size_t)r * ldy + n, pairs ? glu_act_f32(s0, s1, unit) : glu ? silu_f32(s0) * s1 : gg_act(s0, act));
   }
 }
 
@@ -1224,19 +1387,40 @@ int ktx_layer_norm(int T, int W, const float* d_x, const float* d_w, const float
 int ktx_gated_norm_add(int T, int W, const float* d_y, int64_t ldy, const float* d_ybias, const float* d_ey, const int32_t* d_pair_pos,
                        const float* d_topk_w, int top, const float* d_gl, int64_t ldg, const float* d_gbias, const float* d_wn,
                        const float* d_bn, float eps, float* d_x, const float* d_next_w, const float* d_next_b, float next_eps,
-                       void* d_next_out, int next_dtype, ktx_stream_t stream) {
+                       void* d_next_out, int next_dtype, int rms, ktx_stream_t stream) {
   KTX_REQUIRE(T >= 0 && W > 0 && d_wn && d_x && (d_y || d_ey), "ktx_gated_norm_add: arguments");
   KTX_REQUIRE(!d_ey || (d_pair_pos && d_topk_w && top > 0), "ktx_gated_norm_add: the gathered term needs pair_pos, topk_w and top");
+  KTX_REQUIRE((!d_y || ldy >= W) && (!d_gl || ldg >= W), "ktx_gated_norm_add: row strides");
   KTX_REQUIRE(!d_next_w || (d_next_out && dtype_ok(next_dtype)), "ktx_gated_norm_add: the following norm needs its output");
   KTX_REQUIRE((size_t)W * 4 <= 64 * 1024, "ktx_gated_norm_add: rows up to 16384 entries");
   if (T == 0) return 0;
   hipStream_t st = (hipStream_t)stream;
-  if (d_next_w && next_dtype == KTX_SEQ_BF16)
+  const bool lp = d_next_w && next_dtype == KTX_SEQ_BF16;
+  auto al = [](const void* p) { return !p || aligned16(p); };
+  if (W % 4 == 0 && W <= 4096 && (!d_y || ldy % 4 == 0) && (!d_gl || ldg % 4 == 0) && al(d_y) && al(d_ybias) && al(d_ey) && al(d_gl) && al(d_gbias) &&
+      al(d_wn) && al(d_bn) && al(d_x) && al(d_next_w) && al(d_next_b) && al(d_next_out)) {
+#define KTX_GN_GO(OT, EV, RMS)                                                                                                                    \
+  gated_norm_vec_kernel<OT, EV, RMS><<<T, 256, 0, st>>>(W, d_y, ldy, d_ybias, d_ey, d_pair_pos, d_topk_w, top, d_gl, ldg, d_gbias, d_wn, d_bn, eps, \
+                                                        d_x, d_next_w, d_next_b, next_eps, (OT*)d_next_out)
+#define KTX_GN_EV(OT, RMS)                       \
+  do {                                           \
+    if (W <= 1024) KTX_GN_GO(OT, 1, RMS);        \
+    else if (W <= 2048) KTX_GN_GO(OT, 2, RMS);   \
+    else KTX_GN_GO(OT, 4, RMS);                  \
+  } while (0)
+    if (lp && rms) KTX_GN_EV(bf16_t, true);
+    else if (lp) KTX_GN_EV(bf16_t, false);
+    else if (rms) KTX_GN_EV(float, true);
+    else KTX_GN_EV(float, false);
+#undef KTX_GN_EV
+#undef KTX_GN_GO
+  } else if (lp) {
     gated_norm_add_kernel<bf16_t><<<T, 256, (size_t)W * 4, st>>>(W, d_y, ldy, d_ybias, d_ey, d_pair_pos, d_topk_w, top, d_gl, ldg, d_gbias, d_wn,
-                                                                 d_bn, eps, d_x, d_next_w, d_next_b, next_eps, (bf16_t*)d_next_out);
-  else
+                                                                 d_bn, eps, d_x, d_next_w, d_next_b, next_eps, (bf16_t*)d_next_out, rms);
+  } else {
     gated_norm_add_kernel<float><<<T, 256, (size_t)W * 4, st>>>(W, d_y, ldy, d_ybias, d_ey, d_pair_pos, d_topk_w, top, d_gl, ldg, d_gbias, d_wn,
-                                                                d_bn, eps, d_x, d_next_w, d_next_b, next_eps, (float*)d_next_out);
+                                                                d_bn, eps, d_x, d_next_w, d_next_b, next_eps, (float*)d_next_out, rms);
+  }
   KTX_HIP(hipGetLastError());
   return 0;
 }
@@ -1286,16 +1470,21 @@ int ktx_postnorm_mix(int T, int W, const float* d_x_in, float* d_x_out, const kt
   return 0;
 }
 
-int ktx_glu_clamp_rows(int R, int F, const float* d_in, int64_t ldi, float limit, float slope, float up_shift, int paired, void* d_out,
-                       int out_dtype, ktx_stream_t stream) {
-  KTX_REQUIRE(R >= 0 && F > 0 && d_in && d_out && dtype_ok(out_dtype) && ldi >= 2 * (int64_t)F && limit > 0.f, "ktx_glu_clamp_rows: arguments");
+int ktx_glu_clamp_rows(int R, int F, const float* d_in, int64_t ldi, const ktx_glu_act* glu, int paired, void* d_out, int out_dtype,
+                       ktx_stream_t stream) {
+  KTX_REQUIRE(R >= 0 && F > 0 && d_in && d_out && dtype_ok(out_dtype) && ldi >= 2 * (int64_t)F && glu_act_ok(glu), "ktx_glu_clamp_rows: arguments");
   if (R == 0) return 0;
   const size_t n = (size_t)R * F;
   hipStream_t st = (hipStream_t)stream;
-  if (out_dtype == KTX_SEQ_F32)
-    glu_clamp_rows_kernel<float><<<(unsigned)((n + 255) / 256), 256, 0, st>>>(n, F, d_in, ldi, limit, slope, up_shift, paired, (float*)d_out);
-  else
-    glu_clamp_rows_kernel<bf16_t><<<(unsigned)((n + 255) / 256), 256, 0, st>>>(n, F, d_in, ldi, limit, slope, up_shift, paired, (bf16_t*)d_out);
+  if (paired && F % 4 == 0 && ldi % 4 == 0 && aligned16(d_in) && aligned16(d_out)) {
+    const dim3 grid(R, (F / 4 + 255) / 256);
+    if (out_dtype == KTX_SEQ_F32) glu_pairs_vec_kernel<float><<<grid, 256, 0, st>>>(F, d_in, ldi, *glu, (float*)d_out);
+    else glu_pairs_vec_kernel<bf16_t><<<grid, 256, 0, st>>>(F, d_in, ldi, *glu, (bf16_t*)d_out);
+  } else if (out_dtype == KTX_SEQ_F32) {
+    glu_clamp_rows_kernel<float><<<(unsigned)((n + 255) / 256), 256, 0, st>>>(n, F, d_in, ldi, *glu, paired, (float*)d_out);
+  } else {
+    glu_clamp_rows_kernel<bf16_t><<<(unsigned)((n + 255) / 256), 256, 0, st>>>(n, F, d_in, ldi, *glu, paired, (bf16_t*)d_out);
+  }
   KTX_HIP(hipGetLastError());
   return 0;
 }
@@ -1421,6 +1610,31 @@ int ktx_latattn_prep(const ktx_latattn_config* cfg, int T, const float* d_proj, 
   return 0;
 }
 
+int ktx_latattn_latents(const ktx_latattn_config* cfg, int T, const float* d_proj, int64_t ldp, int cq_off, int q_rank, int c_off,
+                        const float* d_wq, const float* d_wn, const double* d_inv_freq, const int32_t* d_pos, const int32_t* d_cache_loc,
+                        void* d_cache, void* d_q_lat, int q_dtype, ktx_stream_t stream) {
+  if (latattn_check(cfg, "ktx_latattn_latents")) return -1;
+  KTX_REQUIRE(T >= 0 && q_rank > 0 && d_proj && d_wq && d_wn && (d_inv_freq || cfg->rot_dims == 0) && d_pos && d_cache_loc && d_cache && d_q_lat &&
+                  dtype_ok(q_dtype) && cq_off >= 0 && c_off >= 0 && ldp >= cq_off + q_rank && ldp >= c_off + cfg->kv_rank + cfg->rot_dim,
+              "ktx_latattn_latents: rows that hold both latents, pointers");
+  if (T == 0) return 0;
+  hipStream_t st = (hipStream_t)stream;
+  const size_t lds = (size_t)std::max(cfg->rot_dims, 2) * 4;
+#define KTX_LL_GO(KT, OT)                                                                                                             \
+  latattn_latents_kernel<KT, OT><<<dim3(T, 2), 256, lds, st>>>(*cfg, d_proj, ldp, cq_off, q_rank, c_off, d_wq, d_wn, d_inv_freq, d_pos, \
+                                                               d_cache_loc, (KT*)d_cache, (OT*)d_q_lat)
+  if (cfg->cache_dtype == KTX_SEQ_F32) {
+    if (q_dtype == KTX_SEQ_F32) KTX_LL_GO(float, float);
+    else KTX_LL_GO(float, bf16_t);
+  } else {
+    if (q_dtype == KTX_SEQ_F32) KTX_LL_GO(bf16_t, float);
+    else KTX_LL_GO(bf16_t, bf16_t);
+  }
+#undef KTX_LL_GO
+  KTX_HIP(hipGetLastError());
+  return 0;
+}
+
 int ktx_latattn_forward(const ktx_latattn_config* cfg, int T, const float* d_q, const void* d_cache, const int32_t* d_tok_req,
                         const int32_t* d_pos, const int32_t* d_page_indptr, const int32_t* d_page_indices, const float* d_sink,
                         int nsplit, float* d_scratch, void* d_out, int out_dtype, ktx_stream_t stream) {
@@ -1542,9 +1756,11 @@ int ktx_moe_plan(int T, int E, int top, int tile_m, const int32_t* d_topk_idx, i
 int ktx_grouped_gemm(int G, int M, int N, int K, const void* d_A, int a_dtype, int64_t lda, int64_t a_goff, const int32_t* d_a_rows,
                      const void* d_W, int w_dtype, void* d_Y, int y_dtype, int64_t ldy, int64_t y_goff, const int32_t* d_group_off,
                      const int32_t* d_tile_group, const int32_t* d_tile_row0, const int32_t* d_num_tiles, int max_tiles, int tile_m,
-                     int act, ktx_stream_t stream) {
+                     int act, const ktx_glu_act* glu, ktx_stream_t stream) {
   KTX_REQUIRE(G > 0 && M >= 0 && N > 0 && K > 0 && d_A && d_W && d_Y, "ktx_grouped_gemm: G, N, K > 0, pointers");
-  KTX_REQUIRE(act == KTX_GG_ACT_NONE || act == KTX_GG_ACT_RELU_SQ, "ktx_grouped_gemm: epilogue none or relu^2");
+  KTX_REQUIRE(act == KTX_GG_ACT_NONE || act == KTX_GG_ACT_RELU_SQ || (act == KTX_GG_ACT_GLU_PAIRS && N % 2 == 0 && glu_act_ok(glu)),
+              "ktx_grouped_gemm: epilogue none, relu^2, or a gated unit over an even number of columns");
+  const ktx_glu_act unit = act == KTX_GG_ACT_GLU_PAIRS ? *glu : ktx_glu_act{};
   KTX_REQUIRE(dtype_ok(a_dtype) && dtype_ok(w_dtype) && dtype_ok(y_dtype), "ktx_grouped_gemm: unknown element type");
   KTX_REQUIRE(!(w_dtype == KTX_SEQ_F32 && (a_dtype != KTX_SEQ_F32 || y_dtype != KTX_SEQ_F32)),
               "ktx_grouped_gemm: an fp32 product takes and writes fp32");
@@ -1563,7 +1779,8 @@ int ktx_grouped_gemm(int G, int M, int N, int K, const void* d_A, int a_dtype, i
     hipStream_t st1 = (hipStream_t)stream;
 #define KTX_GG128_GO(AT, YT)                                                                                                       \
   grouped_gemm128_kernel<AT, YT><<<grid128, 256, 0, st1>>>(N, K, (const AT*)d_A, lda, d_a_rows, (const bf16_t*)d_W, (YT*)d_Y, ldy, \
-                                                           d_group_off, d_tile_group, d_tile_row0, d_num_tiles, va, vw, G, act)
+                                                           d_group_off, d_tile_group, d_tile_row0, d_num_tiles, va, vw, G, act, \
+                                                           unit)
     if (a_dtype == KTX_SEQ_F32 && y_dtype == KTX_SEQ_F32) KTX_GG128_GO(float, float);
     else if (a_dtype == KTX_SEQ_F32) KTX_GG128_GO(float, bf16_t);
     else if (y_dtype == KTX_SEQ_F32) KTX_GG128_GO(bf16_t, float);
@@ -1581,7 +1798,8 @@ int ktx_grouped_gemm(int G, int M, int N, int K, const void* d_A, int a_dtype, i
   hipStream_t st = (hipStream_t)stream;
 #define KTX_GG_GO(AT, CT, YT)                                                                                                  \
   grouped_gemm_kernel<AT, CT, YT><<<grid, 256, 0, st>>>(M, N, K, (const AT*)d_A, lda, a_goff, d_a_rows, (const CT*)d_W, (YT*)d_Y, ldy, \
-                                                        y_goff, d_group_off, d_tile_group, d_tile_row0, d_num_tiles, vec_a, vec_w, G, act)
+                                                        y_goff, d_group_off, d_tile_group, d_tile_row0, d_num_tiles, vec_a, vec_w, G, act, \
+                                                        unit)
   if (w_dtype == KTX_SEQ_BF16) {
     if (a_dtype == KTX_SEQ_F32 && y_dtype == KTX_SEQ_F32) KTX_GG_GO(float, bf16_t, float);
     else if (a_dtype == KTX_SEQ_F32) KTX_GG_GO(float, bf16_t, bf16_t);
@@ -1596,10 +1814,14 @@ int ktx_grouped_gemm(int G, int M, int N, int K, const void* d_A, int a_dtype, i
 }
 
 int ktx_grouped_gemv(int R, int N, int K, const void* d_A, int a_dtype, int64_t lda, const int32_t* d_a_rows, const void* d_W, int w_dtype,
-                     void* d_Y, int y_dtype, int64_t ldy, const int32_t* d_row_group, int act, int G, ktx_stream_t stream) {
+                     void* d_Y, int y_dtype, int64_t ldy, const int32_t* d_row_group, int act, const ktx_glu_act* glu_unit, int G,
+                     ktx_stream_t stream) {
   KTX_REQUIRE(R >= 0 && N > 0 && K > 0 && G > 0 && d_A && d_W && d_Y && d_row_group, "ktx_grouped_gemv: N, K, G > 0, pointers");
-  KTX_REQUIRE(act == KTX_GG_ACT_NONE || act == KTX_GG_ACT_GLU_SILU || act == KTX_GG_ACT_RELU_SQ, "ktx_grouped_gemv: unknown epilogue");
-  const int glu = act == KTX_GG_ACT_GLU_SILU;
+  KTX_REQUIRE(act == KTX_GG_ACT_NONE || act == KTX_GG_ACT_GLU_SILU || act == KTX_GG_ACT_RELU_SQ ||
+                  (act == KTX_GG_ACT_GLU_PAIRS && glu_act_ok(glu_unit)),
+              "ktx_grouped_gemv: unknown epilogue");
+  const bool glu = act == KTX_GG_ACT_GLU_SILU || act == KTX_GG_ACT_GLU_PAIRS;
+  const ktx_glu_act unit = act == KTX_GG_ACT_GLU_PAIRS ? *glu_unit : ktx_glu_act{};
   KTX_REQUIRE(dtype_ok(a_dtype) && dtype_ok(w_dtype) && dtype_ok(y_dtype), "ktx_grouped_gemv: unknown element type");
   KTX_REQUIRE(R <= 65535, "ktx_grouped_gemv: up to 65535 rows");
   if (R == 0) return 0;
@@ -1610,7 +1832,7 @@ int ktx_grouped_gemv(int R, int N, int K, const void* d_A, int a_dtype, int64_t 
   hipStream_t st = (hipStream_t)stream;
 #define KTX_GV_GO(AT, CT, YT)                                                                                                          \
   grouped_gemv_kernel<AT, CT, YT><<<grid, 256, 0, st>>>(N, K, (const AT*)d_A, lda, d_a_rows, (const CT*)d_W, w_rows, (YT*)d_Y, ldy, \
-                                                        d_row_group, act, vec, G)
+                                                        d_row_group, act, unit, vec, G)
   if (w_dtype == KTX_SEQ_BF16) {
     if (a_dtype == KTX_SEQ_F32 && y_dtype == KTX_SEQ_F32) KTX_GV_GO(float, bf16_t, float);
     else if (a_dtype == KTX_SEQ_F32) KTX_GV_GO(float, bf16_t, bf16_t);

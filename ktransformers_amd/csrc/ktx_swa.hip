@@ -187,15 +187,16 @@ __global__ void __launch_bounds__(256) swa_prep_kernel(ktx_swa_config c, const f
   float* vc = cs + 2 * NP;
   float* row = vc + 2 * NV;                // [H * D | G * D | G * V]: read once, coalesced; the heads' passes below stay in LDS
   const float* base = proj + (size_t)t * ldp;
-  const int nq = H * D, nk = G * D, nv = G * V;
+  const bool own = kcache != nullptr;      // (otherwise only the queries are this layer's)
+  const int nq = H * D, nk = own ? G * D : 0, nv = own ? G * V : 0;
   for (int i = tid; i < nq + nk + nv; i += 256)
     row[i] = base[i < nq ? q_off + i : i < nq + nk ? k_off + (i - nq) : v_off + (i - nq - nk)];
   const double p = (double)pos[t];
   for (int i = tid; i < NP; i += 256) {
     double si, co;
     sincos(p * inv_freq[i], &si, &co);
-    cs[i] = (float)co;
-    cs[NP + i] = (float)si;
+    cs[i] = (float)co * c.rot_scale;
+    cs[NP + i] = (float)si * c.rot_scale;
   }
   for (int i = tid; i < NV; i += 256) {
     double sd, cd;
@@ -215,7 +216,7 @@ __global__ void __launch_bounds__(256) swa_prep_kernel(ktx_swa_config c, const f
     return (j & 1) ? bb * tab[i] + a * tab[np + i] : a * tab[i] - bb * tab[np + i];
   };
   const size_t loc = (size_t)cache_loc[t];
-  for (int u = wave; u < H + 2 * G; u += 4) {
+  for (int u = wave; u < (own ? H + 2 * G : H); u += 4) {
     if (u < H + G) {        // a query or key head: rotate, then norm
       const bool isq = u < H;
       const float* v = row + (size_t)u * D;      // (key heads follow the query heads in the row)
@@ -257,8 +258,8 @@ __device__ __forceinline__ void conv_prep_angles(const ktx_swa_config& c, int po
   for (int i = threadIdx.x; i < NP; i += 256) {
     double si, co;
     sincos((double)pos * inv_freq[i], &si, &co);
-    cs[i] = (float)co;
-    cs[NP + i] = (float)si;
+    cs[i] = (float)co * c.rot_scale;
+    cs[NP + i] = (float)si * c.rot_scale;
   }
 }
 template <typename KT>
@@ -630,7 +631,7 @@ __global__ void __launch_bounds__(256) swa_mfma_kernel(ktx_swa_config c, int T, 
                                                        OT* __restrict__ out) {
   constexpr int V = NT * 16;
   extern __shared__ __attribute__((aligned(16))) unsigned char sm_raw[];
-  const int H = c.heads, G = c.kv_heads, HPG = H / G, D = c.dim, DPP = D + 8, KS = D / 32;
+  const int H = c.heads, G = c.kv_heads, HPG = H / G, D = c.dim, KS = (D + 31) / 32, DPP = KS * 32 + 8;
   bf16_t* Ks = reinterpret_cast<bf16_t*>(sm_raw);            // [SM_KT][DPP]
   bf16_t* Vt = Ks + (size_t)SM_KT * DPP;                      // [V][SM_PST]
   bf16_t* Ps = Vt + (size_t)V * SM_PST;                       // [4][16][SM_PST]
@@ -659,8 +660,8 @@ __global__ void __launch_bounds__(256) swa_mfma_kernel(ktx_swa_config c, int T, 
       float v[8];
 #pragma unroll
       for (int i = 0; i < 8; i++) v[i] = 0.f;
-      if (kk < KS && live) {
-        const int e0 = kk * 32 + lq * 8;
+      const int e0 = kk * 32 + lq * 8;     // (D % 8 == 0: a piece lies inside or outside the head)
+      if (kk < KS && live && e0 < D) {
         const float4 x = *reinterpret_cast<const float4*>(qrow + e0), y = *reinterpret_cast<const float4*>(qrow + e0 + 4);
         v[0] = x.x; v[1] = x.y; v[2] = x.z; v[3] = x.w; v[4] = y.x; v[5] = y.y; v[6] = y.z; v[7] = y.w;
       }
@@ -691,7 +692,7 @@ __global__ void __launch_bounds__(256) swa_mfma_kernel(ktx_swa_config c, int T, 
 #pragma unroll
   for (int n = 0; n < NT; n++) acc[n] = (v4f){0.f, 0.f, 0.f, 0.f};
   const int32_t* pages = page_indices + page_indptr[b];
-  const int ksegs = D / 8, vsegs = V / 8;
+  const int ksegs = KS * 4, vsegs = V / 8;
   bf16_t* Pw = Ps + (size_t)wave * 16 * SM_PST;
   const float icap = c.softcap > 0.f ? 2.8853900817779268f / c.softcap : 0.f;      // 2 log2(e) / cap
   for (int jt = j0; jt < j1; jt += SM_KT) {
@@ -706,7 +707,7 @@ __global__ void __launch_bounds__(256) swa_mfma_kernel(ktx_swa_config c, int T, 
       const int key = idx / ksegs, e0 = (idx % ksegs) * 8;
       uint4 v = make_uint4(0u, 0u, 0u, 0u);
       const int row = rowidx[key];
-      if (row >= 0) v = *reinterpret_cast<const uint4*>(kcache + ((size_t)row * G + g) * D + e0);
+      if (row >= 0 && e0 < D) v = *reinterpret_cast<const uint4*>(kcache + ((size_t)row * G + g) * D + e0);
       *reinterpret_cast<uint4*>(Ks + (size_t)key * DPP + e0) = v;
     }
     for (int idx = tid; idx < SM_KT * vsegs; idx += 256) {
@@ -802,7 +803,7 @@ __global__ void __launch_bounds__(256) swa_mfma_kernel(ktx_swa_config c, int T, 
 }
 
 size_t swa_mfma_lds(const ktx_swa_config& c) {
-  return ((size_t)SM_KT * (c.dim + 8) + (size_t)c.vdim * SM_PST + 4 * 16 * SM_PST) * 2 + SM_KT * 4;
+  return ((size_t)SM_KT * (((c.dim + 31) & ~31) + 8) + (size_t)c.vdim * SM_PST + 4 * 16 * SM_PST) * 2 + SM_KT * 4;
 }
 
 // ---------------------------------------------------------------------------------------------------------------------
@@ -973,13 +974,15 @@ __global__ void __launch_bounds__(256) ssm_scan_kernel(ktx_ssm_config c, const i
 // router: one wavefront per token; lane holds outputs lane, lane + 64, ... (E <= 64 * SR_RE)
 constexpr int SR_RE = 16;
 __device__ __forceinline__ void softmax_route_token(int t, int lane, int E, int top, float sum_eps, const float* __restrict__ logits,
-                                                    int64_t ldl, const float* __restrict__ corr, int32_t* idx, float* wts) {
+                                                    int64_t ldl, const float* __restrict__ bias, const float* __restrict__ corr, int32_t* idx,
+                                                    float* wts) {
   float s[SR_RE], ch[SR_RE];
   float mx = -INFINITY;
 #pragma unroll
   for (int i = 0; i < SR_RE; i++) {
     const int e = lane + i * 64;
-    s[i] = e < E ? logits[(size_t)t * ldl + e] : -INFINITY;
+    s[i] = e < E ? logits[(size_t)t * ldl + e] + (bias ? bias[e] : 0.f) : -INFINITY;
+    ch[i] = s[i];
     mx = fmaxf(mx, s[i]);
   }
   mx = wave_max(mx);
@@ -994,7 +997,7 @@ __device__ __forceinline__ void softmax_route_token(int t, int lane, int E, int 
   for (int i = 0; i < SR_RE; i++) {
     const int e = lane + i * 64;
     s[i] = s[i] / den;
-    ch[i] = e < E ? s[i] + (corr ? corr[e] : 0.f) : -INFINITY;
+    if (corr && e < E) ch[i] = s[i] + corr[e];
   }
   float sum = 0.f;
   for (int k = 0; k < top; k++) {
@@ -1037,22 +1040,23 @@ __device__ __forceinline__ void softmax_route_token(int t, int lane, int E, int 
 }
 
 __global__ void __launch_bounds__(256) softmax_route_kernel(int T, int E, int top, float sum_eps, const float* __restrict__ logits,
-                                                            int64_t ldl, const float* __restrict__ corr, int32_t* __restrict__ idx,
-                                                            float* __restrict__ wts) {
+                                                            int64_t ldl, const float* __restrict__ bias, const float* __restrict__ corr,
+                                                            int32_t* __restrict__ idx, float* __restrict__ wts) {
   const int t = blockIdx.x * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63;
-  if (t < T) softmax_route_token(t, lane, E, top, sum_eps, logits, ldl, corr, idx, wts);
+  if (t < T) softmax_route_token(t, lane, E, top, sum_eps, logits, ldl, bias, corr, idx, wts);
 }
 
 // router and expert sort of a SMALL step (decode) in one launch: the sixteen wavefronts of the one workgroup route the tokens, then the
 // workgroup sorts the pairs it has just written (moe_plan_block)
 __global__ void __launch_bounds__(1024) softmax_route_plan_kernel(int T, int E, int top, float sum_eps, const float* __restrict__ logits,
-                                                                  int64_t ldl, const float* __restrict__ corr, int32_t* idx, float* wts,
+                                                                  int64_t ldl, const float* __restrict__ bias, const float* __restrict__ corr,
+                                                                  int32_t* idx, float* wts,
                                                                   int tile_m, int32_t* __restrict__ group_off,
                                                                   int32_t* __restrict__ sorted_tok, int32_t* __restrict__ pair_pos,
                                                                   int32_t* __restrict__ sorted_group, int32_t* __restrict__ tile_group,
                                                                   int32_t* __restrict__ tile_row0, int32_t* __restrict__ num_tiles) {
   extern __shared__ int32_t pl[];          // counts [E] | offsets [E + 1] | cursor [E]
-  for (int t = threadIdx.x >> 6; t < T; t += 16) softmax_route_token(t, threadIdx.x & 63, E, top, sum_eps, logits, ldl, corr, idx, wts);
+  for (int t = threadIdx.x >> 6; t < T; t += 16) softmax_route_token(t, threadIdx.x & 63, E, top, sum_eps, logits, ldl, bias, corr, idx, wts);
   __threadfence_block();
   __syncthreads();
   moe_plan_block(T * top, E, top, tile_m, idx, group_off, sorted_tok, pair_pos, sorted_group, tile_group, tile_row0, num_tiles, pl);
@@ -1148,7 +1152,8 @@ int ktx_swa_prep(const ktx_swa_config* cfg, int T, const float* d_proj, int64_t 
                  const double* d_inv_freq, const double* d_v_inv_freq, const int32_t* d_pos, const int32_t* d_cache_loc, void* d_kcache,
                  void* d_vcache, float* d_q_out, float* d_vcs, ktx_stream_t stream) {
   if (swa_check(cfg, "ktx_swa_prep")) return -1;
-  KTX_REQUIRE(T >= 0 && d_proj && d_pos && d_cache_loc && d_kcache && d_vcache && d_q_out, "ktx_swa_prep: null pointer");
+  KTX_REQUIRE(T >= 0 && d_proj && d_pos && d_q_out && ((d_cache_loc && d_kcache && d_vcache) || (!d_kcache && !d_vcache && !cfg->rot_values)),
+              "ktx_swa_prep: null pointer");
   KTX_REQUIRE(cfg->rot_dims == 0 || d_inv_freq, "ktx_swa_prep: rotation without frequencies");
   KTX_REQUIRE(!cfg->rot_values || (d_v_inv_freq && d_vcs), "ktx_swa_prep: rotated values need their frequencies and the table");
   if (T == 0) return 0;
@@ -1293,7 +1298,7 @@ int ktx_swa_forward(const ktx_swa_config* cfg, int T, const float* d_q, const vo
 
 int ktx_swa_mfma_eligible(const ktx_swa_config* c) {
   if (!c || c->cache_dtype != KTX_SEQ_BF16) return 0;
-  if (c->dim % 32 != 0 || c->dim > 32 * SM_KSMAX) return 0;
+  if (c->dim % 8 != 0 || c->dim > 32 * SM_KSMAX) return 0;
   const int V = c->vdim;
   if (!((V % 16 == 0 && V >= 16 && V <= 128) || V == 256)) return 0;
   return swa_mfma_lds(*c) <= 150 * 1024;
@@ -1304,7 +1309,7 @@ int ktx_swa_mfma(const ktx_swa_config* cfg, int B, int T, int max_q_len, const f
                  const float* d_sink, const float* d_dist_bias, const float* d_vcs, int nsplit, float* d_scratch, void* d_out, int out_dtype,
                  ktx_stream_t stream) {
   if (swa_check(cfg, "ktx_swa_mfma")) return -1;
-  KTX_REQUIRE(ktx_swa_mfma_eligible(cfg), "ktx_swa_mfma: bf16 caches, dim a multiple of 32 up to 256, vdim a multiple of 16 up to 128, or 256");
+  KTX_REQUIRE(ktx_swa_mfma_eligible(cfg), "ktx_swa_mfma: bf16 caches, dim a multiple of 8 up to 256, vdim a multiple of 16 up to 128, or 256");
   KTX_REQUIRE(B >= 0 && T >= 0 && max_q_len >= 0 && d_q && d_kcache && d_vcache && d_q_indptr && d_pos0 && d_page_indptr &&
                   d_page_indices && d_out && dtype_ok(out_dtype),
               "ktx_swa_mfma: null pointer");
@@ -1406,18 +1411,19 @@ int ktx_ssm_scan(const ktx_ssm_config* cfg, int B, int T, int max_q_len, const i
   return 0;
 }
 
-int ktx_softmax_route(int T, int E, int top, float sum_eps, const float* d_logits, int64_t ldl, const float* d_correction,
+int ktx_softmax_route(int T, int E, int top, float sum_eps, const float* d_logits, int64_t ldl, const float* d_bias, const float* d_correction,
                       int32_t* d_topk_idx, float* d_topk_w, ktx_stream_t stream) {
   KTX_REQUIRE(T >= 0 && E > 0 && top > 0 && top <= E && E <= 64 * SR_RE && d_logits && d_topk_idx && d_topk_w && ldl >= E,
               "ktx_softmax_route: 0 < top <= outputs <= 1024");
   if (T == 0) return 0;
-  softmax_route_kernel<<<(T + 3) / 4, 256, 0, (hipStream_t)stream>>>(T, E, top, sum_eps, d_logits, ldl, d_correction, d_topk_idx, d_topk_w);
+  softmax_route_kernel<<<(T + 3) / 4, 256, 0, (hipStream_t)stream>>>(T, E, top, sum_eps, d_logits, ldl, d_bias, d_correction, d_topk_idx,
+                                                                         d_topk_w);
   KTX_HIP(hipGetLastError());
   return 0;
 }
 
-int ktx_softmax_route_plan(int T, int E, int top, float sum_eps, const float* d_logits, int64_t ldl, const float* d_correction,
-                           int32_t* d_topk_idx, float* d_topk_w, int tile_m, int32_t* d_group_off, int32_t* d_sorted_tok,
+int ktx_softmax_route_plan(int T, int E, int top, float sum_eps, const float* d_logits, int64_t ldl, const float* d_bias,
+                           const float* d_correction, int32_t* d_topk_idx, float* d_topk_w, int tile_m, int32_t* d_group_off, int32_t* d_sorted_tok,
                            int32_t* d_pair_pos, int32_t* d_sorted_group, int32_t* d_tile_group, int32_t* d_tile_row0, int32_t* d_num_tiles,
                            ktx_stream_t stream) {
   KTX_REQUIRE(T >= 0 && T <= KTX_ROUTE_PLAN_MAX_T && E > 0 && top > 0 && top <= E && E <= 64 * SR_RE && d_logits && d_topk_idx && d_topk_w &&
@@ -1425,7 +1431,7 @@ int ktx_softmax_route_plan(int T, int E, int top, float sum_eps, const float* d_
                   d_num_tiles,
               "ktx_softmax_route_plan: a small step (T <= 256), 0 < top <= outputs <= 1024, pointers");
   softmax_route_plan_kernel<<<1, 1024, (size_t)(3 * E + 1) * 4, (hipStream_t)stream>>>(
-      T, E, top, sum_eps, d_logits, ldl, d_correction, d_topk_idx, d_topk_w, tile_m, d_group_off, d_sorted_tok, d_pair_pos, d_sorted_group,
+      T, E, top, sum_eps, d_logits, ldl, d_bias, d_correction, d_topk_idx, d_topk_w, tile_m, d_group_off, d_sorted_tok, d_pair_pos, d_sorted_group,
       d_tile_group, d_tile_row0, d_num_tiles);
   KTX_HIP(hipGetLastError());
   return 0;

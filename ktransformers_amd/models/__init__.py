@@ -100,6 +100,17 @@ def _dunusun_cache(config, max_tokens, max_requests, dtype, device):
     return KHybridCache(dunusun_layer_specs(config), max_tokens, max_requests=max_requests, dtype=dtype, device=device)
 
 
+def _beronex_config(d, dtype):
+    from ktransformers_amd.models.modeling_beronex import make_beronex_config
+    return make_beronex_config(d, dtype)
+
+
+def _beronex_cache(config, max_tokens, max_requests, dtype, device):
+    from ktransformers_amd.models.custom_cache import KHybridCache
+    from ktransformers_amd.models.modeling_beronex import beronex_layer_specs
+    return KHybridCache(beronex_layer_specs(config), max_tokens, max_requests=max_requests, dtype=dtype, device=device)
+
+
 def _cls(module: str, name: str):
     def get():
         import importlib
@@ -124,6 +135,8 @@ MODEL_REGISTRY = {
                           _vigodra_cache, dtypes=(torch.bfloat16, torch.float32)),
     "Dunusun": ModelEntry(_dunusun_config, _cls("ktransformers_amd.models.modeling_dunusun", "DunusunForCausalLM"), "Dunusun.yaml",
                           _dunusun_cache, dtypes=(torch.bfloat16, torch.float32)),
+    "Beronex": ModelEntry(_beronex_config, _cls("ktransformers_amd.models.modeling_beronex", "BeronexForCausalLM"), "Beronex.yaml",
+                          _beronex_cache, dtypes=(torch.bfloat16, torch.float32)),
 }
 
 

@@ -178,12 +178,12 @@ class KHybridCache:
                                  fp32) for grouped-query attention, stored as the attention reads them (rotated, normed);
       "rec": (heads, dim, vdim)   — fp32 state slots S [slots, heads, dim, vdim], n [slots, heads, dim], m [slots, heads] (mLSTM);
       "delta": (heads, dim, vdim) — fp32 state slots S alone (delta rule);
-      "decay": (heads, dim, vdim) — fp32 state slots S alone (gated linear attention, the state-space-dual scan);
+      "decay": (heads, dim, vdim) — fp32 state slots S alone (gated linear and lightning attention, the state-space-dual scan);
       "ssm": (channels, state)    — fp32 state slots S [slots, channels, state] (selective scan);
       "conv": (channels, taps)    — fp32 slots [slots, taps - 1, channels]: the inputs a short causal convolution still needs;
       "pre": [(channels, taps), ...] — the same kind of slots for convolutions on what the layer's sublayers read, one per sublayer
                                  (an entry with taps <= 1 or None holds nothing).
-    A layer that runs several times with the same weights (a repeated block) has one spec, and so one cache or state, per run.
+    A layer that reads another layer's rows has an empty spec.  A layer that runs several times with the same weights (a repeated block) has one spec, and so one cache or state, per run.
     A request holds a list of pages (grown as it grows) and one slot from admit() to release(); freed pages and slots go back on
     LIFO free lists and are handed out again without being cleared: the attention kernels never read past a request's length and
     the recurrences start from zero at position 0 whatever the slot holds.

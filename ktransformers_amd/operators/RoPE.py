@@ -41,6 +41,20 @@ def yarn_inv_freq(dim, base, scaling_factor, original_max_position_embeddings=40
     return freq_inter * (1 - mask) + freq_extra * mask
 
 
+def turning_frequencies(base: float, dims: int, scaling: dict | None = None):
+    """(angle per position of each turning pair, fp64 [dims / 2]; factor on cosines and sines) of a rotation over `dims` entries: base^(-2i / dims),
+    with YaRN scaling {"factor", "original", "fast", "slow"} interpolated towards 1 / factor of that between the pairs that turn `fast` and
+    `slow` times within `original` positions — the frequencies of the attention operators whose kernels take them in fp64."""
+    i = torch.arange(dims // 2, dtype=torch.float64)
+    freq = torch.pow(torch.tensor(float(base), dtype=torch.float64), -2.0 * i / max(dims, 1))
+    if not scaling:
+        return freq, 1.0
+    factor = float(scaling["factor"])
+    lo, hi = yarn_find_correction_range(float(scaling["fast"]), float(scaling["slow"]), dims, float(base), float(scaling["original"]))
+    ramp = torch.clamp((i - lo) / max(hi - lo, 0.001), 0.0, 1.0)
+    return freq / factor * ramp + freq * (1.0 - ramp), 0.1 * math.log(factor) + 1.0
+
+
 class RotaryEmbeddingV3(BaseInjectedModule):
     """Plain RoPE (RoPE.py:64-113)."""
 

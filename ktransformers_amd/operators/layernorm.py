@@ -36,8 +36,9 @@ KQwen2MoeRMSNorm = KQwen3MoeRMSNorm = DeepseekV3RMSNorm = RMSNorm
 class KResidualRMSNorm(BaseInjectedModule):
     """RMS norm of an fp32 residual stream: y / sqrt(mean(y^2) + eps) * w, or * (1 + w) for weights stored around zero (`one_plus`),
     applied to a SUBLAYER'S OUTPUT and added into the residual in the same launch (post-norm decoders: x += norm(f(x))), or written
-    out in the compute type (the model's last norm, with an optional row gather so that only the wanted positions reach the head).
-    include/ktx_seq.h `ktx_rms_combine`.  The checkpoint tensor is the module's key itself (no `.weight` suffix) unless
+    out in the compute type (the model's last norm, with an optional row gather so that only the wanted positions reach the head;
+    a pre-norm).  include/ktx_seq.h `ktx_rms_combine`.  `gated_add(x, y=, ...)` is KLayerNormBias's with RMS norms: the residual update behind a
+    sublayer, a mixture's weighted rows gathered, and the pre-norm of what follows in one launch (include/ktx_hyb.h `ktx_gated_norm_add`).  The checkpoint tensor is the module's key itself (no `.weight` suffix) unless
     `weight_suffix` says otherwise."""
 
     def __init__(self, key: str, gguf_loader, config, orig_module, prefill_device: str = "cuda", generate_device: str = "cuda",
@@ -46,6 +47,7 @@ class KResidualRMSNorm(BaseInjectedModule):
         object.__setattr__(self, "eps", float(orig_module.eps))
         object.__setattr__(self, "one_plus", bool(orig_module.one_plus if one_plus is None else one_plus))
         object.__setattr__(self, "weight_suffix", weight_suffix)
+        object.__setattr__(self, "compute_dtype", getattr(config, "compute_dtype", None))
         object.__setattr__(self, "weight_f32", None)
 
     def load(self):
@@ -58,6 +60,16 @@ class KResidualRMSNorm(BaseInjectedModule):
         from ktransformers_amd._native_seq import rms_combine
         return rms_combine(y, self.weight_f32, self.eps, one_plus=self.one_plus, residual=residual, rows=rows,
                            out_dtype=out_dtype or torch.float32)
+
+    def gated_add(self, x, y=None, expert_rows=None, pair_pos=None, topk_w=None, next_norm=None):
+        """x += norm(y + the weighted expert rows), in place; with next_norm (another KResidualRMSNorm) also returns next_norm(x): (x, h)."""
+        import torch
+        from ktransformers_amd._native_hyb import gated_norm_add
+        if self.one_plus or (next_norm is not None and next_norm.one_plus):
+            raise NotImplementedError(f"{self.key}: weights stored around zero go through forward()")
+        nn_ = None if next_norm is None else (next_norm.weight_f32, None, next_norm.eps, next_norm.compute_dtype or torch.float32)
+        return gated_norm_add(x, self.weight_f32, None, self.eps, y=y, expert_rows=expert_rows, pair_pos=pair_pos, topk_w=topk_w, next_norm=nn_,
+                              rms=True)
 
 
 class KLayerNormBias(BaseInjectedModule):

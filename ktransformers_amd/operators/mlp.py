@@ -172,8 +172,9 @@ class KPolyNormMLP(BaseInjectedModule):
 
 
 class KClampedGLUMLP(BaseInjectedModule):
-    """Three-matrix gated feed-forward on an fp32 residual stream whose halves are bounded before they meet:
-    W_down (g sigmoid(slope g) (u + up_shift)), g = min(W_gate h, limit), u = clamp(W_up h, -limit, limit).  gate and up are one product
+    """Three-matrix gated feed-forward on an fp32 residual stream whose halves may be bounded before they meet:
+    W_down (act(g) (u + up_shift)), g = min(W_gate h, limit), u = clamp(W_up h, -limit, limit); act(g) = g sigmoid(slope g), or with the replaced
+    module's `activation` = "gelu_tanh" the tanh form of GELU.  gate and up are one product
     (merged at load with their rows ALTERNATING, so a pair's two products meet in neighbouring lanes): for decode-sized steps product and
     activation are one launch (include/ktx_seq.h `ktx_dense_gemv_glu`), otherwise the activation follows the product
     (include/ktx_hyb.h `ktx_glu_clamp_rows`, paired form); fp32 out.  limit (None: unbounded),
@@ -182,8 +183,10 @@ class KClampedGLUMLP(BaseInjectedModule):
 
     def __init__(self, key: str, gguf_loader, config, orig_module, prefill_device: str = "cuda", generate_device: str = "cuda", **kwargs):
         BaseInjectedModule.__init__(self, key, gguf_loader, config, orig_module, prefill_device, generate_device, **kwargs)
-        for name in ("width", "ff", "limit", "slope", "up_shift"):
+        for name in ("width", "ff", "limit"):
             object.__setattr__(self, name, getattr(orig_module, name))
+        for name, default in (("slope", 1.0), ("up_shift", 0.0), ("activation", "swish")):
+            object.__setattr__(self, name, getattr(orig_module, name, default))
         object.__setattr__(self, "compute_dtype", getattr(config, "compute_dtype", torch.bfloat16))
         object.__setattr__(self, "w", {})
 
@@ -198,9 +201,11 @@ class KClampedGLUMLP(BaseInjectedModule):
     def forward(self, h: torch.Tensor) -> torch.Tensor:
         """h [T, width] in the compute type -> fp32 [T, width]."""
         from ktransformers_amd._native_hyb import glu_clamp_rows
-        from ktransformers_amd._native_seq import dense_gemm, dense_gemv_glu, dense_gemv_glu_eligible
+        from ktransformers_amd._native_seq import dense_gemm, dense_gemv_glu, dense_gemv_glu_eligible, glu_act
+        if "unit" not in self.w:
+            self.w["unit"] = glu_act(self.activation, self.limit, self.slope, self.up_shift)
         if dense_gemv_glu_eligible(h, self.w["gate_up"]):
-            a = dense_gemv_glu(h, self.w["gate_up"], self.limit, self.slope, self.up_shift, out_dtype=self.compute_dtype)
+            a = dense_gemv_glu(h, self.w["gate_up"], self.w["unit"], out_dtype=self.compute_dtype)
         else:
-            a = glu_clamp_rows(dense_gemm(h, self.w["gate_up"]), self.limit, self.slope, self.up_shift, out_dtype=self.compute_dtype, paired=True)
+            a = glu_clamp_rows(dense_gemm(h, self.w["gate_up"]), self.w["unit"], out_dtype=self.compute_dtype, paired=True)
         return dense_gemm(a, self.w["down"])

@@ -26,7 +26,11 @@ Further options, each off unless the replaced module names it:
     keep_first            the sequence's first positions stay visible behind the window;
     sink = "learned"      the sink's score is `<key>.sink` [heads];
     softcap               the scaled score becomes softcap tanh(score / softcap);
-    gated                 the concatenated heads are multiplied by sigmoid(W_g h) (`<key>.g`) in front of W_o (include/ktx_gla.h `ktx_gate_segments`).
+    gated                 the concatenated heads are multiplied by sigmoid(W_g h) (`<key>.g`) in front of W_o (include/ktx_gla.h `ktx_gate_segments`);
+                          "per_head": one gate per head (`<key>.g` [heads, width]);
+    rot_scaling           YaRN scaling of the rotation (operators/RoPE.py `turning_frequencies`);
+    kv_from = j           the layer has no key and value projections and reads the rows that the layer with cache index j appended in the same step
+                          (equal kv_heads, sizes and rotation), with its own queries, window and scale.
 With any of the first three the prep is `ktx_swa_conv_prep` (q and k turn behind the convolution there; values do not turn, and turning
 heads are not normed).  Inside a parallel mixer (operators/mixers.py) the input projections and the output product are shared with the
 other mixer's (`in_weight_names`, `gated_segment`)."""
@@ -36,6 +40,7 @@ import torch
 from torch import nn
 
 from ktransformers_amd.operators.base_operator import BaseInjectedModule
+from ktransformers_amd.operators.RoPE import turning_frequencies
 from ktransformers_amd.operators.linear import padded_rows
 
 
@@ -52,24 +57,31 @@ class KWindowGQAttention(BaseInjectedModule):
                      "eps", "width"):
             object.__setattr__(self, name, getattr(o, name))
         for name, default in (("qkv_bias", False), ("out_bias_on", False), ("conv_taps", 0), ("proj_norm", False), ("dist_far", None),
-                              ("keep_first", 0), ("sink", None), ("softcap", None), ("gated", False)):
+                              ("keep_first", 0), ("sink", None), ("softcap", None), ("gated", False), ("rot_scaling", None), ("kv_from", None)):
             object.__setattr__(self, name, getattr(o, name, default))
         object.__setattr__(self, "conv_form", bool(self.qkv_bias or self.conv_taps or self.proj_norm))
         if self.conv_form and (self.rot_values or self.qk_norm or (self.rot_dims and self.proj_norm)):
             raise ValueError(f"{key}: biases, a convolution or whole-projection norms go with un-normed heads and values that do not turn")
+        if self.kv_from is not None and (self.conv_form or self.rot_values):
+            raise ValueError(f"{key}: another layer's keys and values go with plain projections")
         object.__setattr__(self, "compute_dtype", getattr(config, "compute_dtype", torch.bfloat16))
         object.__setattr__(self, "w", {})
         object.__setattr__(self, "_cfg", {})
 
     def state_spec(self) -> dict:
-        spec = {"kv": (self.kv_heads, self.dim, self.vdim)}
+        spec = {"kv": (self.kv_heads, self.dim, self.vdim)} if self.kv_from is None else {}
         if self.conv_taps > 1:
             spec["conv"] = (self.heads * self.dim + self.kv_heads * (self.dim + self.vdim), self.conv_taps)
         return spec
 
     def in_weight_names(self):
         H, G, D, V = self.heads, self.kv_heads, self.dim, self.vdim
-        return [("qkv", H * D + G * (D + V))] + ([("g", H * V)] if self.gated else [])
+        own = G * (D + V) if self.kv_from is None else 0
+        return [("qkv", H * D + own)] + ([("g", self.gate_columns)] if self.gated else [])
+
+    @property
+    def gate_columns(self) -> int:
+        return self.heads if self.gated == "per_head" else self.heads * self.vdim
 
     @property
     def out_columns(self) -> int:
@@ -94,19 +106,18 @@ class KWindowGQAttention(BaseInjectedModule):
         ld, dev, cd = self.gguf_loader, torch.device(self.device), self.compute_dtype
         H, G, D, V = self.heads, self.kv_heads, self.dim, self.vdim
         get = lambda n: ld.load_tensor(f"{self.key}.{n}", device=dev).to(cd)
-        q, k, v, o = get("q"), get("k"), get("v"), get("o")
-        if tuple(q.shape) != (H * D, self.width) or tuple(k.shape) != (G * D, self.width) or tuple(v.shape) != (G * V, self.width) or \
-                tuple(o.shape) != (self.width, H * V):
+        own, o = [("q", H * D)] + ([("k", G * D), ("v", G * V)] if self.kv_from is None else []), get("o")
+        qkv = [get(n) for n, _ in own]
+        if any(tuple(t.shape) != (rows, self.width) for t, (_, rows) in zip(qkv, own)) or tuple(o.shape) != (self.width, H * V):
             raise ValueError(f"{self.key}: tensor shapes do not fit heads={H} kv_heads={G} dim={D} vdim={V} width={self.width}")
-        self.w.update(qkv=torch.cat([q, k, v]).contiguous(), o=o.contiguous())
+        self.w.update(qkv=torch.cat(qkv).contiguous(), o=o.contiguous())
         if self.gated:
             self.w["g"] = get("g").contiguous()
-            if tuple(self.w["g"].shape) != (H * V, self.width):
-                raise ValueError(f"{self.key}.g: expected {(H * V, self.width)}, got {tuple(self.w['g'].shape)}")
-        f64 = lambda n: torch.pow(torch.tensor(float(self.rot_base), dtype=torch.float64),
-                                  -2.0 * torch.arange(n // 2, dtype=torch.float64) / max(n, 1)).to(dev)
-        self.w["inv_freq"] = f64(self.rot_dims) if self.rot_dims else None
-        self.w["v_inv_freq"] = f64(V) if self.rot_values else None
+            if tuple(self.w["g"].shape) != (self.gate_columns, self.width):
+                raise ValueError(f"{self.key}.g: expected {(self.gate_columns, self.width)}, got {tuple(self.w['g'].shape)}")
+        freq, self.w["rot_scale"] = turning_frequencies(self.rot_base, self.rot_dims, self.rot_scaling)
+        self.w["inv_freq"] = freq.to(dev) if self.rot_dims else None
+        self.w["v_inv_freq"] = turning_frequencies(self.rot_base, V)[0].to(dev) if self.rot_values else None
         self.w["sink"] = None if self.sink_score is None else torch.full((H,), float(self.sink_score), dtype=torch.float32, device=dev)
         f32 = lambda n: ld.load_tensor(f"{self.key}.{n}", device=dev).to(torch.float32).contiguous()
         if self.sink == "learned":
@@ -138,7 +149,8 @@ class KWindowGQAttention(BaseInjectedModule):
         if k not in self._cfg:
             self._cfg[k] = swa_config(self.heads, self.kv_heads, self.dim, self.vdim, self.rot_dims, self.rot_values, self.qk_norm,
                                       self.eps, self.scale, self.window or 0, cache.page_size, cache.dtype, keep_first=self.keep_first,
-                                      bias_span=0 if self.w["dist_bias"] is None else self.w["dist_bias"].shape[0] - 1, softcap=self.softcap)
+                                      bias_span=0 if self.w["dist_bias"] is None else self.w["dist_bias"].shape[0] - 1, softcap=self.softcap,
+                                      rot_scale=self.w["rot_scale"])
         return self._cfg[k]
 
     def forward(self, h: torch.Tensor, batch, cache, cache_idx: int) -> torch.Tensor:
@@ -157,19 +169,24 @@ class KWindowGQAttention(BaseInjectedModule):
         from ktransformers_amd._native_gla import gate_seg
         (_, n_qkv), (_, n_g) = self.in_weight_names()
         o = self.attend(proj[:, base:base + n_qkv], batch, cache, cache_idx)
-        return gate_seg(o, proj[:, base + n_qkv:base + n_qkv + n_g], "sigmoid", scale=scale)
+        return gate_seg(o, proj[:, base + n_qkv:base + n_qkv + n_g], "sigmoid", scale=scale, gate_div=self.vdim if self.gated == "per_head" else 1)
 
     def attend(self, proj: torch.Tensor, batch, cache, cache_idx: int) -> torch.Tensor:
         """proj fp32 rows with q | k | v at column 0 -> the concatenated heads [T, heads * vdim] in the compute type (no gate, no W_o)."""
         from ktransformers_amd._native_swa import swa_conv_prep, swa_forward, swa_mfma, swa_mfma_eligible, swa_prep
         H, G, D = self.heads, self.kv_heads, self.dim
         cfg, T = self._config(cache), proj.shape[0]
-        kc, vc = cache.k_caches[cache_idx], cache.v_caches[cache_idx]
+        own = self.kv_from is None
+        src = cache_idx if own else self.kv_from
+        kc, vc = cache.k_caches[src], cache.v_caches[src]
+        if kc is None:
+            raise ValueError(f"{self.key}: cache entry {src} holds no key and value rows")
         if self.conv_form:
             q, vcs = swa_conv_prep(cfg, proj, self.w.get("qkv_b"), self.w.get("conv"), self.w.get("q_norm"), self.w.get("k_norm"), batch,
                                    cache.conv[cache_idx] if self.conv_taps > 1 else None, kc, vc, inv_freq=self.w["inv_freq"]), None
         else:
-            q, vcs = swa_prep(cfg, proj, 0, H * D, (H + G) * D, self.w["inv_freq"], self.w["v_inv_freq"], batch.positions, batch.cache_loc, kc, vc)
+            q, vcs = swa_prep(cfg, proj, 0, H * D, (H + G) * D, self.w["inv_freq"], self.w["v_inv_freq"], batch.positions, batch.cache_loc,
+                              kc if own else None, vc if own else None)
         bias = self.w["dist_bias"]
         span = batch.max_kv_len if not self.window else min(batch.max_kv_len, self.window + self.keep_first + batch.max_q_len)
         if self.USE_MATRIX_CORES and kc.dtype == torch.bfloat16 and swa_mfma_eligible(cfg):

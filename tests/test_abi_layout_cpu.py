@@ -15,6 +15,7 @@ PAIRS = [("ktx_moe_config", "_MoeConfig", "ktx_moe.h"), ("ktx_linear_config", "_
          ("ktx_attn_decode_args", "_AttnDecodeArgs", "ktx_attn.h"),
          # (the sequence-mixer structs are mirrored in ktransformers_amd/_native_seq.py)
          ("ktx_sigattn_config", "_SigAttnConfig", "ktx_seq.h"), ("ktx_mlstm_config", "_MlstmConfig", "ktx_seq.h"),
+         ("ktx_glu_act", "_GluAct", "ktx_seq.h"),
          # (ktransformers_amd/_native_hyb.py, _native_swa.py)
          ("ktx_delta_config", "_DeltaConfig", "ktx_hyb.h"), ("ktx_latattn_config", "_LatAttnConfig", "ktx_hyb.h"),
          ("ktx_postnorm_args", "_PostNormArgs", "ktx_hyb.h"),
