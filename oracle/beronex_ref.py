@@ -6,6 +6,7 @@ Notation: x is the residual at all positions (positions count from 0), W a weigh
 `P[name]` a tensor of the checkpoint, `cfg` the parsed config.json."""
 from __future__ import annotations
 
+import copy
 import math
 
 import torch
@@ -147,8 +148,12 @@ def routed(z, top):
     return idx[:, :top], torch.softmax(zs[:, :top], dim=-1)
 
 
+def router_scores(P, pre, h):
+    return h @ P[pre + "router"].T + P[pre + "router.b"]
+
+
 def mixture(P, pre, c, h):
-    idx, w = routed(h @ P[pre + "router"].T + P[pre + "router.b"], c["router"]["top"])
+    idx, w = routed(router_scores(P, pre, h), c["router"]["top"])
     out = torch.zeros_like(h)
     for e in range(c["router"]["experts"]):
         tok, k = torch.nonzero(idx == e, as_tuple=True)
@@ -157,12 +162,13 @@ def mixture(P, pre, c, h):
     return out
 
 
-def run(P, cfg, tokens, dtype=torch.float64):
-    """(logits [T, vocab], residual after every layer [layers, T, width])."""
-    P = {n: (t if t.dtype == torch.int32 else t.to(dtype)) for n, t in P.items()}
+def forward(P, cfg, tokens, dtype=torch.float64, return_layers=False, return_gaps=False):
+    """tokens: list of ids -> logits [T, vocab]; if asked also the residual after every layer [layers, T, width], and per position the
+    smallest distance between the last chosen and the first left-out router score of any mixture (how close a call the routing was)."""
+    P = {n: (t.to(dtype) if t.is_floating_point() else t) for n, t in P.items()}
     eps = float(cfg["norm"]["eps"])
     x = P["embed"][torch.as_tensor(tokens, dtype=torch.long)] * float(cfg["embedding"]["scale"])
-    kept, trail = {}, []
+    kept, trail, gaps = {}, [], torch.full((len(tokens),), float("inf"), dtype=dtype)
     for i, L in enumerate(cfg["layers"]):
         pre, c = f"l{i}.", L["mixer"]
         h = rms_norm(x, P[pre + "norm1"], eps)
@@ -177,7 +183,100 @@ def run(P, cfg, tokens, dtype=torch.float64):
         m = L.get("mlp")
         if m is not None:
             h = rms_norm(x, P[pre + "norm2"], eps)
-            y = dense_feed_forward(P, pre + "mlp.", h) if m["kind"] == "dense" else mixture(P, pre + "mlp.", m, h)
+            if m["kind"] == "dense":
+                y = dense_feed_forward(P, pre + "mlp.", h)
+            else:
+                y = mixture(P, pre + "mlp.", m, h)
+                top = m["router"]["top"]
+                if top < m["router"]["experts"]:
+                    z = torch.sort(router_scores(P, pre + "mlp.", h), dim=-1, descending=True).values
+                    gaps = torch.minimum(gaps, z[:, top - 1] - z[:, top])
             x = x + rms_norm(y, P[pre + "norm2b"], eps)
         trail.append(x)
-    return rms_norm(x, P["final.norm"], eps) @ P["head"].T, torch.stack(trail)
+    logits = rms_norm(x, P["final.norm"], eps) @ P["head"].T
+    extra = ([torch.stack(trail)] if return_layers else []) + ([gaps] if return_gaps else [])
+    return (logits, *extra) if extra else logits
+
+
+# ---- small configurations and random checkpoints for the tests ---------------------------------------------------------------------
+def rot_of(dims, base=500.0, factor=6.0, original=64, fast=8.0, slow=1.0, scaled=True):
+    if not dims:
+        return None
+    return {"base": base, "dims": dims, "scaling": {"factor": factor, "original": original, "fast": fast, "slow": slow} if scaled else None}
+
+
+def dense_mlp(ff=40):
+    return {"kind": "dense", "ff": ff}
+
+
+def moe_mlp(experts=6, top=2, ff=20, limit=1.5):
+    return {"kind": "moe", "expert": {"ff": ff, "limit": limit}, "router": {"experts": experts, "top": top}}
+
+
+def attention_layer(heads=4, kv_heads=2, dim=12, vdim=10, window=9, scale=None, rot=rot_of(8), kv_from=None, mlp="dense"):
+    m = {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": vdim, "mask": {"size": window} if window else None,
+         "scale": scale if scale is not None else 1.7 * dim ** -0.5, "rot": copy.deepcopy(rot)}
+    if kv_from is not None:
+        m["kv_from"] = kv_from
+    return {"type": "attention", "mixer": m, "mlp": dense_mlp() if mlp == "dense" else mlp}
+
+
+def latent_layer(heads=3, dim=10, rot_dim=8, vdim=14, q_rank=18, kv_rank=20, scale=None, rot=rot_of(8, base=300.0, factor=4.0), mlp="dense"):
+    m = {"heads": heads, "dim": dim, "rot_dim": rot_dim, "vdim": vdim, "q_rank": q_rank, "kv_rank": kv_rank,
+         "scale": scale if scale is not None else 1.3 * (dim + rot_dim) ** -0.5, "rot": copy.deepcopy(rot)}
+    return {"type": "latent_attention", "mixer": m, "mlp": dense_mlp() if mlp == "dense" else mlp}
+
+
+def lightning_layer(heads=3, dim=8, vdim=12, decay=None, mlp="dense"):
+    decay = [0.5 + 0.49 * (i + 1) / heads for i in range(heads)] if decay is None else list(decay)
+    return {"type": "lightning", "mixer": {"heads": heads, "dim": dim, "vdim": vdim, "decay": decay}, "mlp": dense_mlp() if mlp == "dense" else mlp}
+
+
+def make_config(layers, width=32, vocab=61, eps=1e-5, embed_scale=3.0):
+    return {"architecture": "Beronex", "width": width, "vocab": vocab, "norm": {"eps": eps}, "embedding": {"scale": embed_scale}, "layers": layers}
+
+
+def random_checkpoint(cfg: dict, seed: int = 0) -> dict:
+    """Random bf16-representable weights with the checkpoint's tensor names for a config of the design."""
+    g = torch.Generator().manual_seed(seed)
+    W = cfg["width"]
+
+    def mat(o, i, s=None):
+        return (torch.randn(o, i, generator=g) * (s if s is not None else 1.0 / math.sqrt(i))).to(torch.bfloat16)
+
+    def vec(k, mean=1.0, s=0.2):
+        return (mean + torch.randn(k, generator=g) * s).to(torch.bfloat16)
+
+    P = {"embed": mat(cfg["vocab"], W, 0.4), "head": mat(cfg["vocab"], W, 2.0 / math.sqrt(W)), "final.norm": vec(W)}
+    for li, layer in enumerate(cfg["layers"]):
+        p, m, c = f"l{li}.", layer["mixer"], layer.get("mlp")
+        for n in ("norm1", "norm1b") + (("norm2", "norm2b") if c else ()):
+            P[p + n] = vec(W, 0.7 if n.endswith("b") else 1.0)
+        H, V = m["heads"], m["vdim"]
+        if layer["type"] == "attention":
+            D, G = m["dim"], m["kv_heads"]
+            for t, rows in (("q", H * D), ("k", G * D), ("v", G * V)) if m.get("kv_from") is None else (("q", H * D),):
+                P[p + f"mix.{t}"] = mat(rows, W)
+            P[p + "mix.g"] = mat(H, W, 1.5 / math.sqrt(W))
+        elif layer["type"] == "latent_attention":
+            D, R, Q, L = m["dim"], m["rot_dim"], m["q_rank"], m["kv_rank"]
+            P[p + "mix.dq"], P[p + "mix.dq.norm"], P[p + "mix.uq"] = mat(Q, W), vec(Q), mat(H * (D + R), Q, 1.3 / math.sqrt(Q))
+            P[p + "mix.dkv"], P[p + "mix.dkv.norm"] = mat(L + R, W), vec(L)
+            P[p + "mix.uk"], P[p + "mix.uv"] = mat(H * D, L), mat(H * V, L)
+        else:
+            for t, rows in (("q", H * m["dim"]), ("k", H * m["dim"]), ("v", H * V), ("g", H * V)):
+                P[p + f"mix.{t}"] = mat(rows, W)
+            P[p + "mix.norm"] = vec(H * V)
+        P[p + "mix.o"] = mat(W, H * V)
+        if c and c["kind"] == "dense":
+            P[p + "mlp.gate"], P[p + "mlp.up"], P[p + "mlp.down"] = mat(c["ff"], W), mat(c["ff"], W), mat(W, c["ff"])
+        elif c:
+            P[p + "mlp.router"], P[p + "mlp.router.b"] = mat(c["router"]["experts"], W, 2.5 / math.sqrt(W)), vec(c["router"]["experts"], 0.0, 1.0)
+            for e in range(c["router"]["experts"]):
+                for t, o, i in (("gate", c["expert"]["ff"], W), ("up", c["expert"]["ff"], W), ("down", W, c["expert"]["ff"])):
+                    P[p + f"mlp.e{e}.{t}"] = mat(o, i, (1.5 if t != "down" else 1.0) / math.sqrt(i))
+    return P
+
+
+def as_double(P: dict) -> dict:
+    return {k: (v.double() if v.is_floating_point() else v) for k, v in P.items()}
