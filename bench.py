@@ -1889,14 +1889,18 @@ def family_measure(args, dev, cfg, loader, timer_cls, window, T, ctx):
     eng = BatchEngine(model, cache, use_graph=not args.no_graph)
     g = torch.Generator().manual_seed(5)
     prompt = torch.randint(0, 32000, (T,), generator=g).tolist()
-    state = {"pairs": 0, "keys": 0}
+    state = {"pairs": 0, "keys": 0, "all_pairs": 0, "all_keys": 0}      # inside the window; without one
     seen = lambda n: min(n, window) if window else n
 
+    def counts():
+        return state["pairs"], state["keys"]
+    counts.unwindowed = lambda: (state["all_pairs"], state["all_keys"])
+
     def prefill():
-        state.update(pairs=sum(seen(i + 1) for i in range(T)), keys=T)
+        state.update(pairs=sum(seen(i + 1) for i in range(T)), keys=T, all_pairs=T * (T + 1) // 2, all_keys=T)
         eng.step([{"id": "p", "tokens": prompt, "want": [T - 1]}], ["p"])
     ms = timed_ms(prefill, 3)
-    with timer_cls(lambda: (state["pairs"], state["keys"])) as kt:
+    with timer_cls(counts) as kt:
         prefill()
     res = {"prefill": {"tok_s": round(T / ms * 1e3, 1), "ms": round(ms, 3), "per_kernel": kt.table(ms)}}
     for B in (1, 8):
@@ -1905,12 +1909,12 @@ def family_measure(args, dev, cfg, loader, timer_cls, window, T, ctx):
         eng.step([{"id": r, "tokens": ctx_prompt, "want": []} for r in ids])
 
         def decode():
-            n = seen(cache.seq_len(ids[0]))
-            state.update(pairs=B * n, keys=B * n)
+            n, n_all = seen(cache.seq_len(ids[0])), cache.seq_len(ids[0])
+            state.update(pairs=B * n, keys=B * n, all_pairs=B * n_all, all_keys=B * n_all)
             eng.step([{"id": r, "tokens": [7], "want": [0]} for r in ids])
         ms = timed_ms(decode, 20)
         eng.use_graph = False           # the per-kernel pass brackets eager launches
-        with timer_cls(lambda: (state["pairs"], state["keys"])) as kt:
+        with timer_cls(counts) as kt:
             decode()
         eng.use_graph = not args.no_graph
         res[f"decode_bs{B}"] = {"tok_s": round(B / ms * 1e3, 1), "ms_per_step": round(ms, 3), "per_kernel": kt.table(ms),
@@ -2429,6 +2433,165 @@ def run_dunusun(args, dev):
     print(json.dumps(line), flush=True)
 
 
+# ---------------------------------------------------------------------------------------------------------------------
+# --beronex: the family of lightning attention, full latent attention with a query latent and head-gated window attention with shared keys
+# (models/modeling_beronex.py) at a few layer sizes, beside Pilavik — the closest existing family: pre- and post-norms around every sublayer
+# of the same fp32 residual, a latent attention, a matrix state per head, dense feed-forwards and mixtures of gated experts — at equal width
+# and depth; Sadosun, whose grouped-query window attention has the like kernels; and Dunusun, whose per-head scan is the like of lightning's
+# ---------------------------------------------------------------------------------------------------------------------
+BERONEX_SIZES = {
+    # per block of 4 layers: attention, lightning, attention on the first one's keys, latent attention; feed-forwards dense, moe, dense, moe
+    "w1024": dict(width=1024, heads=8, kv_heads=2, dim=128, vdim=128, window=1024, s_heads=8, s_dim=128, s_vdim=128, l_heads=8, l_dim=64, l_rot=32,
+                  l_vdim=64, q_rank=512, kv_rank=256, ff=2816, experts=16, top=2, e_ff=704, like="w1024"),
+    "w2048": dict(width=2048, heads=16, kv_heads=4, dim=128, vdim=128, window=1024, s_heads=16, s_dim=128, s_vdim=128, l_heads=16, l_dim=128,
+                  l_rot=64, l_vdim=128, q_rank=768, kv_rank=512, ff=5632, experts=32, top=4, e_ff=704, like="w2048"),
+    "w4096": dict(width=4096, heads=32, kv_heads=8, dim=128, vdim=128, window=2048, s_heads=32, s_dim=128, s_vdim=128, l_heads=32, l_dim=128,
+                  l_rot=64, l_vdim=128, q_rank=1536, kv_rank=512, ff=11008, experts=64, top=6, e_ff=1024, like="w4096"),
+}
+
+
+def beronex_config(sz, n_layers, vocab=32000):
+    rot = lambda dims: {"base": 50000.0, "dims": dims, "scaling": {"factor": 8.0, "original": 4096, "fast": 32.0, "slow": 1.0}}
+    attn = {"heads": sz["heads"], "kv_heads": sz["kv_heads"], "dim": sz["dim"], "vdim": sz["vdim"], "scale": sz["dim"] ** -0.5,
+            "mask": {"size": sz["window"]}, "rot": rot(sz["dim"])}
+    light = {"heads": sz["s_heads"], "dim": sz["s_dim"], "vdim": sz["s_vdim"],
+             "decay": [math.exp(-2.0 ** (-8.0 * (h + 1) / sz["s_heads"])) for h in range(sz["s_heads"])]}
+    lat = {"heads": sz["l_heads"], "dim": sz["l_dim"], "rot_dim": sz["l_rot"], "vdim": sz["l_vdim"], "q_rank": sz["q_rank"], "kv_rank": sz["kv_rank"],
+           "scale": (sz["l_dim"] + sz["l_rot"]) ** -0.5, "rot": rot(sz["l_rot"])}
+    dense = {"kind": "dense", "ff": sz["ff"]}
+    moe = {"kind": "moe", "expert": {"ff": sz["e_ff"], "limit": 7.0}, "router": {"experts": sz["experts"], "top": sz["top"]}}
+    layers = []
+    for i in range(n_layers):
+        kind = ("attention", "lightning", "attention", "latent_attention")[i % 4]
+        mixer = {"lightning": light, "latent_attention": lat, "attention": dict(attn, kv_from=i - 2) if i % 4 == 2 else attn}[kind]
+        layers.append({"type": kind, "mixer": mixer, "mlp": (dense, moe)[i % 2]})
+    return {"architecture": "Beronex", "width": sz["width"], "vocab": vocab, "norm": {"eps": 1e-6}, "embedding": {"scale": 12.0}, "layers": layers}
+
+
+class BerRandomLoader(HybRandomLoader):
+    """Random bf16 weights by tensor name for a Beronex config (names and shapes of models/modeling_beronex.py's checkpoint)."""
+
+    def __init__(self, cfg, dev):
+        self.dev, self.tensor_device_map, self.shapes = dev, {}, {}
+        W, S = cfg["width"], self.shapes
+        S.update({"embed": (cfg["vocab"], W), "head": (cfg["vocab"], W), "final.norm": (W,)})
+        for i, L in enumerate(cfg["layers"]):
+            p, m, c = f"l{i}.", L["mixer"], L.get("mlp")
+            for n in ("norm1", "norm1b") + (("norm2", "norm2b") if c else ()):
+                S[p + n] = (W,)
+            H, V = m["heads"], m["vdim"]
+            S[p + "mix.o"] = (W, H * V)
+            if L["type"] == "attention":
+                D, G = m["dim"], m["kv_heads"]
+                S.update({p + "mix.q": (H * D, W), p + "mix.g": (H, W)})
+                if m.get("kv_from") is None:
+                    S.update({p + "mix.k": (G * D, W), p + "mix.v": (G * V, W)})
+            elif L["type"] == "latent_attention":
+                D, R, Q, Lr = m["dim"], m["rot_dim"], m["q_rank"], m["kv_rank"]
+                S.update({p + "mix.dq": (Q, W), p + "mix.dq.norm": (Q,), p + "mix.uq": (H * (D + R), Q), p + "mix.dkv": (Lr + R, W),
+                          p + "mix.dkv.norm": (Lr,), p + "mix.uk": (H * D, Lr), p + "mix.uv": (H * V, Lr)})
+            else:
+                for t, rows in (("q", H * m["dim"]), ("k", H * m["dim"]), ("v", H * V), ("g", H * V)):
+                    S[p + f"mix.{t}"] = (rows, W)
+                S[p + "mix.norm"] = (H * V,)
+            if c and c["kind"] == "dense":
+                S.update({p + "mlp.gate": (c["ff"], W), p + "mlp.up": (c["ff"], W), p + "mlp.down": (W, c["ff"])})
+            elif c:
+                F = c["expert"]["ff"]
+                S.update({p + "mlp.router": (c["router"]["experts"], W), p + "mlp.router.b": (c["router"]["experts"],)})
+                for e in range(c["router"]["experts"]):
+                    S.update({p + f"mlp.e{e}.gate": (F, W), p + f"mlp.e{e}.up": (F, W), p + f"mlp.e{e}.down": (W, F)})
+
+    def load_tensor(self, name, device="cpu"):
+        t = super().load_tensor(name, device)
+        return t.mul_(0.1).add_(1.0) if name.endswith((".dq.norm", "final.norm")) else t
+
+
+class BerKernelTimer(GlaKernelTimer):
+    """HIP events around every binding a Beronex step calls."""
+    HYB = ("gated_norm_add", "glu_clamp_rows", "latattn_latents", "latattn_prep", "latattn_forward", "latattn_mfma", "head_gemm", "expert_gemm", "moe_plan")
+    SWA = ("swa_prep", "swa_forward", "swa_mfma", "softmax_route", "softmax_route_plan")
+    SEQ = ("embed_rows", "dense_gemm", "dense_gemv_glu", "rms_combine")
+    GLA = ("decay_scan", "gate_segments")
+
+    def _cost(self, name, a, kw, out):
+        nb = lambda t: t.numel() * t.element_size() if isinstance(t, torch.Tensor) else 0
+        if name == "dense_gemv_glu":
+            M, K = a[0].shape
+            return "dense_gemm M=decode", 2.0 * M * a[1].shape[0] * K, M * K * a[0].element_size() + nb(a[1]) + nb(out)
+        if name == "swa_prep" and a[9] is None:
+            return name, 0.0, 2 * a[1].shape[0] * a[0].heads * a[0].dim * 4
+        if name == "latattn_latents":
+            cfg, T = a[0], a[1].shape[0]
+            return name, 0.0, T * (a[3] + cfg.kv_rank + cfg.rot_dim) * 4 + nb(out) + T * (cfg.kv_rank + cfg.rot_dim) * 2
+        if name == "latattn_prep":          # (the queries' rotated parts)
+            return name, 0.0, 2 * a[1].shape[0] * a[0].heads * a[0].rot_dim * 4
+        if name in ("latattn_forward", "latattn_mfma"):      # no window in this family's latent layers
+            cfg, q, cache = a[0], a[1], a[2]
+            pairs, keys = self.kv_len_of.unwindowed()
+            E = cfg.kv_rank + cfg.rot_dim
+            return name, 2.0 * pairs * cfg.heads * (E + cfg.kv_rank), keys * E * cache.element_size() + nb(q) + nb(out)
+        if name == "decay_scan":
+            return super()._cost(name, a[:3] + (a[3][:1],) + a[4:], kw, out) if a[3].stride(0) == 0 else super()._cost(name, a, kw, out)
+        if name == "gated_norm_add":
+            x = a[0]
+            er = kw.get("expert_rows")
+            return name, 0.0, 2 * nb(x) + nb(kw.get("y")) + nb(er) + (nb(out[1]) if isinstance(out, tuple) else 0)
+        return super()._cost(name, a, kw, out)
+
+
+def run_beronex(args, dev):
+    """Prefill (one prompt of --prefill-tokens) and decode (batch 1 and 8 at a 2048-token context) throughput of Beronex at
+    BERONEX_SIZES, each beside Pilavik, Sadosun and Dunusun of equal width and depth, with a per-kernel table and the fraction of its roofline (bf16
+    MFMA peak or HBM peak, whichever bounds).  Random weights, synthetic tokens.  Prints one JSON line; the whole record goes to
+    bench_beronex.json beside this file."""
+    n_layers, T, ctx = args.layers or 4, args.prefill_tokens, 2048
+    sizes = [s for s in (args.beronex.split(",") if args.beronex != "all" else BERONEX_SIZES) if s in BERONEX_SIZES]
+    record = {"metric": "beronex_prefill_decode", "unit": "tok/s", "layers": n_layers, "prefill_tokens": T, "decode_ctx": ctx,
+              "dtype": "bf16 weights / activations / key, value and latent caches, fp32 residual, norms, scores, router, state", "data": "synthetic",
+              "sizes": {}}
+
+    def other(family, name):
+        if family == "pilavik":
+            sz = PILAVIK_SIZES[name]
+            cfg = pilavik_config(sz, n_layers)
+            return cfg, HybRandomLoader(cfg, dev), HybKernelTimer, sz["window"]
+        if family == "sadosun":
+            sz = SADOSUN_SIZES[name]
+            cfg = sadosun_config(sz, n_layers)
+            return cfg, SwaRandomLoader(cfg, dev), SwaKernelTimer, sz["window"]
+        cfg = dunusun_config(DUNUSUN_SIZES[name], n_layers)
+        return cfg, GlaRandomLoader(cfg, dev), GlaKernelTimer, 0
+
+    others = ("pilavik", "sadosun", "dunusun")
+    for name in sizes:
+        sz = BERONEX_SIZES[name]
+        cfg = beronex_config(sz, n_layers)
+        loader = BerRandomLoader(cfg, dev)
+        res = family_measure(args, dev, cfg, loader, BerKernelTimer, sz["window"], T, ctx)
+        active = loader.active_params(cfg)
+        res["weights_GB"] = round(sum(math.prod(v) for k, v in loader.shapes.items() if k != "embed") * 2 / 1e9, 3)
+        res["active_weights_GB"] = round(active * 2 / 1e9, 3)
+        res["decode_bs1"]["frac_of_hbm_peak"] = round(active * 2 / (res["decode_bs1"]["ms_per_step"] * 1e-3) / (HBM_PEAK_GBS * 1e9), 4)
+        for o in others:
+            try:
+                ocfg, ol, timer, window = other(o, sz["like"])
+                res[o] = family_measure(args, dev, ocfg, ol, timer, window, T, ctx)
+                res[o]["active_weights_GB"] = round((ol.active_params(ocfg) - math.prod(ol.shapes.get("side.embed", (0,)))) * 2 / 1e9, 3)
+            except Exception as e:      # the comparison must not lose the new family's numbers
+                res[o] = {"error": f"{type(e).__name__}: {e}"}
+        record["sizes"][name] = res
+        log(f"[beronex] {name}: prefill {res['prefill']['tok_s']} tok/s, decode bs1 {res['decode_bs1']['tok_s']} tok/s, "
+            f"bs8 {res['decode_bs8']['tok_s']} tok/s")
+    with open(os.path.join(ROOT, "bench_beronex.json"), "w") as f:
+        json.dump(record, f, indent=1)
+    line = {"metric": record["metric"], "unit": "tok/s", "layers": n_layers, "data": "synthetic",
+            "sizes": {k: {"prefill": v["prefill"]["tok_s"], "decode_bs1": v["decode_bs1"]["tok_s"], "decode_bs8": v["decode_bs8"]["tok_s"],
+                          **{f"{o}_{w}": v[o].get(w, {}).get("tok_s") for o in others for w in ("prefill", "decode_bs1", "decode_bs8")}}
+                      for k, v in record["sizes"].items()}}
+    print(json.dumps(line), flush=True)
+
+
 def main():
     ap = argparse.ArgumentParser()
     ap.add_argument("--gpus", type=int, default=1)
@@ -2487,6 +2650,11 @@ def main():
                          "soft-capped grouped-query attention beside gated linear attention, a state-space-dual scan, relu^2 feed-forwards) at "
                          "layer sizes from DUNUSUN_SIZES (comma-separated, or 'all'), beside Mitotar and Sadosun of equal width and depth; one "
                          "JSON line, detail in bench_dunusun.json")
+    ap.add_argument("--beronex", default="", metavar="SIZES",
+                    help="instead of the default workload: prefill / decode throughput of the Beronex family (lightning attention, latent attention "
+                         "with a query latent, head-gated window attention with shared keys, GELU-gated feed-forwards and mixtures of bounded "
+                         "experts) at layer sizes from BERONEX_SIZES (comma-separated, or 'all'), beside Pilavik, Sadosun and Dunusun of equal "
+                         "width and depth; one JSON line, detail in bench_beronex.json")
     ap.add_argument("--pmc-child", action="store_true", help=argparse.SUPPRESS)
     ap.add_argument("--trace-child", action="store_true", help=argparse.SUPPRESS)
     args = ap.parse_args()
@@ -2524,6 +2692,10 @@ def main():
     if args.dunusun:
         torch.cuda.set_device(dev)
         run_dunusun(args, dev)
+        return
+    if args.beronex:
+        torch.cuda.set_device(dev)
+        run_beronex(args, dev)
         return
     torch.cuda.set_device(dev)
     if args.pmc_child:

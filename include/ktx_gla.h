@@ -89,7 +89,7 @@ int ktx_decay_scan(int B, int T, int max_q_len, const int32_t* d_q_indptr, const
                    const ktx_decay_scan_args* a, ktx_stream_t stream);
 
 /* ---- gate / norm segments side by side ------------------------------------------------------------------------------------------------ */
-/* out[t][out_off + c] = scale * f(o[t][c], gate[t][c / gate_div]), c < n (gate_div = 1: a gate per column; a head's size: one per head), for up to KTX_GATE_SEGS segments in one launch; per segment
+/* out[t][out_off + c] = scale * f(o[t][c], gate[t][c]), c < n, for up to KTX_GATE_SEGS segments in one launch; per segment
  *   group == 0:                 f = o act(gate)
  *   gate_first == 0:            f = o r w act(gate), r = 1 / sqrt(mean(o^2 over the group of c) + eps)
  *   gate_first != 0:            f = p r w,           p = o act(gate), r = 1 / sqrt(mean(p^2 over the group of c) + eps)
@@ -103,7 +103,7 @@ typedef struct ktx_gate_seg {
   const float* gate;
   int64_t ldg;
   const float* w;
-  int32_t n, group, w_mod, act, gate_first, gate_div;
+  int32_t n, group, w_mod, act, gate_first;
   float eps, scale;
   int32_t out_off;
 } ktx_gate_seg;

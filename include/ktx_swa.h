@@ -123,13 +123,14 @@ int ktx_swa_conv_prep(const ktx_swa_config* cfg, int B, int T, int max_q_len, in
 
 /* out[t][h] = turn_back(sum_j p_j v_j), p = softmax over {cap(q[t][h] . k_j) + dist_bias[min(i - j, bias_span)][h] : j visible to t at
  * position i: j <= i and (i - j < window or j < keep_first)} and, with sink (fp32 [heads]), one more score sink[h] that has no value.
+ * head_gate (fp32 rows of stride ldg, heads entries each; NULL: no gates): a head's result is multiplied by sigmoid(head_gate[t][h]).
  * dist_bias: fp32 [bias_span + 1][heads] or NULL (not scaled: scale is folded into q).  Vector-ALU form, any sizes and either cache type: one token x the query heads of one key head x
  * one key range per workgroup; nsplit key ranges leave partial sums in scratch fp32 [nsplit][T][heads][vdim + 2], merged afterwards.
  * out [T][heads * vdim] of out_dtype. */
 int ktx_swa_forward(const ktx_swa_config* cfg, int T, const float* d_q, const void* d_kcache, const void* d_vcache,
                     const int32_t* d_tok_req, const int32_t* d_pos, const int32_t* d_page_indptr, const int32_t* d_page_indices,
-                    const float* d_sink, const float* d_dist_bias, const float* d_vcs, int nsplit, float* d_scratch, void* d_out,
-                    int out_dtype, ktx_stream_t stream);
+                    const float* d_sink, const float* d_dist_bias, const float* d_vcs, const float* d_head_gate, int64_t ldg, int nsplit,
+                    float* d_scratch, void* d_out, int out_dtype, ktx_stream_t stream);
 
 /* The same operator on the matrix cores for prompts, portions and decode steps: the (token, head) pairs of a request that share a key
  * head are the rows of one query matrix; workgroups of 64 rows walk 32-key tiles, bf16 MFMA for q . k and weights x values, scores /
@@ -137,8 +138,8 @@ int ktx_swa_forward(const ktx_swa_config* cfg, int T, const float* d_q, const vo
 int ktx_swa_mfma_eligible(const ktx_swa_config* cfg);
 int ktx_swa_mfma(const ktx_swa_config* cfg, int B, int T, int max_q_len, const float* d_q, const void* d_kcache, const void* d_vcache,
                  const int32_t* d_q_indptr, const int32_t* d_pos0, const int32_t* d_page_indptr, const int32_t* d_page_indices,
-                 const float* d_sink, const float* d_dist_bias, const float* d_vcs, int nsplit, float* d_scratch, void* d_out, int out_dtype,
-                 ktx_stream_t stream);
+                 const float* d_sink, const float* d_dist_bias, const float* d_vcs, const float* d_head_gate, int64_t ldg, int nsplit,
+                 float* d_scratch, void* d_out, int out_dtype, ktx_stream_t stream);
 
 /* ---- selective scan --------------------------------------------------------------------------------------------------------------- */
 typedef struct ktx_ssm_config {

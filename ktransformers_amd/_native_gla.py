@@ -26,7 +26,7 @@ class _DecayScanArgs(C.Structure):   # include/ktx_gla.h: ktx_decay_scan_args
 
 class _GateSeg(C.Structure):         # include/ktx_gla.h: ktx_gate_seg
     _fields_ = [("o", _P), ("ldo", _L), ("o_dtype", _I32), ("gate", _P), ("ldg", _L), ("w", _P), ("n", _I32), ("group", _I32), ("w_mod", _I32),
-                ("act", _I32), ("gate_first", _I32), ("gate_div", _I32), ("eps", _F), ("scale", _F), ("out_off", _I32)]
+                ("act", _I32), ("gate_first", _I32), ("eps", _F), ("scale", _F), ("out_off", _I32)]
 
 
 if not hasattr(lib, "ktx_decay_scan"):
@@ -169,18 +169,15 @@ def decay_scan(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, decay: torch.T
     return o
 
 
-def gate_seg(o: torch.Tensor, gate: torch.Tensor, act: str, norm: tuple | None = None, gate_first: bool = False, scale: float = 1.0,
-             gate_div: int = 1):
-    """One segment of gate_segments: o [T, n] (fp32 | bf16 rows), gate fp32 rows [T, n], or [T, n / gate_div]: one gate per gate_div columns; norm = (weight fp32, group, eps): RMS norm over
+def gate_seg(o: torch.Tensor, gate: torch.Tensor, act: str, norm: tuple | None = None, gate_first: bool = False, scale: float = 1.0):
+    """One segment of gate_segments: o [T, n] (fp32 | bf16 rows), gate fp32 rows [T, n]; norm = (weight fp32, group, eps): RMS norm over
     groups of `group` columns, weight of `group` (shared by the groups) or n entries; gate_first: the gate multiplies before the norm."""
     gp, ldg = _rows_f32(gate, "gate_seg gate")
-    if not o.is_cuda or o.dtype not in SEQ_DTYPE or o.dim() != 2 or o.stride(1) != 1 or gate.shape[0] != o.shape[0] or \
-            gate.shape[1] * gate_div != o.shape[1]:
+    if not o.is_cuda or o.dtype not in SEQ_DTYPE or o.dim() != 2 or o.stride(1) != 1 or tuple(o.shape) != tuple(gate.shape):
         raise KtxError("gate_seg: o must be rows of the gate's shape")
     s = _GateSeg()
     s.tensors = [o, gate]            # (the struct holds addresses only: the segment keeps what it points to alive)
     s.o, s.ldo, s.o_dtype, s.gate, s.ldg, s.n = o.data_ptr(), o.stride(0), SEQ_DTYPE[o.dtype], gp, ldg, o.shape[1]
-    s.gate_div = int(gate_div)
     s.act, s.gate_first, s.scale = {"sigmoid": 0, "silu": 1}[act], int(bool(gate_first)), float(scale)
     if norm is not None:
         w, group, eps = norm

@@ -37,9 +37,9 @@ lib.ktx_input_conv.argtypes = [_I, _I, _I, _I, _P, _P, _P, _P, _P, _P, _P, _I, _
 lib.ktx_rows_mul_lookup.argtypes = [_I, _I, _P, _L, _P, _I, _L, _I, _P, _P, _I, _P]
 lib.ktx_swa_prep.argtypes = [C.POINTER(_SwaConfig), _I, _P, _L, _I, _I, _I, _P, _P, _P, _P, _P, _P, _P, _P, _P]
 lib.ktx_swa_conv_prep.argtypes = [C.POINTER(_SwaConfig), _I, _I, _I, _I, _P, _L] + [_P] * 15
-lib.ktx_swa_forward.argtypes = [C.POINTER(_SwaConfig), _I, _P, _P, _P, _P, _P, _P, _P, _P, _P, _P, _I, _P, _P, _I, _P]
+lib.ktx_swa_forward.argtypes = [C.POINTER(_SwaConfig), _I] + [_P] * 11 + [_L, _I, _P, _P, _I, _P]
 lib.ktx_swa_mfma_eligible.argtypes = [C.POINTER(_SwaConfig)]
-lib.ktx_swa_mfma.argtypes = [C.POINTER(_SwaConfig), _I, _I, _I, _P, _P, _P, _P, _P, _P, _P, _P, _P, _P, _I, _P, _P, _I, _P]
+lib.ktx_swa_mfma.argtypes = [C.POINTER(_SwaConfig), _I, _I, _I] + [_P] * 11 + [_L, _I, _P, _P, _I, _P]
 lib.ktx_ssm_conv.argtypes = [C.POINTER(_SsmConfig), _I, _I, _P, _P, _P, _P, _P, _L, _I, _P, _P, _P, _P, _P]
 lib.ktx_ssm_scan.argtypes = [C.POINTER(_SsmConfig), _I, _I, _I, _P, _P, _P, _P, _P, _P, _L, _P, _L, _P, _P, _P, _P, _L, _I, _I, _P, _P, _P,
                              _I, _P]
@@ -245,17 +245,28 @@ def _dist_bias_ok(cfg: _SwaConfig, dist_bias) -> None:
         raise KtxError(f"dist_bias: expected fp32 [{cfg.bias_span + 1}, {cfg.heads}], got {tuple(dist_bias.shape)}")
 
 
+def _head_gate(cfg: _SwaConfig, T: int, head_gate):
+    hg, ldg = _rows_f32(head_gate, "head_gate")
+    if head_gate is not None and tuple(head_gate.shape) != (T, cfg.heads):
+        raise KtxError(f"head_gate: expected fp32 [{T}, {cfg.heads}], got {tuple(head_gate.shape)}")
+    return hg, ldg
+
+
 def swa_forward(cfg: _SwaConfig, q: torch.Tensor, kcache: torch.Tensor, vcache: torch.Tensor, batch, sink: torch.Tensor | None,
-                vcs: torch.Tensor | None, nsplit: int = 1, out_dtype=torch.float32, dist_bias: torch.Tensor | None = None) -> torch.Tensor:
+                vcs: torch.Tensor | None, nsplit: int = 1, out_dtype=torch.float32, dist_bias: torch.Tensor | None = None,
+                head_gate: torch.Tensor | None = None) -> torch.Tensor:
     """The vector-ALU form (ktx_swa_forward) -> [T, heads * vdim] of out_dtype.  dist_bias fp32 [cfg.bias_span + 1, heads]: added to the
-    score by distance (the last row serves every larger distance)."""
+    score by distance (the last row serves every larger distance).  head_gate fp32 rows [T, heads]: every head's result times sigmoid of its
+    logit."""
     _f32(q, "swa_forward q"), _f32(sink, "swa_forward sink"), _f32(vcs, "swa_forward vcs"), _dist_bias_ok(cfg, dist_bias)
     T = q.shape[0]
+    hg, ldg = _head_gate(cfg, T, head_gate)
     out = torch.empty((T, cfg.heads * cfg.vdim), dtype=out_dtype, device=q.device)
     scratch = torch.empty((nsplit, T, cfg.heads, cfg.vdim + 2), dtype=torch.float32, device=q.device) if nsplit > 1 else None
     check(lib.ktx_swa_forward(C.byref(cfg), T, q.data_ptr(), kcache.data_ptr(), vcache.data_ptr(), batch.tok_req.data_ptr(),
                               batch.positions.data_ptr(), batch.page_indptr.data_ptr(), batch.page_indices.data_ptr(), _ptr(sink),
-                              _ptr(dist_bias), _ptr(vcs), int(nsplit), _ptr(scratch), out.data_ptr(), SEQ_DTYPE[out_dtype], _stream_ptr(q.device)))
+                              _ptr(dist_bias), _ptr(vcs), hg, ldg, int(nsplit), _ptr(scratch), out.data_ptr(), SEQ_DTYPE[out_dtype],
+                              _stream_ptr(q.device)))
     return out
 
 
@@ -264,15 +275,17 @@ def swa_mfma_eligible(cfg: _SwaConfig) -> bool:
 
 
 def swa_mfma(cfg: _SwaConfig, q: torch.Tensor, kcache: torch.Tensor, vcache: torch.Tensor, batch, sink: torch.Tensor | None,
-             vcs: torch.Tensor | None, nsplit: int = 1, out_dtype=torch.bfloat16, dist_bias: torch.Tensor | None = None) -> torch.Tensor:
+             vcs: torch.Tensor | None, nsplit: int = 1, out_dtype=torch.bfloat16, dist_bias: torch.Tensor | None = None,
+             head_gate: torch.Tensor | None = None) -> torch.Tensor:
     """The matrix-core form, prompts and decode steps (ktx_swa_mfma) -> [T, heads * vdim] of out_dtype."""
     _f32(q, "swa_mfma q"), _f32(sink, "swa_mfma sink"), _f32(vcs, "swa_mfma vcs"), _dist_bias_ok(cfg, dist_bias)
     T = q.shape[0]
+    hg, ldg = _head_gate(cfg, T, head_gate)
     out = torch.empty((T, cfg.heads * cfg.vdim), dtype=out_dtype, device=q.device)
     scratch = torch.empty((nsplit, T, cfg.heads, cfg.vdim + 2), dtype=torch.float32, device=q.device) if nsplit > 1 else None
     check(lib.ktx_swa_mfma(C.byref(cfg), batch.B, T, int(batch.max_q_len), q.data_ptr(), kcache.data_ptr(), vcache.data_ptr(),
                            batch.q_indptr.data_ptr(), batch.pos0.data_ptr(), batch.page_indptr.data_ptr(), batch.page_indices.data_ptr(),
-                           _ptr(sink), _ptr(dist_bias), _ptr(vcs), int(nsplit), _ptr(scratch), out.data_ptr(), SEQ_DTYPE[out_dtype],
+                           _ptr(sink), _ptr(dist_bias), _ptr(vcs), hg, ldg, int(nsplit), _ptr(scratch), out.data_ptr(), SEQ_DTYPE[out_dtype],
                            _stream_ptr(q.device)))
     return out
 

@@ -708,16 +708,35 @@ __global__ void __launch_bounds__(256) chunk_chain_kernel(ScanDims c, const int3
 // ---------------------------------------------------------------------------------------------------------------------
 // gate / norm segments: a wavefront takes a unit — one norm group of at most GS_WAVE columns, or GS_WAVE columns of an un-normed segment —,
 // wider groups take a workgroup
-constexpr int GS_PER = 8, GS_WAVE = 64 * GS_PER;
+constexpr int GS_PER = 8, GS_WAVE = 64 * GS_PER, GS_WIDE = 2;
 struct GateSegs {
   ktx_gate_seg s[KTX_GATE_SEGS];
+  bool vec[KTX_GATE_SEGS];                 // aligned pieces of eight columns: a lane owns consecutive columns
 };
+// eight columns of a row, 16-byte aligned
+__device__ __forceinline__ void f8_ld(const float* p, float (&v)[8]) {
+  const float4 a = *reinterpret_cast<const float4*>(p), b = *reinterpret_cast<const float4*>(p + 4);
+  v[0] = a.x; v[1] = a.y; v[2] = a.z; v[3] = a.w; v[4] = b.x; v[5] = b.y; v[6] = b.z; v[7] = b.w;
+}
+__device__ __forceinline__ void seg_o8(const ktx_gate_seg& s, int t, int c, float (&v)[8]) {
+  if (s.o_dtype == KTX_SEQ_F32) {
+    f8_ld(reinterpret_cast<const float*>(s.o) + (size_t)t * s.ldo + c, v);
+  } else {
+    const uint4 u = *reinterpret_cast<const uint4*>(reinterpret_cast<const bf16_t*>(s.o) + (size_t)t * s.ldo + c);
+    v[0] = ktx_lo_f32(u.x); v[1] = ktx_hi_f32(u.x); v[2] = ktx_lo_f32(u.y); v[3] = ktx_hi_f32(u.y);
+    v[4] = ktx_lo_f32(u.z); v[5] = ktx_hi_f32(u.z); v[6] = ktx_lo_f32(u.w); v[7] = ktx_hi_f32(u.w);
+  }
+}
+__device__ __forceinline__ void st8(float* p, const float (&v)[8]) {
+  *reinterpret_cast<float4*>(p) = make_float4(v[0], v[1], v[2], v[3]);
+  *reinterpret_cast<float4*>(p + 4) = make_float4(v[4], v[5], v[6], v[7]);
+}
+__device__ __forceinline__ void st8(bf16_t* p, const float (&v)[8]) {
+  *reinterpret_cast<uint4*>(p) = make_uint4(ktx_pk_bf16(v[0], v[1]), ktx_pk_bf16(v[2], v[3]), ktx_pk_bf16(v[4], v[5]), ktx_pk_bf16(v[6], v[7]));
+}
 __device__ __forceinline__ float seg_o(const ktx_gate_seg& s, int t, int c) {
   return s.o_dtype == KTX_SEQ_F32 ? reinterpret_cast<const float*>(s.o)[(size_t)t * s.ldo + c]
                                   : bf16_to_f32(reinterpret_cast<const bf16_t*>(s.o)[(size_t)t * s.ldo + c]);
-}
-__device__ __forceinline__ float seg_gate(const ktx_gate_seg& s, int t, int c) {
-  return s.gate[(size_t)t * s.ldg + (s.gate_div == 1 ? c : c / s.gate_div)];
 }
 __device__ __forceinline__ float seg_act(const ktx_gate_seg& s, float g) { return s.act ? silu_f32(g) : sigmoid_f32(g); }
 
@@ -738,13 +757,28 @@ __global__ void __launch_bounds__(256) gate_segments_kernel(int n_segs, GateSegs
         const int c0 = (u - base) * width, nc = min(width, s.n - c0);
         float p[GS_PER], g[GS_PER], w[GS_PER];
         float ss = 0.f;
+        const bool vec = sg.vec[si];
+        if (vec) {                         // (whole pieces: nc, c0 and w_mod are multiples of 8)
+          const int c = lane * 8;
 #pragma unroll
-        for (int i = 0; i < GS_PER; i++) {
-          const int c = lane + i * 64;
-          const bool ok = c < nc;
-          p[i] = ok ? seg_o(s, t, c0 + c) : 0.f;
-          g[i] = ok ? seg_gate(s, t, c0 + c) : 0.f;
-          w[i] = ok && s.group ? s.w[(c0 + c) % s.w_mod] : 1.f;
+          for (int i = 0; i < GS_PER; i++) {
+            p[i] = g[i] = 0.f;
+            w[i] = 1.f;
+          }
+          if (c < nc) {
+            seg_o8(s, t, c0 + c, p);
+            f8_ld(s.gate + (size_t)t * s.ldg + c0 + c, g);
+            if (s.group) f8_ld(s.w + (c0 + c) % s.w_mod, w);
+          }
+        } else {
+#pragma unroll
+          for (int i = 0; i < GS_PER; i++) {
+            const int c = lane + i * 64;
+            const bool ok = c < nc;
+            p[i] = ok ? seg_o(s, t, c0 + c) : 0.f;
+            g[i] = ok ? s.gate[(size_t)t * s.ldg + c0 + c] : 0.f;
+            w[i] = ok && s.group ? s.w[(c0 + c) % s.w_mod] : 1.f;
+          }
         }
 #pragma unroll
         for (int i = 0; i < GS_PER; i++) {
@@ -753,6 +787,12 @@ __global__ void __launch_bounds__(256) gate_segments_kernel(int n_segs, GateSegs
           ss += p[i] * p[i];
         }
         const float r = s.group ? 1.0f / sqrtf(wave_sum(ss) / (float)s.group + s.eps) : 1.0f;
+        if (vec) {
+#pragma unroll
+          for (int i = 0; i < GS_PER; i++) p[i] = p[i] * r * w[i] * (s.gate_first ? 1.f : g[i]) * s.scale;
+          if (lane * 8 < nc) st8(orow + c0 + lane * 8, p);
+          continue;
+        }
 #pragma unroll
         for (int i = 0; i < GS_PER; i++) {
           const int c = lane + i * 64;
@@ -764,10 +804,44 @@ __global__ void __launch_bounds__(256) gate_segments_kernel(int n_segs, GateSegs
       for (int gI = blockIdx.y; gI < s.n / s.group; gI += gridDim.y) {
         const int c0 = gI * s.group;
         float ss = 0.f;
+        if (sg.vec[si] && s.group <= 8 * 256 * GS_WIDE) {      // a thread's pieces stay in registers, all requested before the first is used
+          float p[GS_WIDE][8], g[GS_WIDE][8], w[8];
+#pragma unroll
+          for (int k = 0; k < GS_WIDE; k++) {
+            const int c = (tid + k * 256) * 8;
+            if (c < s.group) {
+              seg_o8(s, t, c0 + c, p[k]);
+              f8_ld(s.gate + (size_t)t * s.ldg + c0 + c, g[k]);
+            } else {
+#pragma unroll
+              for (int i = 0; i < 8; i++) p[k][i] = g[k][i] = 0.f;
+            }
+          }
+#pragma unroll
+          for (int k = 0; k < GS_WIDE; k++)
+#pragma unroll
+            for (int i = 0; i < 8; i++) {
+              g[k][i] = seg_act(s, g[k][i]);
+              if (s.gate_first) p[k][i] *= g[k][i];
+              ss += p[k][i] * p[k][i];
+            }
+          const float r = 1.0f / sqrtf(block_sum256(ss, red) / (float)s.group + s.eps) * s.scale;
+#pragma unroll
+          for (int k = 0; k < GS_WIDE; k++) {
+            const int c = (tid + k * 256) * 8;
+            if (c < s.group) {
+              f8_ld(s.w + (c0 + c) % s.w_mod, w);
+#pragma unroll
+              for (int i = 0; i < 8; i++) p[k][i] *= r * w[i] * (s.gate_first ? 1.f : g[k][i]);
+              st8(orow + c0 + c, p[k]);
+            }
+          }
+          continue;
+        }
 #pragma unroll 4
         for (int c = tid; c < s.group; c += 256) {
           float p = seg_o(s, t, c0 + c);
-          if (s.gate_first) p *= seg_act(s, seg_gate(s, t, c0 + c));
+          if (s.gate_first) p *= seg_act(s, s.gate[(size_t)t * s.ldg + c0 + c]);
           row[c] = p;
           ss += p * p;
         }
@@ -775,7 +849,7 @@ __global__ void __launch_bounds__(256) gate_segments_kernel(int n_segs, GateSegs
 #pragma unroll 4
         for (int c = tid; c < s.group; c += 256) {      // (each thread re-reads only what it wrote)
           float p = row[c] * r * s.w[(c0 + c) % s.w_mod];
-          if (!s.gate_first) p *= seg_act(s, seg_gate(s, t, c0 + c));
+          if (!s.gate_first) p *= seg_act(s, s.gate[(size_t)t * s.ldg + c0 + c]);
           st_elem(orow, c0 + c, p);
         }
       }
@@ -1003,13 +1077,16 @@ int ktx_gate_segments(int T, int n_segs, const ktx_gate_seg* segs, void* d_out, 
   size_t lds = 0;
   for (int i = 0; i < n_segs; i++) {
     const ktx_gate_seg& s = segs[i];
-    KTX_REQUIRE(s.o && s.gate && s.n > 0 && s.group >= 0 && dtype_ok(s.o_dtype) && s.ldo >= s.n && s.gate_div > 0 && s.ldg >= (s.n + s.gate_div - 1) / s.gate_div && s.out_off >= 0 &&
+    KTX_REQUIRE(s.o && s.gate && s.n > 0 && s.group >= 0 && dtype_ok(s.o_dtype) && s.ldo >= s.n && s.ldg >= s.n && s.out_off >= 0 &&
                     ldout >= s.out_off + s.n && (s.act == 0 || s.act == 1),
                 "ktx_gate_segments: rows that hold the segment, a known activation");
     KTX_REQUIRE(s.group == 0 || (s.n % s.group == 0 && s.w && (s.w_mod == s.group || s.w_mod == s.n)), "ktx_gate_segments: groups divide the columns");
     if (s.group > GS_WAVE) lds = std::max(lds, (size_t)s.group * 4), units += 4 * (s.n / s.group);
     else units += s.group ? s.n / s.group : (s.n + GS_WAVE - 1) / GS_WAVE;
     sg.s[i] = s;
+    const int osz = out_dtype == KTX_SEQ_F32 ? 4 : 2;
+    sg.vec[i] = s.n % 8 == 0 && s.group % 8 == 0 && s.ldo % 8 == 0 && s.ldg % 4 == 0 && ldout % 8 == 0 && s.out_off % 8 == 0 && aligned16(s.o) &&
+                aligned16(s.gate) && (!s.group || aligned16(s.w)) && aligned16(d_out) && ((size_t)ldout * osz) % 16 == 0;
   }
   KTX_REQUIRE(lds <= 150 * 1024, "ktx_gate_segments: a norm group must fit the LDS");
   if (T == 0) return 0;

@@ -428,13 +428,18 @@ __global__ void __launch_bounds__(256) swa_conv_prep_vec_kernel(ktx_swa_config c
 // tiles of KTN <= 64 keys and values staged in LDS as fp32; scores thread = (head, key); running maximum / sum per head by wavefronts;
 // outputs thread = (head, value entry) in registers.
 constexpr int SW_NACC = 32;
+// the factor on a head's result: sigmoid of its gate logit when the heads are gated
+__device__ __forceinline__ float head_gate(const float* __restrict__ hgate, int64_t ldg, int t, int h) {
+  return hgate ? sigmoid_f32(hgate[(size_t)t * ldg + h]) : 1.0f;
+}
 template <typename KT, typename OT>
 __global__ void __launch_bounds__(256) swa_fwd_kernel(ktx_swa_config c, int T, int HG, int parts, int KTN, const float* __restrict__ q,
                                                       const KT* __restrict__ kcache, const KT* __restrict__ vcache,
                                                       const int32_t* __restrict__ tok_req, const int32_t* __restrict__ pos,
                                                       const int32_t* __restrict__ page_indptr, const int32_t* __restrict__ page_indices,
                                                       const float* __restrict__ sink, const float* __restrict__ dist_bias,
-                                                      const float* __restrict__ vcs, int nsplit, float* __restrict__ scratch,
+                                                      const float* __restrict__ vcs, const float* __restrict__ hgate, int64_t ldg, int nsplit,
+                                                      float* __restrict__ scratch,
                                                       OT* __restrict__ out) {
   extern __shared__ float lds[];
   const int D = c.dim, V = c.vdim, DP = D + 1, VP = V + 1, G = c.kv_heads, HPG = c.heads / G;
@@ -543,6 +548,7 @@ __global__ void __launch_bounds__(256) swa_fwd_kernel(ktx_swa_config c, int T, i
         } else {
           o = lrow[h] > 0.f ? acc[i] / lrow[h] : 0.f;
         }
+        o *= head_gate(hgate, ldg, t, h0 + h);
       }
       if (c.rot_values) {      // turn the pair (2m, 2m + 1) back by the token's own angle; the partner sits in the neighbouring thread
         const float other = __shfl_xor(o, 1);
@@ -571,7 +577,7 @@ __global__ void __launch_bounds__(256) swa_fwd_kernel(ktx_swa_config c, int T, i
 template <typename OT>
 __global__ void __launch_bounds__(256) swa_merge_kernel(int T, int H, int V, int nsplit, int rot_values, const float* __restrict__ scratch,
                                                         const float* __restrict__ sink, const float* __restrict__ vcs,
-                                                        OT* __restrict__ out) {
+                                                        const float* __restrict__ hgate, int64_t ldg, OT* __restrict__ out) {
   extern __shared__ float mw[];            // [nsplit] maxima, then [nsplit] weights exp(m_z - M) (0 for an empty range)
   float* ws = mw + nsplit;
   const int t = blockIdx.x, h = blockIdx.y;
@@ -589,7 +595,7 @@ __global__ void __launch_bounds__(256) swa_merge_kernel(int T, int H, int V, int
   __syncthreads();
   for (int z = threadIdx.x; z < nsplit; z += 256) ws[z] = mw[z] == -INFINITY ? 0.f : expf(mw[z] - M);
   __syncthreads();
-  const float inv = den > 0.f ? 1.0f / den : 0.f;
+  const float inv = (den > 0.f ? 1.0f / den : 0.f) * head_gate(hgate, ldg, t, h);
   const int NV = V / 2;
   for (int l0 = 0; l0 < V; l0 += 256) {
     const int l = l0 + threadIdx.x;
@@ -627,7 +633,8 @@ __global__ void __launch_bounds__(256) swa_mfma_kernel(ktx_swa_config c, int T, 
                                                        const int32_t* __restrict__ q_indptr, const int32_t* __restrict__ pos0,
                                                        const int32_t* __restrict__ page_indptr, const int32_t* __restrict__ page_indices,
                                                        const float* __restrict__ sink, const float* __restrict__ dist_bias,
-                                                       const float* __restrict__ vcs, int nsplit, float* __restrict__ scratch,
+                                                       const float* __restrict__ vcs, const float* __restrict__ hgate, int64_t ldg, int nsplit,
+                                                      float* __restrict__ scratch,
                                                        OT* __restrict__ out) {
   constexpr int V = NT * 16;
   extern __shared__ __attribute__((aligned(16))) unsigned char sm_raw[];
@@ -779,6 +786,7 @@ __global__ void __launch_bounds__(256) swa_mfma_kernel(ktx_swa_config c, int T, 
       } else {
         inv = lrun[r] > 0.f ? 1.0f / lrun[r] : 0.f;
       }
+      inv *= head_gate(hgate, ldg, tok, head);
 #pragma unroll
       for (int n = 0; n < NT; n++) {
         float o = acc[n][r] * inv;
@@ -1240,23 +1248,24 @@ int ktx_swa_conv_prep(const ktx_swa_config* cfg, int B, int T, int max_q_len, in
 }
 
 static int swa_merge(const ktx_swa_config* cfg, int T, int nsplit, const float* d_scratch, const float* d_sink, const float* d_vcs,
-                     void* d_out, int out_dtype, hipStream_t st) {
+                     const float* d_head_gate, int64_t ldg, void* d_out, int out_dtype, hipStream_t st) {
   const dim3 mg(T, cfg->heads);
   if (out_dtype == KTX_SEQ_F32)
     swa_merge_kernel<float><<<mg, 256, (size_t)nsplit * 8, st>>>(T, cfg->heads, cfg->vdim, nsplit, cfg->rot_values, d_scratch, d_sink, d_vcs,
-                                                                 (float*)d_out);
+                                                                 d_head_gate, ldg, (float*)d_out);
   else
     swa_merge_kernel<bf16_t><<<mg, 256, (size_t)nsplit * 8, st>>>(T, cfg->heads, cfg->vdim, nsplit, cfg->rot_values, d_scratch, d_sink, d_vcs,
-                                                                  (bf16_t*)d_out);
+                                                                  d_head_gate, ldg, (bf16_t*)d_out);
   KTX_HIP(hipGetLastError());
   return 0;
 }
 
 int ktx_swa_forward(const ktx_swa_config* cfg, int T, const float* d_q, const void* d_kcache, const void* d_vcache,
                     const int32_t* d_tok_req, const int32_t* d_pos, const int32_t* d_page_indptr, const int32_t* d_page_indices,
-                    const float* d_sink, const float* d_dist_bias, const float* d_vcs, int nsplit, float* d_scratch, void* d_out,
-                    int out_dtype, ktx_stream_t stream) {
+                    const float* d_sink, const float* d_dist_bias, const float* d_vcs, const float* d_head_gate, int64_t ldg, int nsplit,
+                    float* d_scratch, void* d_out, int out_dtype, ktx_stream_t stream) {
   if (swa_check(cfg, "ktx_swa_forward")) return -1;
+  KTX_REQUIRE(!d_head_gate || ldg >= cfg->heads, "ktx_swa_forward: a gate per head");
   KTX_REQUIRE(T >= 0 && d_q && d_kcache && d_vcache && d_tok_req && d_pos && d_page_indptr && d_page_indices && d_out && dtype_ok(out_dtype),
               "ktx_swa_forward: null pointer");
   KTX_REQUIRE(!cfg->rot_values || d_vcs, "ktx_swa_forward: rotated values need the table of their angles");
@@ -1281,7 +1290,8 @@ int ktx_swa_forward(const ktx_swa_config* cfg, int T, const float* d_q, const vo
   do {                                                                                                                             \
     KTX_HIP(ktx_set_max_lds((const void*)swa_fwd_kernel<KT, OT>, 150 * 1024));                                                     \
     swa_fwd_kernel<KT, OT><<<grid, 256, lds, st>>>(*cfg, T, HG, parts, KTN, d_q, (const KT*)d_kcache, (const KT*)d_vcache, d_tok_req, \
-                                                   d_pos, d_page_indptr, d_page_indices, d_sink, d_dist_bias, d_vcs, nsplit, d_scratch, (OT*)d_out); \
+                                                   d_pos, d_page_indptr, d_page_indices, d_sink, d_dist_bias, d_vcs, d_head_gate, ldg, nsplit, \
+                                                   d_scratch, (OT*)d_out); \
   } while (0)
   if (cfg->cache_dtype == KTX_SEQ_F32) {
     if (out_dtype == KTX_SEQ_F32) KTX_SW_GO(float, float);
@@ -1292,7 +1302,7 @@ int ktx_swa_forward(const ktx_swa_config* cfg, int T, const float* d_q, const vo
   }
 #undef KTX_SW_GO
   KTX_HIP(hipGetLastError());
-  if (nsplit > 1) return swa_merge(cfg, T, nsplit, d_scratch, d_sink, d_vcs, d_out, out_dtype, st);
+  if (nsplit > 1) return swa_merge(cfg, T, nsplit, d_scratch, d_sink, d_vcs, d_head_gate, ldg, d_out, out_dtype, st);
   return 0;
 }
 
@@ -1306,9 +1316,10 @@ int ktx_swa_mfma_eligible(const ktx_swa_config* c) {
 
 int ktx_swa_mfma(const ktx_swa_config* cfg, int B, int T, int max_q_len, const float* d_q, const void* d_kcache, const void* d_vcache,
                  const int32_t* d_q_indptr, const int32_t* d_pos0, const int32_t* d_page_indptr, const int32_t* d_page_indices,
-                 const float* d_sink, const float* d_dist_bias, const float* d_vcs, int nsplit, float* d_scratch, void* d_out, int out_dtype,
-                 ktx_stream_t stream) {
+                 const float* d_sink, const float* d_dist_bias, const float* d_vcs, const float* d_head_gate, int64_t ldg, int nsplit,
+                 float* d_scratch, void* d_out, int out_dtype, ktx_stream_t stream) {
   if (swa_check(cfg, "ktx_swa_mfma")) return -1;
+  KTX_REQUIRE(!d_head_gate || ldg >= cfg->heads, "ktx_swa_mfma: a gate per head");
   KTX_REQUIRE(ktx_swa_mfma_eligible(cfg), "ktx_swa_mfma: bf16 caches, dim a multiple of 8 up to 256, vdim a multiple of 16 up to 128, or 256");
   KTX_REQUIRE(B >= 0 && T >= 0 && max_q_len >= 0 && d_q && d_kcache && d_vcache && d_q_indptr && d_pos0 && d_page_indptr &&
                   d_page_indices && d_out && dtype_ok(out_dtype),
@@ -1328,8 +1339,8 @@ int ktx_swa_mfma(const ktx_swa_config* cfg, int B, int T, int max_q_len, const f
   do {                                                                                                                                \
     KTX_HIP(ktx_set_max_lds((const void*)swa_mfma_kernel<NT, OT>, 150 * 1024));                                                       \
     swa_mfma_kernel<NT, OT><<<grid, 256, lds, st>>>(*cfg, T, row_tiles, d_q, (const bf16_t*)d_kcache, (const bf16_t*)d_vcache,        \
-                                                    d_q_indptr, d_pos0, d_page_indptr, d_page_indices, d_sink, d_dist_bias, d_vcs, nsplit, d_scratch, \
-                                                    (OT*)d_out);                                                                      \
+                                                    d_q_indptr, d_pos0, d_page_indptr, d_page_indices, d_sink, d_dist_bias, d_vcs, d_head_gate, ldg, \
+                                                    nsplit, d_scratch, (OT*)d_out);                                                                      \
   } while (0)
 #define KTX_SM_NT(OT)                  \
   do {                                 \
@@ -1348,7 +1359,7 @@ int ktx_swa_mfma(const ktx_swa_config* cfg, int B, int T, int max_q_len, const f
 #undef KTX_SM_NT
 #undef KTX_SM_GO
   KTX_HIP(hipGetLastError());
-  if (nsplit > 1) return swa_merge(cfg, T, nsplit, d_scratch, d_sink, d_vcs, d_out, out_dtype, st);
+  if (nsplit > 1) return swa_merge(cfg, T, nsplit, d_scratch, d_sink, d_vcs, d_head_gate, ldg, d_out, out_dtype, st);
   return 0;
 }
 

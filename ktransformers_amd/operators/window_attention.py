@@ -27,7 +27,7 @@ Further options, each off unless the replaced module names it:
     sink = "learned"      the sink's score is `<key>.sink` [heads];
     softcap               the scaled score becomes softcap tanh(score / softcap);
     gated                 the concatenated heads are multiplied by sigmoid(W_g h) (`<key>.g`) in front of W_o (include/ktx_gla.h `ktx_gate_segments`);
-                          "per_head": one gate per head (`<key>.g` [heads, width]);
+                          "per_head": one gate per head (`<key>.g` [heads, width]), multiplied in by the attention's own launch;
     rot_scaling           YaRN scaling of the rotation (operators/RoPE.py `turning_frequencies`);
     kv_from = j           the layer has no key and value projections and reads the rows that the layer with cache index j appended in the same step
                           (equal kv_heads, sizes and rotation), with its own queries, window and scale.
@@ -161,18 +161,24 @@ class KWindowGQAttention(BaseInjectedModule):
             return dense_gemm(self.attend(dense_gemm(h, self.w["qkv"]), batch, cache, cache_idx), self.w["o"])
         if "in" not in self.w:
             self.w["in"] = padded_rows([self.w["qkv"], self.w["g"]])
+        if self.gated == "per_head":
+            proj, n = dense_gemm(h, self.w["in"]), self.w["qkv"].shape[0]
+            return dense_gemm(self.attend(proj, batch, cache, cache_idx, head_gate=proj[:, n:n + self.heads]), self.w["o"])
         seg = self.gated_segment(dense_gemm(h, self.w["in"]), 0, batch, cache, cache_idx)
         return dense_gemm(gate_segments([seg], h.shape[0], h.device, out_dtype=self.compute_dtype), self.w["o"])
 
     def gated_segment(self, proj: torch.Tensor, base: int, batch, cache, cache_idx: int, scale: float = 1.0):
         """proj fp32 rows with q | k | v | g from column `base`: the attention, and the segment of gate_segments that gates its heads."""
         from ktransformers_amd._native_gla import gate_seg
+        if self.gated == "per_head":
+            raise NotImplementedError(f"{self.key}: heads gated by one number each are gated inside the attention")
         (_, n_qkv), (_, n_g) = self.in_weight_names()
         o = self.attend(proj[:, base:base + n_qkv], batch, cache, cache_idx)
-        return gate_seg(o, proj[:, base + n_qkv:base + n_qkv + n_g], "sigmoid", scale=scale, gate_div=self.vdim if self.gated == "per_head" else 1)
+        return gate_seg(o, proj[:, base + n_qkv:base + n_qkv + n_g], "sigmoid", scale=scale)
 
-    def attend(self, proj: torch.Tensor, batch, cache, cache_idx: int) -> torch.Tensor:
-        """proj fp32 rows with q | k | v at column 0 -> the concatenated heads [T, heads * vdim] in the compute type (no gate, no W_o)."""
+    def attend(self, proj: torch.Tensor, batch, cache, cache_idx: int, head_gate: torch.Tensor | None = None) -> torch.Tensor:
+        """proj fp32 rows with q | k | v at column 0 -> the concatenated heads [T, heads * vdim] in the compute type (no W_o; no gate but the
+        heads' own, logits [T, heads])."""
         from ktransformers_amd._native_swa import swa_conv_prep, swa_forward, swa_mfma, swa_mfma_eligible, swa_prep
         H, G, D = self.heads, self.kv_heads, self.dim
         cfg, T = self._config(cache), proj.shape[0]
@@ -192,9 +198,11 @@ class KWindowGQAttention(BaseInjectedModule):
         if self.USE_MATRIX_CORES and kc.dtype == torch.bfloat16 and swa_mfma_eligible(cfg):
             blocks = batch.B * G * ((batch.max_q_len * (H // G) + 63) // 64)
             nsplit = max(1, min(self.TARGET_WORKGROUPS // max(blocks, 1), (span + self.KEYS_PER_SPLIT - 1) // self.KEYS_PER_SPLIT))
-            o = swa_mfma(cfg, q, kc, vc, batch, self.w["sink"], vcs, nsplit=nsplit, out_dtype=self.compute_dtype, dist_bias=bias)
+            o = swa_mfma(cfg, q, kc, vc, batch, self.w["sink"], vcs, nsplit=nsplit, out_dtype=self.compute_dtype, dist_bias=bias,
+                         head_gate=head_gate)
         else:
             span = batch.max_kv_len if not self.window else min(batch.max_kv_len, self.window + self.keep_first)
             nsplit = max(1, min(self.TARGET_WORKGROUPS // max(T * G, 1), (span + self.KEYS_PER_SPLIT - 1) // self.KEYS_PER_SPLIT))
-            o = swa_forward(cfg, q, kc, vc, batch, self.w["sink"], vcs, nsplit=nsplit, out_dtype=self.compute_dtype, dist_bias=bias)
+            o = swa_forward(cfg, q, kc, vc, batch, self.w["sink"], vcs, nsplit=nsplit, out_dtype=self.compute_dtype, dist_bias=bias,
+                            head_gate=head_gate)
         return o

@@ -287,7 +287,7 @@ def test_latent_preps_scaled_half_rotation_and_the_query_latent(rot, dtype):
 
 
 # ---- attention kernels --------------------------------------------------------------------------------------------------------------------
-def run_attention(q, k, v, scale, window, dtype, kernel, nsplit=1, page_size=8, t_new=None):
+def run_attention(q, k, v, scale, window, dtype, kernel, nsplit=1, page_size=8, t_new=None, head_gate=None):
     """The attention kernels on keys and values written straight into paged caches; the last t_new positions are the queries."""
     from ktransformers_amd._native_swa import swa_config, swa_forward, swa_mfma, swa_mfma_eligible
     from ktransformers_amd.models.custom_cache import KHybridCache
@@ -307,7 +307,7 @@ def run_attention(q, k, v, scale, window, dtype, kernel, nsplit=1, page_size=8, 
     qn = f32d((q * scale)[T - t_new:].reshape(t_new, H * D))
     assert kernel != "mfma" or swa_mfma_eligible(cfg)
     fn = swa_mfma if kernel == "mfma" else swa_forward
-    return fn(cfg, qn, cache.k_caches[0], cache.v_caches[0], b, None, None, nsplit=nsplit, out_dtype=F32).view(t_new, H, V)
+    return fn(cfg, qn, cache.k_caches[0], cache.v_caches[0], b, None, None, nsplit=nsplit, out_dtype=F32, head_gate=head_gate).view(t_new, H, V)
 
 
 @pytest.mark.parametrize("kernel,dtype", [("valu", F32), ("valu", BF16), ("mfma", BF16)])
@@ -419,23 +419,42 @@ def test_lightning_scan_remembers_one_far_token():
 
 
 # ---- gates --------------------------------------------------------------------------------------------------------------------------------
+@pytest.mark.parametrize("kernel,dtype", [("valu", F32), ("valu", BF16), ("mfma", BF16)])
+@pytest.mark.parametrize("nsplit", [1, 3])
+def test_one_gate_per_head_inside_the_attention(kernel, dtype, nsplit):
+    H, G, D, V, T, window = 6, 2, 40, 48, 70, 21
+    g = torch.Generator().manual_seed(3)
+    q, k, v = (torch.randn(T, n, d, generator=g).to(dtype).double() for n, d in ((H, D), (G, D), (G, V)))
+    gate = torch.randn(T, H + 7, generator=g) * 3               # (a column slice: strided rows)
+    want = R.softmax_attention(q, k, v, 0.125, window) * torch.sigmoid(gate[:, 4:4 + H].double()).view(T, H, 1)
+    for t_new in (T, 1, 2):
+        got = run_attention(q, k, v, 0.125, window, dtype, kernel, nsplit=nsplit, t_new=t_new, head_gate=f32d(gate[T - t_new:])[:, 4:4 + H])
+        assert rel(got, want[T - t_new:]) < (2e-5 if kernel == "valu" else 1.5e-2), t_new
+    for i in (0, T - 1):                                        # a gate that is shut is that token's and that head's alone
+        shut = torch.zeros(T, H)
+        shut[i, 4] = -200.0
+        got = run_attention(q, k, v, 0.125, window, dtype, kernel, nsplit=nsplit, head_gate=f32d(shut)).cpu()
+        assert float(got[i, 4].abs().max()) == 0.0 and int((got.abs().amax(dim=2) == 0).sum()) == 1
+
+
 @pytest.mark.parametrize("dtype", [F32, BF16])
 @pytest.mark.parametrize("T", [1, 3, 70])
-def test_one_gate_per_head_and_a_norm_over_all_heads(dtype, T):
+def test_gate_and_norm_over_all_heads(dtype, T):
+    """Norm groups as wide as all heads together: aligned pieces held in registers, rows in LDS beyond that, odd sizes, strided gates."""
     from ktransformers_amd._native_gla import gate_seg, gate_segments
     g = torch.Generator().manual_seed(T)
     tol = 2e-6 if dtype == F32 else 4e-3
-    for H, V, odt in ((4, 24, BF16), (3, 7, F32), (16, 128, BF16), (1, 5, F32), (6, 1, F32), (9, 130, F32)):
-        o, gate, w = torch.randn(T, H * V, generator=g).to(odt), torch.randn(T, H * V + 9, generator=g), torch.randn(H * V, generator=g)
-        od, gd = o.to(DEV), f32d(gate)
-        got = gate_segments([gate_seg(od, gd[:, 4:4 + H], "sigmoid", gate_div=V)], T, DEV, out_dtype=dtype)
-        want = o.double().view(T, H, V) * torch.sigmoid(gate[:, 4:4 + H].double()).view(T, H, 1)
-        assert got.dtype == dtype and rel(got.view(T, H, V), want) < tol, (H, V)
-        got = gate_segments([gate_seg(od, gd[:, 4:4 + H * V], "sigmoid", norm=(f32d(w), H * V, 1e-2))], T, DEV, out_dtype=dtype)
-        assert rel(got, R.rms_norm(o.double(), w.double(), 1e-2) * torch.sigmoid(gate[:, 4:4 + H * V].double())) < tol, (H, V)
-        got = gate_segments([gate_seg(od, gd[:, 4:4 + H], "silu", norm=(f32d(w), H * V, 1e-2), gate_first=True, gate_div=V)], T, DEV, out_dtype=dtype)
-        z = o.double().view(T, H, V) * R.silu(gate[:, 4:4 + H].double()).view(T, H, 1)
-        assert rel(got, R.rms_norm(z.reshape(T, -1), w.double(), 1e-2)) < tol, (H, V)
+    for n, odt in ((96, BF16), (21, F32), (2048, F32), (2048, BF16), (5, F32), (1170, F32), (1168, F32), (4096, F32), (4104, BF16), (512, F32), (520, BF16)):
+        for off in (4, 3):
+            o, gate, w = torch.randn(T, n, generator=g).to(odt), torch.randn(T, n + 8, generator=g), torch.randn(n, generator=g)
+            od, gd = o.to(DEV), f32d(gate)[:, off:off + n]
+            z = gate[:, off:off + n].double()
+            got = gate_segments([gate_seg(od, gd, "sigmoid", norm=(f32d(w), n, 1e-2))], T, DEV, out_dtype=dtype)
+            assert got.dtype == dtype and rel(got, R.rms_norm(o.double(), w.double(), 1e-2) * torch.sigmoid(z)) < tol, (n, off)
+            got = gate_segments([gate_seg(od, gd, "silu", norm=(f32d(w), n, 1e-2), gate_first=True, scale=0.7)], T, DEV, out_dtype=dtype)
+            assert rel(got, 0.7 * R.rms_norm(o.double() * R.silu(z), w.double(), 1e-2)) < tol, (n, off)
+            got = gate_segments([gate_seg(od, gd, "sigmoid")], T, DEV, out_dtype=dtype)
+            assert rel(got, o.double() * torch.sigmoid(z)) < tol, (n, off)
 
 
 # ---- mixers and feed-forwards alone ---------------------------------------------------------------------------------------------------
