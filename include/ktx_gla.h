@@ -1,6 +1,7 @@
 /* ktx_gla.h — C ABI of the kernels (libktx_hip.so / libktx_seq.so) for decoders whose residual is several parallel streams mixed by
  * learned weights around every sublayer (hyper-connections) and whose layers carry a matrix state per head that decays and takes in
- * outer products: gated linear attention (a decay per key channel, from a low-rank projection) and the state-space-dual scan of Mamba-2
+ * outer products: gated linear attention (a decay per key channel, from a low-rank projection), lightning attention (a constant decay per
+ * head, silu on queries, keys and values) and the state-space-dual scan of Mamba-2
  * (one decay per head, keys and queries shared by the heads of a group, behind a short causal convolution).  Plus the output stage such
  * mixers share: heads gated and RMS-normed in either order, the results of several mixers laid side by side for one output product.
  *

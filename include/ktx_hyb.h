@@ -1,7 +1,7 @@
 /* ktx_hyb.h — C ABI of the hybrid-decoder kernels (libktx_hip.so / libktx_seq.so): what a decoder needs whose layers alternate a
  * gated delta-rule recurrence (short causal convolutions in front, state slots behind) with a sliding-window softmax attention over a
  * paged LATENT cache (normed latent + one rotated key part per token, a per-head sink in the denominator), under layer norms with
- * bias, a sigmoid-gated post-normed residual, a PolyNorm feed-forward and a sigmoid-routed mixture of GLU experts.
+ * bias or RMS norms, a (sigmoid-gated) post-normed residual, a PolyNorm or GLU feed-forward and a routed mixture of GLU experts.
  *
  * Batching contract: that of ktx_seq.h — the T tokens of all scheduled requests are flattened, request b owns rows
  * q_indptr[b] .. q_indptr[b+1]; a token knows its request, its position and the cache row of its key.  The residual stream, norms,

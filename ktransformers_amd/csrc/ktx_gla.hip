@@ -1,6 +1,6 @@
 // ktx_gla.hip — kernels behind include/ktx_gla.h: the hyper-connection step (residual streams mixed around a sublayer, read and layer-
 // normed for the next one in the same launch), the low-rank decay of gated linear attention, the convolved inputs, steps and decays of
-// the state-space-dual scan, the decayed outer-product scan both recurrences share (chunks of a prompt run side by side), and the gate /
+// the state-space-dual scan, the decayed outer-product scan the recurrences share (chunks of a prompt run side by side; silu on the way in for lightning attention), and the gate /
 // norm segments in front of an output product.
 //
 // Streams, norms, decays, steps and the state are fp32; element types only select how activations are stored.
